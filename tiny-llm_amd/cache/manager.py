@@ -10,7 +10,8 @@ never run out and frees everything when the whole batch is done
   layer has its own tensors, the ones its CacheSpec describes (keys and values
   [blocks, kv_heads, block_size, head_dim] for attention), indexed by those ids.
 * A "window" group gives a request's blocks back as soon as every position in them
-  is more than `window` behind the next query; a "full" group when the request ends.
+  is more than `window` behind the next query (blocks with one of the request's first `keep`
+  positions stay); a "full" group when the request ends.
 * Blocks that are given back are used again by later growth, most recently freed first.
 * `grow` is all-or-nothing over all groups, so a step that cannot be held changes nothing.
 * Every group has a pool of its own size: a window group never holds more of a request than
@@ -82,12 +83,13 @@ def blocks_held_at_most(spec: CacheSpec, block_size: int, total_len: int, portio
     """The most blocks a request of `total_len` tokens holds in a group at any time when it is
     fed in portions of at most `portion` tokens.  A full group keeps every position.  A window
     group keeps, while a portion runs, the window behind its first token and the portion itself:
-    at most window - 1 + portion positions, which may start anywhere in a block."""
+    at most window - 1 + portion positions, which may start anywhere in a block; and the blocks of the
+    first `keep` positions."""
     whole = -(-max(0, int(total_len)) // block_size)
     if spec.kind != "window" or spec.window <= 0:
         return whole
     span = spec.window - 1 + max(1, int(portion))
-    return min(whole, (span + block_size - 2) // block_size + 1)
+    return min(whole, (span + block_size - 2) // block_size + 1 + -(-spec.keep // block_size))
 
 
 class CacheManager:
@@ -320,10 +322,11 @@ class CacheManager:
         rc.num_tokens = new_len
         for gi, g in enumerate(self.groups):
             first = self._first_needed_block(g, new_len)
-            gone = [b for b in rc.blocks[gi][:first] if b != RELEASED]
+            kept = -(-g.spec.keep // self.block_size)       # blocks of the first positions, which a window may keep
+            gone = [b for b in rc.blocks[gi][kept:first] if b != RELEASED]
             if gone:
                 g.pool.free(gone)
-                for i in range(first):
+                for i in range(kept, first):
                     rc.blocks[gi][i] = RELEASED
 
     def free_request(self, req_id) -> None:

@@ -30,6 +30,28 @@ __device__ __forceinline__ int first_visible_key(int pos, int window) {
   return 0;
 }
 
+// Which keys a row at position `pos` sees, and what happens to their scores: the keys from first_visible_key up to its
+// own, and, of the ones in front of those, the request's first `keep` (tokens a sliding window keeps for good);
+// cap > 0: a score s (scale applied) becomes cap * tanh(s / cap).
+struct KeyMask {
+  int window;
+  int keep;
+  float cap;
+};
+__device__ __forceinline__ bool key_visible(int j, int pos, int row_lo, int keep) {
+  return j <= pos && (j >= row_lo || j < keep);
+}
+// How many of the 64-key tiles in front of `first_tile` (the first tile the windows reach into) hold kept keys: these
+// are tiles 0, 1, ...; a kernel walks them and then goes on at first_tile.
+__device__ __forceinline__ int kept_key_tiles(int keep, int first_tile) { return min((keep + 63) / 64, first_tile); }
+
+// cap * tanh(s * scale / cap) in units of log2 e, for c_in = 2 log2(e) scale / cap and c_out = cap log2(e):
+// tanh(x) = 1 - 2 / (1 + exp(2 x)).  The error is that of the two hardware functions, some 1e-7 * cap whatever s is.
+__device__ __forceinline__ float capped_score(float s, float c_in, float c_out) {
+  const float e = __builtin_amdgcn_exp2f(s * c_in);
+  return c_out * __builtin_fmaf(-2.f, __builtin_amdgcn_rcpf(1.f + e), 1.f);
+}
+
 // The `sink` argument of every entry point and kernel here is a set of flags: bit 0, the softmax's denominator has
 // one more term (the sink); bit 1 (the general kernel and the bfloat16 kernels), the result leaves as float32
 // whatever the type of queries and cache (`out` then points to floats, out_stride counts floats): for a caller
@@ -50,13 +72,13 @@ __global__ __launch_bounds__(TL_WAVE) void paged_attention_kernel(
     const T* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ req_of_token, const int32_t* __restrict__ positions,
     T* __restrict__ out, int64_t out_stride, int nq, int nkv, int hd, int block_size, float scale,
-    int window, int sink) {
+    KeyMask mask, int sink) {
   __shared__ float qs[kMaxHd];
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int r = req_of_token[t];
   const int pos = positions[t];
   const int kv_end = pos + 1;
-  const int kv_begin = first_visible_key(pos, window);
+  const int kv_begin = first_visible_key(pos, mask.window);
   const int kvh = h / (nq / nkv);
   const int32_t* bt = block_tables + (int64_t)r * max_blocks;
 
@@ -69,9 +91,12 @@ __global__ __launch_bounds__(TL_WAVE) void paged_attention_kernel(
 #pragma unroll
   for (int i = 0; i < kDPL; ++i) o[i] = 0.f;
 
-  for (int base = kv_begin; base < kv_end; base += TL_WAVE) {
+  // the kept first keys (those the window does not reach anyway), then the window's
+  const int kept_end = min(mask.keep, kv_begin);
+  for (int base = kept_end > 0 ? 0 : kv_begin; base < kv_end;) {
+    const int end = base < kept_end ? kept_end : kv_end;
     const int j = base + lane;
-    const bool valid = j < kv_end;
+    const bool valid = j < end;
     float s = -INFINITY;
     int64_t row_off = 0;  // element offset of key/value row j in its cache
     if (valid) {
@@ -81,6 +106,7 @@ __global__ __launch_bounds__(TL_WAVE) void paged_attention_kernel(
       float dot = 0.f;
       for (int d = 0; d < hd; ++d) dot = fmaf(qs[d], to_f32(kp[d]), dot);
       s = dot * scale;
+      if (mask.cap > 0.f) s = mask.cap * tanhf(s / mask.cap);
     }
     const float m_new = fmaxf(m, wave_max(s));  // lane 0 of every tile is valid, so m_new is finite
     const float p = valid ? expf(s - m_new) : 0.f;
@@ -88,7 +114,7 @@ __global__ __launch_bounds__(TL_WAVE) void paged_attention_kernel(
     l = l * alpha + wave_sum(p);
 #pragma unroll
     for (int i = 0; i < kDPL; ++i) o[i] *= alpha;
-    const int n_keys = min(TL_WAVE, kv_end - base);
+    const int n_keys = min(TL_WAVE, end - base);
     const int lo = (int)(row_off & 0xffffffff), hi = (int)(row_off >> 32);
     for (int jj = 0; jj < n_keys; ++jj) {
       const float pj = __shfl(p, jj, TL_WAVE);
@@ -101,6 +127,8 @@ __global__ __launch_bounds__(TL_WAVE) void paged_attention_kernel(
       }
     }
     m = m_new;
+    base += TL_WAVE;
+    if (end == kept_end && base >= kept_end) base = kv_begin;
   }
   // a sink: one more term in the denominator, exp(0 - m) in the scores' own scale, that carries no value
   if (sink & kFlagSink) l += expf(-m);
@@ -199,14 +227,14 @@ __device__ __forceinline__ bf16x8 rotate_chunk_regs(const bf16x8 x, const bf16x8
   return r;
 }
 
-template <int HDT, int WAVES>
+template <int HDT, int WAVES, bool CAP>
 __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
     const bf16_t* __restrict__ q, int64_t q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
     const int32_t* __restrict__ tile_ntok, const int32_t* __restrict__ positions, bf16_t* __restrict__ out,
     int64_t out_stride, float* __restrict__ part_o, float* __restrict__ part_ml, int nq, int nkv,
-    int block_size, float scale, int window, int sink, int n_splits, int n_tokens, const FusedRope fused) {
+    int block_size, float scale, KeyMask mask, int sink, int n_splits, int n_tokens, const FusedRope fused) {
   constexpr int HD = HDT * 16;
   constexpr int KS = (HD + 31) / 32;       // k-steps of the score product
   constexpr int VS = HD + FA_VPAD;         // row stride of a wave's V tile in LDS
@@ -259,18 +287,21 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
       if (do_rope) qy[ks] = *(const bf16x8*)(qrow + dp);      // uniform
     }
   }
-  const int row_lo = first_visible_key(pos, window);
+  const int row_lo = first_visible_key(pos, mask.window);
 
   // key range of the tile: union over its rows
   const int hi = row_max_i32(pos), lo = row_min_i32(row_valid ? row_lo : 0x7fffffff);
   const int kv_end = hi + 1, kv_begin = lo;
   const int first_tile = kv_begin / FA_KT, last_tile = (kv_end + FA_KT - 1) / FA_KT;
-  // Key tiles are dealt out in turn: tile (it0 + it) * stride + split * WAVES + wave belongs to
+  // Key tiles are dealt out in turn: number (it0 + it) * stride + split * WAVES + wave belongs to
   // iteration `it` of this wave.  Which tiles a wave gets then does not depend on the positions,
   // so the page of its first tile can be looked up before the positions have arrived.
+  // With kept first keys the numbers count the n_kept tiles of those, then the window's: number n is tile n,
+  // or n + skip from n_kept on (without them skip is 0 and number and tile are one).
   const int stride = WAVES * n_splits, mine = split * WAVES + wave;
-  const int it0 = first_tile / stride;
-  const int iters = (last_tile - mine + stride - 1) / stride - it0;      // may be <= 0: no tile
+  const int n_kept = kept_key_tiles(mask.keep, first_tile), skip = mask.keep > 0 ? first_tile - n_kept : 0;
+  const int it0 = mask.keep > 0 ? 0 : first_tile / stride;
+  const int iters = (last_tile - skip - mine + stride - 1) / stride - it0;      // may be <= 0: no tile
   // fused mode: the one new token of the tile, at position kv_end - 1
   const int new_pos = kv_end - 1;
   // (a tile without a valid row has new_pos -1: it reads the angles of position 0 and uses nothing)
@@ -278,12 +309,14 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   const float* sn = do_rope ? fused.sin_t + (int64_t)max(new_pos, 0) * (HD / 2) : nullptr;
 
   const int new_tile = new_pos / FA_KT;
-  const bool owns_new = do_rope && new_tile % (WAVES * n_splits) == split * WAVES + wave;
+  const bool owns_new = do_rope && (new_tile - skip) % (WAVES * n_splits) == split * WAVES + wave;
   float m_run = kNegBig, l_run = 0.f;
   f32x4 o[HDT];
 #pragma unroll
   for (int dt = 0; dt < HDT; ++dt) o[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
-  const float c_log2 = scale * 1.44269504088896341f;     // scores are kept in units of log2 e
+  // scores are kept in units of log2 e (CAP: the cap leaves them so)
+  const float c_log2 = CAP ? 1.f : scale * 1.44269504088896341f;
+  const float cap_in = CAP ? scale * 2.88539008177792681f / mask.cap : 0.f, cap_out = mask.cap * 1.44269504088896341f;
 
   // A wave reads its 64-key tile by itself, so nothing in this loop waits for another wave.  Keys
   // go straight from memory into MFMA operands (lane (r16, g) holds dims ks*32 + g*8.. of key rows
@@ -315,7 +348,11 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   // so that a load instruction covers 1 KB of consecutive rows): with a row per lane an instruction
   // touched 64 cache lines for 16 bytes each, and looking those up was what a round of tiles cost.
   const bf16_t* finite_row = q + (int64_t)tok0 * q_stride + (int64_t)kvh * G * HD;
-  auto tile_base = [&](int it) { return ((it0 + it) * stride + mine) * FA_KT; };
+  auto tile_at = [&](int it) {
+    const int n = (it0 + it) * stride + mine;
+    return n >= n_kept ? n + skip : n;
+  };
+  auto tile_base = [&](int it) { return tile_at(it) * FA_KT; };
   auto fetch = [&](int it, int pages_raw) {
     const int base = tile_base(it);
     const int pages = max(pages_raw, 0);
@@ -323,7 +360,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
 #pragma unroll
     for (int kt = 0; kt < 4; ++kt) {
       const int row = kt * 16 + r16, j = base + row;
-      const bool k_in = j >= kv_begin && j < kv_end;
+      const bool k_in = (j >= kv_begin || j < mask.keep) && j < kv_end;
       const int64_t off = row_offset(j, __shfl(pages, row, TL_WAVE));
       kp[kt] = k_cache + (k_in ? off : 0);
     }
@@ -334,7 +371,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
 #pragma unroll
     for (int c = 0; c < VCH; ++c) {
       const int f = c * TL_WAVE + lane, row = f / VCH, ch = f % VCH, j = base + row;
-      const bool v_in = j >= kv_begin && j < kv_end;
+      const bool v_in = (j >= kv_begin || j < mask.keep) && j < kv_end;
       const int64_t off = row_offset(j, __shfl(pages, row, TL_WAVE));
       const bf16_t* vp = v_in ? v_cache + off : finite_row;
       if (do_rope && j == new_pos) vp = new_v;      // not in the cache yet
@@ -346,7 +383,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   // (Two tiles in flight per wave, in two register sets, were measured to gain nothing: what a
   // compute unit can have on its way from memory is the limit, about 40 GB/s.)
   if (iters > 0) {
-    if (it0 != 0) next_pages = pages_at(tile_base(0));
+    if (it0 != 0 || mask.keep > 0) next_pages = pages_at(tile_base(0));
     fetch(0, next_pages);
     if (iters > 1) next_pages = pages_at(tile_base(1));
   }
@@ -401,7 +438,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   }
 
   for (int it = 0; it < iters; ++it) {
-    const int kt_idx = (it0 + it) * stride + mine;
+    const int kt_idx = tile_at(it);
     if (do_rope && kt_idx == new_tile) {
       // the new token's own key (rotated above) takes the place of what its cache row held, and its
       // value, fetched from the qkv row instead of the cache, is written to the cache
@@ -449,7 +486,8 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int j = kt_idx * FA_KT + kt * 16 + g * 4 + r;
-          const bool ok = row_valid && j <= pos && j >= row_lo;
+          const bool ok = row_valid && key_visible(j, pos, row_lo, mask.keep);
+          if constexpr (CAP) sc[kt][r] = capped_score(sc[kt][r], cap_in, cap_out);
           const float sv = ok ? sc[kt][r] : -INFINITY;
           sc[kt][r] = sv;
           m_tile = fmaxf(m_tile, sv);
@@ -598,8 +636,8 @@ template <int HDT>
 __device__ __forceinline__ void attention_f32_tile(int kb, const int32_t* __restrict__ bt, int max_blocks, int block_size,
                                                    int nkv, int kvh, const float* __restrict__ k_cache,
                                                    const float* __restrict__ v_cache, const float* __restrict__ finite_row,
-                                                   const f32x4 (&qf)[HDT], float c_log2, bool row_valid, int pos, int row_lo,
-                                                   int kv_begin, int kv_end, float* Vl, float& m_t, float& l_t,
+                                                   const f32x4 (&qf)[HDT], float scale, const KeyMask& mask, bool row_valid,
+                                                   int pos, int row_lo, int kv_begin, int kv_end, float* Vl, float& m_t, float& l_t,
                                                    f32x4 (&o)[HDT]) {
   constexpr int HD = HDT * 16;
   const int lane = threadIdx.x % TL_WAVE, l16 = lane % 16, kk = lane / 16;
@@ -613,7 +651,7 @@ __device__ __forceinline__ void attention_f32_tile(int kb, const int32_t* __rest
   // for the rows where the select stands.
   constexpr int VPRE = (HD < A32_VW ? HD : A32_VW) / 4;
   const int vkey = kb + lane;
-  const bool v_in_range = vkey >= kv_begin && vkey < kv_end;
+  const bool v_in_range = (vkey >= kv_begin || vkey < mask.keep) && vkey < kv_end;
   bool k_in[4];
   int page_k[4];
 #pragma unroll
@@ -655,14 +693,23 @@ __device__ __forceinline__ void attention_f32_tile(int kb, const int32_t* __rest
       sc[s0 + si] = acc;
     }
   }
-  // ---- the tile's softmax from scratch
+  // ---- the tile's softmax from scratch (scores in units of log2 e)
+  float c_log2 = scale * 1.44269504088896341f;
+  if (mask.cap > 0.f) {
+    const float c_in = scale / mask.cap;
+#pragma unroll
+    for (int st = 0; st < 4; ++st)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) sc[st][r] = tanhf(sc[st][r] * c_in);
+    c_log2 = mask.cap * 1.44269504088896341f;
+  }
   m_t = -INFINITY;
 #pragma unroll
   for (int st = 0; st < 4; ++st)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int key = kb + st * 16 + kk * 4 + r;
-      const bool vis = row_valid && key <= pos && key >= row_lo;
+      const bool vis = row_valid && key_visible(key, pos, row_lo, mask.keep);
       sc[st][r] = vis ? sc[st][r] * c_log2 : -INFINITY;
       m_t = fmaxf(m_t, sc[st][r]);
     }
@@ -727,7 +774,7 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_kernel(
     const float* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
     const int32_t* __restrict__ tile_ntok, const int32_t* __restrict__ positions, float* __restrict__ out,
-    int64_t out_stride, float* __restrict__ part, int nq, int nkv, int block_size, float scale, int window, int sink,
+    int64_t out_stride, float* __restrict__ part, int nq, int nkv, int block_size, float scale, KeyMask mask, int sink,
     int n_tokens) {
   constexpr int HD = HDT * 16;
   constexpr int PS = HD + 4;                       // row stride of a tile's O in LDS
@@ -752,11 +799,13 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_kernel(
   const bool row_valid = tok_local < TW && tok_local < ntok;
   const int tok = tok0 + (row_valid ? tok_local : 0);
   const int pos = row_valid ? positions[tok] : -1;
-  const int row_lo = first_visible_key(pos, window);
+  const int row_lo = first_visible_key(pos, mask.window);
   const int hi = row_max_i32(pos), lo = row_min_i32(row_valid ? row_lo : 0x7fffffff);
   const int kv_end = hi + 1, kv_begin = lo;
   const int first_tile = kv_begin / FA_KT, last_tile = (kv_end + FA_KT - 1) / FA_KT;
-  const int c_first = gridDim.z > 1 ? (int)blockIdx.z : first_tile / A32_CHUNK;
+  // the tiles of kept first keys (0 .. n_kept - 1) lie in front; chunks between them and the window are left out
+  const int n_kept = kept_key_tiles(mask.keep, first_tile);
+  const int c_first = gridDim.z > 1 ? (int)blockIdx.z : n_kept ? 0 : first_tile / A32_CHUNK;
   const int c_last = gridDim.z > 1 ? (int)blockIdx.z + 1 : (last_tile + A32_CHUNK - 1) / A32_CHUNK;
 
   f32x4 qf[HDT];
@@ -766,7 +815,6 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_kernel(
     for (int g4 = 0; g4 < HDT; ++g4)
       qf[g4] = row_valid ? *(const f32x4*)(qrow + g4 * 16 + kk * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
   }
-  const float c_log2 = scale * 1.44269504088896341f;
 
   // the elements this thread merges: e = tid + 256 u -> (row e / HD, dim e % HD)
   float Mrun[EPT], Lrun[EPT], Orun[EPT];
@@ -778,13 +826,15 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_kernel(
   }
 
   for (int c = c_first; c < c_last; ++c) {
-    const int t_lo = max(c * A32_CHUNK, first_tile), t_hi = min((c + 1) * A32_CHUNK, last_tile);
+    if ((c + 1) * A32_CHUNK <= first_tile && c * A32_CHUNK >= n_kept) continue;      // (the whole workgroup)
+    const int t_lo = n_kept ? c * A32_CHUNK : max(c * A32_CHUNK, first_tile), t_hi = min((c + 1) * A32_CHUNK, last_tile);
     for (int t = t_lo + wave; t < t_hi; t += A32_WAVES) {
+      if (t >= n_kept && t < first_tile) continue;
       float m_t, l_t;
       f32x4 o[HDT];
       attention_f32_tile<HDT>(t * FA_KT, bt, max_blocks, block_size, nkv, kvh, k_cache, v_cache,
-                              q + (int64_t)tok0 * q_stride + (int64_t)kvh * G * HD, qf, c_log2, row_valid, pos, row_lo,
-                              kv_begin, kv_end, Vl, m_t, l_t, o);
+                              q + (int64_t)tok0 * q_stride + (int64_t)kvh * G * HD, qf, scale, mask, row_valid, pos,
+                              row_lo, kv_begin, kv_end, Vl, m_t, l_t, o);
       // ---- the tile's (m, l, O) to its slot: lane (l16, kk) holds row l16, dims 16 dt + 4 kk + r
       const int slot = t - c * A32_CHUNK;
 #pragma unroll
@@ -801,6 +851,7 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_kernel(
       const int e = tid + A32_THREADS * u, row = e / HD, d = e % HD;
       float Mc = kNegBig, Lc = 0.f, Oc = 0.f, wa, wb;
       for (int t = t_lo; t < t_hi; ++t) {
+        if (t >= n_kept && t < first_tile) continue;
         const int slot = t - c * A32_CHUNK;
         merge_f32(Mc, Lc, Pml[(slot * 16 + row) * 2], Pml[(slot * 16 + row) * 2 + 1], wa, wb);
         Oc = merge_f32_value(Oc, Po[(slot * 16 + row) * PS + d], wa, wb);
@@ -844,7 +895,7 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
     const float* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
     const int32_t* __restrict__ tile_ntok, const int32_t* __restrict__ positions, float* __restrict__ out,
-    int64_t out_stride, int nq, int nkv, int block_size, float scale, int window, int sink, int n_tiles) {
+    int64_t out_stride, int nq, int nkv, int block_size, float scale, KeyMask mask, int sink, int n_tiles) {
   constexpr int HD = HDT * 16;
   extern __shared__ __attribute__((aligned(16))) float smem32[];
   const int tid = threadIdx.x, lane = tid % TL_WAVE, wave = tid / TL_WAVE;
@@ -862,11 +913,12 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
   const bool row_valid = tok_local < TW && tok_local < ntok;
   const int tok = tok0 + (row_valid ? tok_local : 0);
   const int pos = row_valid ? positions[tok] : -1;
-  const int row_lo = first_visible_key(pos, window);
+  const int row_lo = first_visible_key(pos, mask.window);
   const int hi = row_max_i32(pos), lo = row_min_i32(row_valid ? row_lo : 0x7fffffff);
   const int kv_end = hi + 1, kv_begin = lo;
   const int first_tile = kv_begin / FA_KT, last_tile = (kv_end + FA_KT - 1) / FA_KT;
-  const int c_first = first_tile / A32_CHUNK, c_last = (last_tile + A32_CHUNK - 1) / A32_CHUNK;
+  const int n_kept = kept_key_tiles(mask.keep, first_tile);      // tiles of kept first keys, as in attention_f32_kernel
+  const int c_first = n_kept ? 0 : first_tile / A32_CHUNK, c_last = (last_tile + A32_CHUNK - 1) / A32_CHUNK;
 
   f32x4 qf[HDT];
   {
@@ -875,7 +927,6 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
     for (int g4 = 0; g4 < HDT; ++g4)
       qf[g4] = row_valid ? *(const f32x4*)(qrow + g4 * 16 + kk * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
   }
-  const float c_log2 = scale * 1.44269504088896341f;
   const float* finite_row = q + (int64_t)tok0 * q_stride + (int64_t)kvh * G * HD;
 
   // lane (l16, kk) holds row l16, dims 16 dt + 4 kk + r of the running result
@@ -884,16 +935,18 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
 #pragma unroll
   for (int dt = 0; dt < HDT; ++dt) Orun[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int c = c_first; c < c_last; ++c) {
-    const int t_lo = max(c * A32_CHUNK, first_tile), t_hi = min((c + 1) * A32_CHUNK, last_tile);
+    if ((c + 1) * A32_CHUNK <= first_tile && c * A32_CHUNK >= n_kept) continue;
+    const int t_lo = n_kept ? c * A32_CHUNK : max(c * A32_CHUNK, first_tile), t_hi = min((c + 1) * A32_CHUNK, last_tile);
     float Mc = kNegBig, Lc = 0.f, wa, wb;
     f32x4 Oc[HDT];
 #pragma unroll
     for (int dt = 0; dt < HDT; ++dt) Oc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
     for (int t = t_lo; t < t_hi; ++t) {
+      if (t >= n_kept && t < first_tile) continue;
       float m_t, l_t;
       f32x4 o[HDT];
-      attention_f32_tile<HDT>(t * FA_KT, bt, max_blocks, block_size, nkv, kvh, k_cache, v_cache, finite_row, qf, c_log2,
-                              row_valid, pos, row_lo, kv_begin, kv_end, Vl, m_t, l_t, o);
+      attention_f32_tile<HDT>(t * FA_KT, bt, max_blocks, block_size, nkv, kvh, k_cache, v_cache, finite_row, qf, scale,
+                              mask, row_valid, pos, row_lo, kv_begin, kv_end, Vl, m_t, l_t, o);
       merge_f32(Mc, Lc, m_t, l_t, wa, wb);
 #pragma unroll
       for (int dt = 0; dt < HDT; ++dt)
@@ -945,14 +998,14 @@ __global__ __launch_bounds__(TL_WAVE) void attention_f32_combine_kernel(const fl
 constexpr int FP_RT = 1;                      // query tiles (of 16 rows) per wave
 // waves (query tiles) of a workgroup: 8, or 4 where 8 would leave compute units without work
 
-template <int HDT, int WAVES>
+template <int HDT, int WAVES, bool CAP>
 __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
     const bf16_t* __restrict__ q, int64_t q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
     const int32_t* __restrict__ tile_ntok, const int32_t* __restrict__ positions, bf16_t* __restrict__ out,
     int64_t out_stride, float* __restrict__ part_o, float* __restrict__ part_ml, int n_tiles, int n_tokens,
-    int n_splits, int nq, int nkv, int block_size, int bs_shift, float scale, int window, int sink) {
+    int n_splits, int nq, int nkv, int block_size, int bs_shift, float scale, KeyMask mask, int sink) {
   constexpr int HD = HDT * 16;
   constexpr int KS = (HD + 31) / 32;
   constexpr int KP = KS * 32 + 8;
@@ -980,8 +1033,17 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
   // the tokens of a tile are consecutive tokens of one request, so their positions are consecutive
   const int pos_first = positions[tok0], pos_last = pos_first + ntok - 1;
   const int kv_end = pos_last + 1;
-  const int kv_begin = first_visible_key(pos_first, window);
+  const int kv_begin = first_visible_key(pos_first, mask.window);
   int first_tile = kv_begin / FA_KT, last_tile = (kv_end + FA_KT - 1) / FA_KT;
+  // Tiles of kept first keys come in front of the window's: the loop counts n_kept + (last - first) numbers, number n
+  // is tile n, or n + skip from n_kept on (first_tile, last_tile are numbers from here on; without kept keys
+  // number and tile are one).
+  const int n_kept = kept_key_tiles(mask.keep, first_tile), skip = mask.keep > 0 ? first_tile - n_kept : 0;
+  if (mask.keep > 0) {
+    last_tile -= skip;
+    first_tile = 0;
+  }
+  auto tile_of = [&](int n) { return n >= n_kept ? n + skip : n; };
   if (n_splits > 1) {       // this workgroup's share of the key tiles (possibly none)
     const int per = (last_tile - first_tile + n_splits - 1) / n_splits;
     first_tile = min(first_tile + split * per, last_tile);
@@ -999,7 +1061,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
     row_valid[rt] = r16 / G < TW && tok_local < ntok;
     tok[rt] = tok0 + (row_valid[rt] ? tok_local : 0);
     pos[rt] = row_valid[rt] ? pos_first + tok_local : -1;
-    row_lo[rt] = first_visible_key(pos[rt], window);
+    row_lo[rt] = first_visible_key(pos[rt], mask.window);
     const bf16_t* qrow = q + (int64_t)tok[rt] * q_stride + (int64_t)head * HD;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
@@ -1031,7 +1093,9 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
 #pragma unroll
     for (int dt = 0; dt < HDT; ++dt) o[rt][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
-  const float c_log2 = scale * 1.44269504088896341f;     // scores are kept in units of log2 e
+  // scores are kept in units of log2 e (CAP: the cap leaves them so)
+  const float c_log2 = CAP ? 1.f : scale * 1.44269504088896341f;
+  const float cap_in = CAP ? scale * 2.88539008177792681f / mask.cap : 0.f, cap_out = mask.cap * 1.44269504088896341f;
   // smallest position and largest window start among this wave's valid rows: a key tile that lies
   // wholly between them is visible to every row and needs no mask
   int wave_lo_pos = 0x7fffffff, wave_hi_lo = 0;
@@ -1060,13 +1124,16 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
   // Rows of a tile outside the request's keys [kv_begin, kv_end) are read from the nearest row
   // inside instead (finite data of the same request; every score of such a key is masked, and its
   // probability is an exact zero): so no load is predicated, which would make it a branch.
-  auto key_row = [&](int kt_idx) { return min(max(kt_idx * FA_KT + lane, kv_begin), kv_end - 1); };
-  auto page_of_row = [&](int kt_idx) {
-    const int j = key_row(kt_idx);
+  auto key_row = [&](int n) {
+    const int j = tile_of(n) * FA_KT + lane;
+    return min(j < mask.keep ? j : max(j, kv_begin), kv_end - 1);
+  };
+  auto page_of_row = [&](int n) {
+    const int j = key_row(n);
     return bt[bs_shift >= 0 ? j >> bs_shift : j / block_size];     // uniform choice: no division
   };
-  auto fetch_tile = [&](int kt_idx, int blk) {
-    const int j = key_row(kt_idx);
+  auto fetch_tile = [&](int n, int blk) {
+    const int j = key_row(n);
     const int jb = bs_shift >= 0 ? j >> bs_shift : j / block_size;
     // rows of the cache fit 32 bits (checked on the host); only the last product is 64 bits wide
     const int row = (max(blk, 0) * nkv + kvh) * block_size + (j - jb * block_size);
@@ -1120,17 +1187,18 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
   __builtin_amdgcn_s_waitcnt(0x0F70);      // vmcnt(0)
   __syncthreads();
 
-  for (int kt_idx = first_tile; kt_idx < last_tile; ++kt_idx) {
-    const int cur = (kt_idx - first_tile) & 1;
+  for (int n = first_tile; n < last_tile; ++n) {
+    const int cur = (n - first_tile) & 1;
     // the next tile (requested one iteration ago) goes into the other buffer, which every wave
     // has finished reading before the last barrier; then the tile after it is requested
-    if (kt_idx + 1 < last_tile) {
+    if (n + 1 < last_tile) {
       store_tile(cur ^ 1);
-      if (kt_idx + 2 < last_tile) {
-        fetch_tile(kt_idx + 2, next_page);
-        if (kt_idx + 3 < last_tile) next_page = page_of_row(kt_idx + 3);
+      if (n + 2 < last_tile) {
+        fetch_tile(n + 2, next_page);
+        if (n + 3 < last_tile) next_page = page_of_row(n + 3);
       }
     }
+    const int kt_idx = tile_of(n);
     const bf16_t* Kl = Kbuf[cur];
     const bf16_t* Vl = Vbuf[cur];
     // The whole tile in two compilations, with and without the mask: written as one body with a
@@ -1154,6 +1222,14 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
           for (int rt = 0; rt < FP_RT; ++rt)
             sc[rt][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[rt][ks], sc[rt][kt], 0, 0, 0);
         }
+      if constexpr (CAP) {
+#pragma unroll
+        for (int rt = 0; rt < FP_RT; ++rt)
+#pragma unroll
+          for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) sc[rt][kt][r] = capped_score(sc[rt][kt][r], cap_in, cap_out);
+      }
       bf16x8 pb[FP_RT][2], pl[FP_RT][2];
       const int tile_j0 = kt_idx * FA_KT;
 #pragma unroll
@@ -1170,7 +1246,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int j = tile_j0 + kt * 16 + g * 4 + r;
-              const bool ok = row_valid[rt] && j <= pos[rt] && j >= row_lo[rt];
+              const bool ok = row_valid[rt] && key_visible(j, pos[rt], row_lo[rt], mask.keep);
               const float sv = ok ? sc[rt][kt][r] : -INFINITY;
               sc[rt][kt][r] = sv;
               m_tile = fmaxf(m_tile, sv);
@@ -1249,7 +1325,8 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
       // a key tile that lies wholly between the wave's smallest position and its largest window
       // start is visible to every row
       const int tile_j0 = kt_idx * FA_KT;
-      const bool no_mask = all_valid && tile_j0 + FA_KT - 1 <= wave_lo_pos && tile_j0 >= wave_hi_lo;
+      const bool no_mask = all_valid && tile_j0 + FA_KT - 1 <= wave_lo_pos &&
+                           (tile_j0 >= wave_hi_lo || tile_j0 + FA_KT <= mask.keep);
       if (no_mask) work_on_tile(std::false_type{});
       else work_on_tile(std::true_type{});
     }
@@ -1367,12 +1444,12 @@ __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __r
   }
 }
 
-template <int HDT, int WAVES>
+template <int HDT, int WAVES, bool CAP>
 static int launch_flash_w(const bf16_t* q, int64_t q_stride, const bf16_t* k_cache, const bf16_t* v_cache,
                           const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                           const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, bf16_t* out,
                           int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq,
-                          int nkv, int block_size, float scale, int window, int sink, int n_splits, const FusedRope& fused,
+                          int nkv, int block_size, float scale, KeyMask mask, int sink, int n_splits, const FusedRope& fused,
                           hipStream_t stream) {
   constexpr int HD = HDT * 16;
   constexpr size_t stage = (size_t)WAVES * FA_KT * (HD + FA_VPAD) * sizeof(bf16_t);
@@ -1380,14 +1457,14 @@ static int launch_flash_w(const bf16_t* q, int64_t q_stride, const bf16_t* k_cac
                 "a wave's merge area must fit its staging area");
   static bool configured = false;
   if (!configured) {
-    if (hipFuncSetAttribute((const void*)flash_attn_bf16_kernel<HDT, WAVES>,
+    if (hipFuncSetAttribute((const void*)flash_attn_bf16_kernel<HDT, WAVES, CAP>,
                             hipFuncAttributeMaxDynamicSharedMemorySize, (int)stage) != hipSuccess)
       return TL_ERR_LAUNCH;
     configured = true;
   }
-  hipLaunchKernelGGL((flash_attn_bf16_kernel<HDT, WAVES>), dim3(n_tiles, nkv, n_splits), dim3(WAVES * TL_WAVE), stage,
+  hipLaunchKernelGGL((flash_attn_bf16_kernel<HDT, WAVES, CAP>), dim3(n_tiles, nkv, n_splits), dim3(WAVES * TL_WAVE), stage,
                      stream, q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
-                     positions, out, out_stride, part_o, part_ml, nq, nkv, block_size, scale, window, sink, n_splits,
+                     positions, out, out_stride, part_o, part_ml, nq, nkv, block_size, scale, mask, sink, n_splits,
                      n_tokens, fused);
   return TL_OK;
 }
@@ -1400,23 +1477,25 @@ static int launch_flash_w(const bf16_t* q, int64_t q_stride, const bf16_t* k_cac
 // has few: measured on whole decode steps, batch 1 and 8 gain 1 %, batch 64 would lose 2 %.
 static int flash_waves(int hd, int groups) { return hd <= 64 && groups > 64 ? 8 : 4; }
 
-template <int HDT>
+template <int HDT, bool CAP>
 static int launch_flash(const bf16_t* q, int64_t q_stride, const bf16_t* k_cache, const bf16_t* v_cache,
                         const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                         const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, bf16_t* out,
                         int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq, int nkv,
-                        int block_size, float scale, int window, int sink, int n_splits, const FusedRope& fused,
+                        int block_size, float scale, KeyMask mask, int sink, int n_splits, const FusedRope& fused,
                         hipStream_t stream) {
   if constexpr (HDT <= 4) {
     if (flash_waves(HDT * 16, n_tiles * nkv) == 8)
-      return launch_flash_w<HDT, 8>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0,
+      return launch_flash_w<HDT, 8, CAP>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0,
                                     tile_ntok, positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv,
-                                    block_size, scale, window, sink, n_splits, fused, stream);
+                                    block_size, scale, mask, sink, n_splits, fused, stream);
   }
-  return launch_flash_w<HDT, 4>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
+  return launch_flash_w<HDT, 4, CAP>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                                 positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, block_size,
-                                scale, window, sink, n_splits, fused, stream);
+                                scale, mask, sink, n_splits, fused, stream);
 }
+
+static bool mask_ok(int keep, float softcap) { return keep >= 0 && softcap >= 0.f; }
 
 }  // namespace
 
@@ -1427,21 +1506,23 @@ extern "C" {
 int tl_paged_attention(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                        const int32_t* block_tables, int max_blocks, const int32_t* req_of_token,
                        const int32_t* positions, void* out, int64_t out_stride, int n_tokens, int nq,
-                       int nkv, int hd, int block_size, float scale, int window, int sink, int dtype,
+                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, int sink, int dtype,
                        hipStream_t stream) {
   if (n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || hd <= 0 || hd > kMaxHd || block_size <= 0 || max_blocks <= 0 ||
       nq > 65535)
     return TL_ERR_ARG;
+  if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
+  const KeyMask mask{window, keep, softcap};
   dim3 g(n_tokens, nq), b(TL_WAVE);
   if (dtype == 0)
     hipLaunchKernelGGL(paged_attention_kernel<float>, g, b, 0, stream, (const float*)q, q_stride,
                        (const float*)k_cache, (const float*)v_cache, block_tables, max_blocks, req_of_token,
-                       positions, (float*)out, out_stride, nq, nkv, hd, block_size, scale, window, sink);
+                       positions, (float*)out, out_stride, nq, nkv, hd, block_size, scale, mask, sink);
   else if (dtype == 1)
     hipLaunchKernelGGL(paged_attention_kernel<bf16_t>, g, b, 0, stream, (const bf16_t*)q, q_stride,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_blocks, req_of_token,
-                       positions, (bf16_t*)out, out_stride, nq, nkv, hd, block_size, scale, window, sink);
+                       positions, (bf16_t*)out, out_stride, nq, nkv, hd, block_size, scale, mask, sink);
   else
     return TL_ERR_ARG;
   return tl_launch_status();
@@ -1455,7 +1536,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
                      const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                      const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, float* out,
                      int64_t out_stride, float* part, int n_tiles, int n_tokens, int nq, int nkv, int hd,
-                     int block_size, float scale, int window, int sink, int n_chunks, hipStream_t stream) {
+                     int block_size, float scale, int window, int keep, float softcap, int sink, int n_chunks, hipStream_t stream) {
   if (n_tiles <= 0 || n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || nq / nkv > 16 || hd <= 0 || hd % 16 || hd > 128 || block_size <= 0 ||
       max_blocks <= 0 || n_chunks < 1 || nkv > 65535 || n_chunks > 65535 || q_stride % 4 ||
@@ -1464,6 +1545,8 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
   if (n_chunks > 1 && !part) return TL_ERR_ARG;
   if (!tile_req && (tile_tok0 || tile_ntok || n_tiles != n_tokens)) return TL_ERR_ARG;
   if (tile_req && (!tile_tok0 || !tile_ntok)) return TL_ERR_ARG;
+  if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
+  const KeyMask mask{window, keep, softcap};
   const size_t smem = (size_t)(A32_WAVES * FA_KT * A32_VS + A32_CHUNK * 16 * (hd + 4) + A32_CHUNK * 16 * 2) * sizeof(float);
   // Many query tiles (prompts): a wave a tile, four neighbouring tiles a workgroup; few (decode steps, small
   // steps): a workgroup a tile, its waves sharing the key tiles out.  The same bits either way.
@@ -1481,7 +1564,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
     hipLaunchKernelGGL(attention_f32_rows_kernel<HDT>, dim3((n_tiles + A32_WAVES - 1) / A32_WAVES, nkv),           \
                        dim3(A32_THREADS), smem_rows, stream, q, q_stride, k_cache, v_cache, block_tables,          \
                        max_blocks, tile_req, tile_tok0, tile_ntok, positions, out, out_stride, nq, nkv,            \
-                       block_size, scale, window, sink, n_tiles);                                                        \
+                       block_size, scale, mask, sink, n_tiles);                                                        \
   } break;
     switch (hd / 16) {
       TL_A32_ROWS(1) TL_A32_ROWS(2) TL_A32_ROWS(3) TL_A32_ROWS(4)
@@ -1501,7 +1584,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
     }                                                                                                             \
     hipLaunchKernelGGL(attention_f32_kernel<HDT>, dim3(n_tiles, nkv, n_chunks), dim3(A32_THREADS), smem, stream,  \
                        q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,   \
-                       positions, out, out_stride, part, nq, nkv, block_size, scale, window, sink, n_tokens);           \
+                       positions, out, out_stride, part, nq, nkv, block_size, scale, mask, sink, n_tokens);           \
   } break;
   switch (hd / 16) {
     TL_A32_CASE(1) TL_A32_CASE(2) TL_A32_CASE(3) TL_A32_CASE(4)
@@ -1521,7 +1604,7 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
                      const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                      const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
                      int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq, int nkv,
-                     int hd, int block_size, float scale, int window, int sink, int tile_waves, int n_splits,
+                     int hd, int block_size, float scale, int window, int keep, float softcap, int sink, int tile_waves, int n_splits,
                      hipStream_t stream) {
   if (n_tiles <= 0) return TL_OK;
   if (tile_waves != 8 && tile_waves != 4) return TL_ERR_ARG;
@@ -1534,19 +1617,23 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
       max_blocks <= 0 || nkv > 65535 || (int64_t)n_tiles * nkv > 0x7fffffff || q_stride % 8 ||
       out_stride % 4)
     return TL_ERR_ARG;
+  if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
+  const KeyMask mask{window, keep, softcap};
   int bs_shift = -1;      // log2 of the page size where it is a power of two
   for (int sh = 0; sh < 31; ++sh)
     if ((1 << sh) == block_size) bs_shift = sh;
-#define TL_PREFILL_LAUNCH(HDT, W)                                                                                 \
-  hipLaunchKernelGGL((flash_prefill_bf16_kernel<HDT, W>), dim3(n_tiles * nkv * n_splits), dim3(W * TL_WAVE), 0,   \
+#define TL_PREFILL_LAUNCH(HDT, W, CAP)                                                                            \
+  hipLaunchKernelGGL((flash_prefill_bf16_kernel<HDT, W, CAP>), dim3(n_tiles * nkv * n_splits), dim3(W * TL_WAVE), 0,   \
                      stream, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,          \
                      block_tables, max_blocks, tile_req, tile_tok0, tile_ntok, positions, (bf16_t*)out,           \
                      out_stride, part_o, part_ml, n_tiles, n_tokens, n_splits, nq, nkv, block_size, bs_shift,     \
-                     scale, window, sink)
+                     scale, mask, sink)
 #define TL_PREFILL_CASE(HDT)                        \
   case HDT:                                         \
-    if (tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8); \
-    else TL_PREFILL_LAUNCH(HDT, 4);                 \
+    if (softcap > 0.f && tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, true); \
+    else if (softcap > 0.f) TL_PREFILL_LAUNCH(HDT, 4, true);               \
+    else if (tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, false);            \
+    else TL_PREFILL_LAUNCH(HDT, 4, false);                                 \
     break;
   switch (hd / 16) {
     TL_PREFILL_CASE(1) TL_PREFILL_CASE(2) TL_PREFILL_CASE(3) TL_PREFILL_CASE(4)
@@ -1576,7 +1663,7 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
                                const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                                const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
                                int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq,
-                               int nkv, int hd, int block_size, float scale, int window, int sink, int n_splits,
+                               int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, int sink, int n_splits,
                                const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
   if (n_tiles <= 0 || n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || nq / nkv > 16 || hd <= 0 || hd % 16 || hd > 128 || block_size <= 0 ||
@@ -1590,12 +1677,14 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
   if (fuse_store && (!rope_cos || !rope_sin || n_tiles != n_tokens)) return TL_ERR_ARG;
   FusedRope fused{fuse_store ? rope_cos : nullptr, fuse_store ? rope_sin : nullptr, (bf16_t*)k_cache, (bf16_t*)v_cache,
                   nq * hd, (nq + nkv) * hd};
+  if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
+  const KeyMask mask{window, keep, softcap};
   int rc = TL_ERR_ARG;
 #define TL_FLASH_CASE(HDT)                                                                                       \
   case HDT:                                                                                                      \
-    rc = launch_flash<HDT>((const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,           \
+    rc = (softcap > 0.f ? launch_flash<HDT, true> : launch_flash<HDT, false>)((const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,           \
                            block_tables, max_blocks, tile_req, tile_tok0, tile_ntok, positions, (bf16_t*)out,    \
-                           out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, block_size, scale, window, sink,   \
+                           out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, block_size, scale, mask, sink,   \
                            n_splits, fused, stream);                                                             \
     break;
   switch (hd / 16) {
@@ -1623,7 +1712,20 @@ int tl_flash_attention(const void* q, int64_t q_stride, const void* k_cache, con
                        const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
   return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                              positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
-                             scale, window, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+                             scale, window, 0, 0.f, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+}
+
+// The same with the rest of the mask: the request's first `keep` tokens stay visible behind a window, and softcap > 0
+// caps the scores, cap * tanh(score / cap).
+int tl_flash_attention_masked(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
+                       const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
+                       const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
+                       int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq,
+                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, int sink, int n_splits,
+                       const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
+  return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
+                             positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
+                             scale, window, keep, softcap, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
 }
 
 // ------------------------------------------------ the entry point that allocates nothing
@@ -1676,7 +1778,7 @@ int tl_flash_attention_static(const void* q, int64_t q_stride, const void* k_cac
   }
   return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                              positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
-                             scale, window, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+                             scale, window, 0, 0.f, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
 }
 
 }  // extern "C"

@@ -105,11 +105,13 @@ __global__ __launch_bounds__(kPrepThreads) void delta_prepare_kernel(
 }
 
 // The convolutions' saved inputs after a step: the last taps - 1 of (what was saved, this step's
-// inputs).  One thread per (request, channel); it reads all it needs before it writes.
+// inputs, each with its channel's bias added if the projections carry one).  One thread per (request, channel); it
+// reads all it needs before it writes.
 constexpr int kMaxTaps = 16;
 template <typename T>
 __global__ void conv_state_update_kernel(const T* __restrict__ p, int64_t p_stride, int conv_off, int channels,
-                                         float* __restrict__ state, int64_t state_stride, int64_t saved_off,
+                                         const float* __restrict__ bias, float* __restrict__ state,
+                                         int64_t state_stride, int64_t saved_off,
                                          const int32_t* __restrict__ cu_seqlens,
                                          const int32_t* __restrict__ state_slots, int taps) {
   const int r = blockIdx.y;
@@ -118,9 +120,14 @@ __global__ void conv_state_update_kernel(const T* __restrict__ p, int64_t p_stri
   if (c >= channels || n <= 0) return;
   float* saved = state + (int64_t)state_slots[r] * state_stride + saved_off + (int64_t)c * (taps - 1);
   float next[kMaxTaps];
+  const float b = bias ? bias[c] : 0.f;
 #pragma unroll
   for (int i = 0; i < kMaxTaps; ++i)
-    if (i < taps - 1) next[i] = conv_input(p, p_stride, t0, n - (taps - 1) + i, conv_off + c, saved, taps);
+    if (i < taps - 1) {
+      const int m = n - (taps - 1) + i;
+      next[i] = conv_input(p, p_stride, t0, m, conv_off + c, saved, taps);
+      if (m >= 0) next[i] += b;           // what is saved has it already
+    }
 #pragma unroll
   for (int i = 0; i < kMaxTaps; ++i)
     if (i < taps - 1) saved[i] = next[i];
@@ -468,14 +475,14 @@ int tl_delta_prepare(const void* p, int64_t p_stride, int conv_off, int b_off, c
   return tl_launch_status();
 }
 
-int tl_conv_state_update(const void* p, int64_t p_stride, int conv_off, int channels, float* state,
+int tl_conv_state_update(const void* p, int64_t p_stride, int conv_off, int channels, const float* bias, float* state,
                          int64_t state_stride, int64_t saved_off, const int32_t* cu_seqlens,
                          const int32_t* state_slots, int n_requests, int taps, int dtype, hipStream_t stream) {
   if (n_requests <= 0 || taps <= 1) return TL_OK;
   if (channels <= 0 || taps > kMaxTaps || n_requests > 65535) return TL_ERR_ARG;
   dim3 g((channels + 255) / 256, n_requests), b(256);
   TL_DISPATCH_T(dtype, hipLaunchKernelGGL(conv_state_update_kernel<T>, g, b, 0, stream, (const T*)p, p_stride,
-                                          conv_off, channels, state, state_stride, saved_off, cu_seqlens, state_slots,
+                                          conv_off, channels, bias, state, state_stride, saved_off, cu_seqlens, state_slots,
                                           taps);)
   return tl_launch_status();
 }

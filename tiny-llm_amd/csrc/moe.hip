@@ -412,6 +412,9 @@ __global__ void moe_combine_kernel(const float* __restrict__ y, const float* __r
 // experts of the `keep` best runs may be chosen (groups <= 1: all may).  The `top` largest scores among those
 // are chosen, largest first (equal scores: the lower index first); ids[t, j] names them, and
 // wts[t, j] = s_j / (sum of the chosen s + 1e-20) * scale.
+// Options: sigmoid scores s = sigmoid(z); a correction per expert that is added to the score for every choice and
+// left out of the weights (choice scores may then be negative: whatever is out counts as minus infinity); a run's
+// score as the sum of its two largest choice scores; weights s_j * scale without the division.
 constexpr int kMaxRouted = 1024;
 
 struct Best {
@@ -433,9 +436,12 @@ __device__ __forceinline__ Best wave_best(Best x) {
 __global__ __launch_bounds__(TL_WAVE) void moe_route_kernel(const float* __restrict__ z, int64_t z_stride,
                                                             const float* __restrict__ bias, int32_t* __restrict__ ids,
                                                             float* __restrict__ wts, int experts, int top, int groups,
-                                                            int keep, float scale) {
-  __shared__ float s[kMaxRouted];         // scores; -1 once an expert is chosen or its run is out
+                                                            int keep, float scale, int sigmoid,
+                                                            const float* __restrict__ correction, int group_top2,
+                                                            int normalize) {
+  __shared__ float s[kMaxRouted];         // choice scores; -inf once an expert is chosen or its run is out
   __shared__ float gs[kMaxRouted];        // the runs' scores
+  __shared__ float plain[kMaxRouted];     // scores without the correction
   const int t = blockIdx.x, lane = threadIdx.x;
   const float* zr = z + (int64_t)t * z_stride;
   float m = -INFINITY;
@@ -444,52 +450,67 @@ __global__ __launch_bounds__(TL_WAVE) void moe_route_kernel(const float* __restr
     s[e] = l;
     m = fmaxf(m, l);
   }
-  m = wave_max(m);
-  float sum = 0.f;
-  for (int e = lane; e < experts; e += TL_WAVE) {
-    const float p = expf(s[e] - m);
-    s[e] = p;
-    sum += p;
+  if (sigmoid) {
+    for (int e = lane; e < experts; e += TL_WAVE) s[e] = 1.f / (1.f + expf(-s[e]));
+  } else {
+    m = wave_max(m);
+    float sum = 0.f;
+    for (int e = lane; e < experts; e += TL_WAVE) {
+      const float p = expf(s[e] - m);
+      s[e] = p;
+      sum += p;
+    }
+    sum = wave_sum(sum);
+    const float inv = 1.f / sum;
+    for (int e = lane; e < experts; e += TL_WAVE) s[e] *= inv;
   }
-  sum = wave_sum(sum);
-  const float inv = 1.f / sum;
-  for (int e = lane; e < experts; e += TL_WAVE) s[e] *= inv;
+  if (correction) {
+    for (int e = lane; e < experts; e += TL_WAVE) {
+      plain[e] = s[e];
+      s[e] += correction[e];
+    }
+  }
   __syncthreads();
   if (groups > 1 && keep < groups) {
     const int per = experts / groups;
     for (int g = lane; g < groups; g += TL_WAVE) {
-      float b = -1.f;
-      for (int e = g * per; e < (g + 1) * per; ++e) b = fmaxf(b, s[e]);
-      gs[g] = b;
+      float b = -INFINITY, second = -INFINITY;
+      for (int e = g * per; e < (g + 1) * per; ++e) {
+        second = fmaxf(second, fminf(b, s[e]));
+        b = fmaxf(b, s[e]);
+      }
+      gs[g] = group_top2 && per > 1 ? b + second : b;
     }
     __syncthreads();
-    for (int k = 0; k < keep; ++k) {      // the best runs, one a pass; a kept run is marked with -2
-      Best b = {-1.f, 0x7fffffff};
+    for (int k = 0; k < keep; ++k) {      // the best runs, one a pass; a kept run is marked with -inf
+      Best b = {-INFINITY, 0x7fffffff};
       for (int g = lane; g < groups; g += TL_WAVE) b = better(b, Best{gs[g], g});
       b = wave_best(b);
       __syncthreads();
-      if (lane == 0) gs[b.i] = -2.f;
+      if (lane == 0) gs[min(b.i, groups - 1)] = -INFINITY;      // (no index at all: every score is NaN)
       __syncthreads();
     }
     for (int e = lane; e < experts; e += TL_WAVE)
-      if (gs[e / per] != -2.f) s[e] = -1.f;
+      if (gs[e / per] != -INFINITY) s[e] = -INFINITY;
     __syncthreads();
   }
   float total = 0.f;
   for (int j = 0; j < top; ++j) {         // the best of what is left, one a pass; gs now keeps the chosen scores
-    Best b = {-2.f, 0x7fffffff};
+    Best b = {-INFINITY, 0x7fffffff};
     for (int e = lane; e < experts; e += TL_WAVE) b = better(b, Best{s[e], e});
     b = wave_best(b);
+    b.i = min(b.i, experts - 1);
     __syncthreads();
+    const float score = correction ? plain[b.i] : b.v;
     if (lane == 0) {
-      s[b.i] = -3.f;
-      gs[j] = b.v;
+      s[b.i] = -INFINITY;
+      gs[j] = score;
       ids[(int64_t)t * top + j] = b.i;
     }
-    total += b.v;
+    total += score;
     __syncthreads();
   }
-  const float f = scale / (total + 1e-20f);
+  const float f = normalize ? scale / (total + 1e-20f) : scale;
   for (int j = lane; j < top; j += TL_WAVE) wts[(int64_t)t * top + j] = gs[j] * f;
 }
 
@@ -662,13 +683,14 @@ int tl_row_dot_sigmoid(const void* a, int64_t a_stride, const void* w, float* ou
 
 // z: float32 [n_tokens, experts] (row stride z_stride); ids: int32 [n_tokens, top]; wts: float32 [n_tokens, top].
 int tl_moe_route(const float* z, int64_t z_stride, const float* bias, int32_t* ids, float* wts, int n_tokens, int experts,
-                 int top, int groups, int keep, float scale, hipStream_t stream) {
+                 int top, int groups, int keep, float scale, int sigmoid, const float* correction, int group_top2,
+                 int normalize, hipStream_t stream) {
   if (n_tokens <= 0) return TL_OK;
   if (experts <= 0 || experts > kMaxRouted || top <= 0 || top > experts || z_stride < experts || !z || !ids || !wts ||
       groups < 0 || (groups > 1 && (experts % groups || keep <= 0 || keep > groups || top > keep * (experts / groups))))
     return TL_ERR_ARG;
   hipLaunchKernelGGL(moe_route_kernel, dim3(n_tokens), dim3(TL_WAVE), 0, stream, z, z_stride, bias, ids, wts, experts, top,
-                     groups, keep, scale);
+                     groups, keep, scale, sigmoid, correction, group_top2, normalize);
   return tl_launch_status();
 }
 

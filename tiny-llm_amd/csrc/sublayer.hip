@@ -99,6 +99,24 @@ __global__ void gelu_glu_kernel(const T* __restrict__ gate_up, T* __restrict__ z
   z[i] = from_f32<T>(act * u);
 }
 
+// z[t, j] = gelu(gate[t, j]) * table[tokens[t], off + j] for j < dim (gelu in its tanh form), zeros up to the row's `wide`.
+template <typename T>
+__global__ void gelu_table_rows_kernel(const float* __restrict__ gate, int64_t gate_stride, const int32_t* __restrict__ tokens,
+                                       const T* __restrict__ table, int64_t table_stride, int off, T* __restrict__ z,
+                                       int64_t total, int dim, int wide) {
+  const int64_t i = (int64_t)blockIdx.x * kThreads + threadIdx.x;
+  if (i >= total) return;
+  const int64_t t = i / wide;
+  const int j = (int)(i - t * wide);
+  float v = 0.f;
+  if (j < dim) {
+    const float g = gate[t * gate_stride + j];
+    const float act = 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+    v = act * to_f32(table[(int64_t)tokens[t] * table_stride + off + j]);
+  }
+  z[i] = from_f32<T>(v);
+}
+
 __global__ void softcap_kernel(float* __restrict__ x, int64_t total, float cap) {
   const int64_t i = (int64_t)blockIdx.x * kThreads + threadIdx.x;
   if (i < total) x[i] = cap * tanhf(x[i] / cap);
@@ -181,6 +199,25 @@ int tl_gelu_glu(const void* gate_up, void* z, int n_rows, int inter, int64_t in_
   else if (dtype == 1)
     hipLaunchKernelGGL(gelu_glu_kernel<bf16_t>, g, b, 0, stream, (const bf16_t*)gate_up, (bf16_t*)z, total, inter,
                        in_stride);
+  else
+    return TL_ERR_ARG;
+  return tl_launch_status();
+}
+
+// gate: float32 [n_rows, >= dim]; table: [vocab, table_stride] in dtype; z: [n_rows, wide] in dtype.
+int tl_gelu_table_rows(const float* gate, int64_t gate_stride, const int32_t* tokens, const void* table, int64_t table_stride,
+                       int off, void* z, int n_rows, int dim, int wide, int dtype, hipStream_t stream) {
+  if (n_rows <= 0) return TL_OK;
+  if (dim <= 0 || wide < dim || off < 0 || off + dim > table_stride || gate_stride < dim || !gate || !tokens || !table || !z)
+    return TL_ERR_ARG;
+  const int64_t total = (int64_t)n_rows * wide;
+  dim3 g((unsigned)ceil_div64(total, kThreads)), b(kThreads);
+  if (dtype == 0)
+    hipLaunchKernelGGL(gelu_table_rows_kernel<float>, g, b, 0, stream, gate, gate_stride, tokens, (const float*)table,
+                       table_stride, off, (float*)z, total, dim, wide);
+  else if (dtype == 1)
+    hipLaunchKernelGGL(gelu_table_rows_kernel<bf16_t>, g, b, 0, stream, gate, gate_stride, tokens, (const bf16_t*)table,
+                       table_stride, off, (bf16_t*)z, total, dim, wide);
   else
     return TL_ERR_ARG;
   return tl_launch_status();

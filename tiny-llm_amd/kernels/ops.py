@@ -8,6 +8,7 @@ computed on the CPU or by a library op.
 from __future__ import annotations
 
 import ctypes
+from dataclasses import dataclass
 from typing import Optional
 
 import torch
@@ -615,9 +616,10 @@ def _attn_types_ok(q, k_cache, v_cache, out) -> bool:
 def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                     block_tables: torch.Tensor, req_of_token: torch.Tensor, positions: torch.Tensor,
                     out: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, scale: float,
-                    window: int = 0, sink: bool = False) -> torch.Tensor:
+                    window: int = 0, sink: bool = False, keep: int = 0, softcap: float = 0.0) -> torch.Tensor:
     """Causal attention of every row of q (at its absolute position) over its
-    request's cached keys 0..position (the last `window` of them if window > 0).
+    request's cached keys 0..position (the last `window` of them if window > 0; the request's first `keep`
+    stay visible behind the window).  softcap > 0: every score s becomes softcap * tanh(s / softcap).
     sink: the softmax's denominator has one more term, exp(0), that carries no value."""
     _dev(q, k_cache, v_cache, block_tables, req_of_token, positions, out)
     _rows_2d(q, "q")
@@ -644,7 +646,8 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         _ptr(q), c_int64(q.stride(0)), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
         c_int(block_tables.shape[1]), _ptr(req_of_token), _ptr(positions), _ptr(out), c_int64(out.stride(0)),
         c_int(T), c_int(num_heads), c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]),
-        c_float(scale), c_int(window), c_int(_attn_flags(sink, q, out)), c_int(_dt(q)), _stream()), "paged_attention")
+        c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_int(_attn_flags(sink, q, out)), c_int(_dt(q)),
+        _stream()), "paged_attention")
     return out
 
 
@@ -660,7 +663,8 @@ def attention_f32_supported(dtype: torch.dtype, num_heads: int, num_kv_heads: in
 def attention_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
                   tiles, positions: torch.Tensor, out: torch.Tensor, num_heads: int, num_kv_heads: int,
                   head_dim: int, scale: float, window: int = 0, n_chunks: int = 1,
-                  scratch: Optional[torch.Tensor] = None, sink: bool = False) -> torch.Tensor:
+                  scratch: Optional[torch.Tensor] = None, sink: bool = False, keep: int = 0,
+                  softcap: float = 0.0) -> torch.Tensor:
     """The same function as `paged_attention` in true float32 on the matrix cores.  `tiles` as for
     `flash_attention` (None: row i is the one new token of request i).  n_chunks == 1: one
     workgroup per tile and kv head walks all keys; n_chunks > 1 (at least ceil(longest context /
@@ -707,7 +711,7 @@ def attention_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         _ptr(q, 16), c_int64(q.stride(0)), _ptr(k_cache, 16), _ptr(v_cache, 16), _ptr(block_tables),
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out), c_int64(out.stride(0)), _ptr(scratch), c_int(n_tiles), c_int(T), c_int(num_heads),
-        c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(1 if sink else 0),
+        c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_int(1 if sink else 0),
         c_int(n_chunks), _stream()), "attention_f32")
     return out
 
@@ -722,7 +726,7 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     tiles, positions: torch.Tensor, out: torch.Tensor, num_heads: int, num_kv_heads: int,
                     head_dim: int, scale: float, window: int = 0, n_splits: int = 1,
                     scratch: Optional[torch.Tensor] = None, fused_rope=None, static_scratch: bool = False,
-                    sink: bool = False) -> torch.Tensor:
+                    sink: bool = False, keep: int = 0, softcap: float = 0.0) -> torch.Tensor:
     """The same function as `paged_attention` on the matrix cores (bfloat16).  `tiles` =
     (tile_req, tile_tok0, tile_ntok): groups of at most 16 // (heads / kv_heads) consecutive
     tokens of one request; None for a decode step, where row i is the one new token of request i
@@ -789,6 +793,7 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         if not (q.stride(0) >= (num_heads + 2 * num_kv_heads) * head_dim):
             _fail("fused mode needs q inside its qkv rows")
     if static_scratch:
+        _need(keep == 0 and softcap == 0.0, "flash_attention: the static entry point takes no kept tokens and no soft cap")
         code = _lib().tl_flash_attention_static(
             _ptr(q, 16), c_int64(q.stride(0)), _ptr(k_cache, 16), _ptr(v_cache, 16), _ptr(block_tables),
             c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
@@ -800,12 +805,12 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                   f"heads x {head_dim + 2} floats exceed its {STATIC_SCRATCH_FLOATS} floats")
         _check(code, "flash_attention_static")
         return out
-    _check(_lib().tl_flash_attention(
+    _check(_lib().tl_flash_attention_masked(
         _ptr(q, 16), c_int64(q.stride(0)), _ptr(k_cache, 16), _ptr(v_cache, 16), _ptr(block_tables),
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out, 8), c_int64(out.stride(0)), _ptr(part_o), _ptr(part_ml), c_int(n_tiles), c_int(T),
         c_int(num_heads), c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale),
-        c_int(window), c_int(_attn_flags(sink, q, out)), c_int(n_splits), _ptr(cos), _ptr(sin),
+        c_int(window), c_int(keep), c_float(softcap), c_int(_attn_flags(sink, q, out)), c_int(n_splits), _ptr(cos), _ptr(sin),
         c_int(1 if fused_rope is not None else 0), _stream()), "flash_attention")
     return out
 
@@ -895,7 +900,8 @@ def prefill_tile_waves(num_tokens: int, num_heads: int, num_kv_heads: int) -> in
 def flash_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
                   tiles, positions: torch.Tensor, out: torch.Tensor, num_heads: int, num_kv_heads: int,
                   head_dim: int, scale: float, window: int = 0, tile_waves: int = 8, n_splits: int = 1,
-                  scratch: Optional[torch.Tensor] = None, sink: bool = False) -> torch.Tensor:
+                  scratch: Optional[torch.Tensor] = None, sink: bool = False, keep: int = 0,
+                  softcap: float = 0.0) -> torch.Tensor:
     """`flash_attention` arranged for prompt portions: `tiles` are groups of at most
     tile_waves * (16 // (heads / kv_heads)) consecutive tokens of one request, and a key or value
     row is staged once per such group.  tile_waves is PREFILL_TILES (8), or 4 for steps with few
@@ -945,7 +951,8 @@ def flash_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out, 16 if out.dtype == torch.float32 else 8), c_int64(out.stride(0)), _ptr(part_o, 16), _ptr(part_ml), c_int(n_tiles), c_int(T),
         c_int(num_heads), c_int(num_kv_heads),
-        c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(_attn_flags(sink, q, out)), c_int(tile_waves), c_int(n_splits),
+        c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_int(_attn_flags(sink, q, out)), c_int(tile_waves),
+        c_int(n_splits),
         _stream()), "flash_prefill")
     return out
 
@@ -1111,6 +1118,24 @@ def cast_rows(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     if not (x.dtype == torch.float32 and x.is_contiguous() and out.is_contiguous() and out.shape == x.shape):
         _fail("cast_rows takes contiguous operands of one shape, the input in float32")
     _check(_lib().tl_cast_rows(_ptr(x), _ptr(out), c_int64(x.numel()), c_int(_dt(out)), _stream()), "cast_rows")
+    return out
+
+
+def gelu_table_rows(gate: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, off: int, dim: int,
+                    out: torch.Tensor) -> torch.Tensor:
+    """out[t, j] = gelu(gate[t, j]) * table[tokens[t], off + j] for j < dim (gelu in its tanh form), zeros in out's
+    further columns; gate float32 [T, >= dim], table [vocab, >= off + dim] and out [T, >= dim] of one type."""
+    _dev(gate, tokens, table, out)
+    _rows_2d(gate, "gelu_table_rows gate")
+    _i32(tokens)
+    T = tokens.numel()
+    _need(gate.dtype == torch.float32 and gate.shape[0] == T and gate.shape[1] >= dim > 0 and off >= 0
+          and table.dim() == 2 and table.is_contiguous() and off + dim <= table.shape[1] and out.dim() == 2
+          and out.is_contiguous() and out.shape[0] == T and out.shape[1] >= dim and out.dtype == table.dtype,
+          "gelu_table_rows: shapes do not fit")
+    _check(_lib().tl_gelu_table_rows(_ptr(gate), c_int64(gate.stride(0)), _ptr(tokens), _ptr(table), c_int64(table.shape[1]),
+                                     c_int(off), _ptr(out), c_int(T), c_int(dim), c_int(out.shape[1]), c_int(_dt(table)),
+                                     _stream()), "gelu_table_rows")
     return out
 
 
@@ -1479,18 +1504,20 @@ def delta_prepare(p: torch.Tensor, conv_off: int, b_off: int, a: torch.Tensor, c
 
 
 def conv_state_update(p: torch.Tensor, conv_off: int, channels: int, state: torch.Tensor, saved_off: int,
-                      cu_seqlens: torch.Tensor, state_slots: torch.Tensor, taps: int) -> None:
+                      cu_seqlens: torch.Tensor, state_slots: torch.Tensor, taps: int,
+                      bias: Optional[torch.Tensor] = None) -> None:
     """The saved inputs of the convolutions after this step: per request and channel the last
-    taps - 1 of (what was saved, the step's inputs), oldest first."""
-    _dev(p, state, cu_seqlens, state_slots)
+    taps - 1 of (what was saved, the step's inputs plus `bias`, float32 per channel), oldest first."""
+    _dev(p, state, cu_seqlens, state_slots, bias)
+    _f32_vec(bias, channels, "conv_state_update bias")
     _rows_2d(p, "projections")
     _i32(cu_seqlens, state_slots)
     R = state_slots.numel()
-    if not (state.dtype == torch.float32 and state.dim() == 2 and state.is_contiguous() and cu_seqlens.numel() == R + 1
+    if not (state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and cu_seqlens.numel() == R + 1
             and saved_off + channels * (taps - 1) <= state.shape[1] and conv_off + channels <= p.shape[1]
             and 1 <= taps <= DELTA_MAX_TAPS):
         _fail("conv_state_update: shapes do not fit")
-    _check(_lib().tl_conv_state_update(_ptr(p), c_int64(p.stride(0)), c_int(conv_off), c_int(channels), _ptr(state),
+    _check(_lib().tl_conv_state_update(_ptr(p), c_int64(p.stride(0)), c_int(conv_off), c_int(channels), _ptr(bias), _ptr(state),
                                        c_int64(state.stride(0)), c_int64(saved_off), _ptr(cu_seqlens),
                                        _ptr(state_slots), c_int(R), c_int(taps), c_int(_dt(p)), _stream()),
            "conv_state_update")
@@ -1829,6 +1856,93 @@ def time_mix_recurrence(x: torch.Tensor, r_off: int, k_off: int, v_off: int, w_o
     return o
 
 
+# ---------------------------- linear recurrences with one decay per head and token (csrc/linear_recurrence.hip)
+LINEAR_MAX_DIM = 256            # rows of a head's state
+LINEAR_DECODE_MAX_VDIM = 256    # value columns the one-token kernel takes
+
+
+def ssd_prepare(p: torch.Tensor, conv_off: int, dt_off: int, conv: ShortConv, conv_b: Optional[torch.Tensor],
+                a_log: torch.Tensor, dt_bias: torch.Tensor, x: torch.Tensor, dt_col: int, a_col: int) -> None:
+    """x[t] = [silu(conv(p[t, conv_off ..]) + conv_b): channels | c = softplus(p[t, dt_off + h] + dt_bias[h]), from column
+    dt_col | exp(-exp(a_log[h]) c), from a_col]; p and x float32."""
+    _dev(p, conv_b, a_log, dt_bias, x, conv.w, conv.state, conv.req_of_token, conv.cu_seqlens, conv.state_slots)
+    _rows_2d(p, "ssd_prepare input")
+    _rows_2d(x, "ssd_prepare output")
+    _i32(conv.req_of_token, conv.cu_seqlens, conv.state_slots)
+    T, heads = p.shape[0], a_log.numel()
+    channels, taps = conv.w.shape
+    _f32_vec(conv.w, channels * taps, "ssd_prepare taps")
+    _f32_vec(conv_b, channels, "ssd_prepare convolution bias")
+    _f32_vec(a_log, heads, "A_log")
+    _f32_vec(dt_bias, heads, "dt_bias")
+    _need(p.dtype == x.dtype == torch.float32 and x.shape[0] == T and conv_off + channels <= p.shape[1]
+          and dt_off + heads <= p.shape[1] and channels <= dt_col and dt_col + heads <= a_col and a_col + heads <= x.shape[1]
+          and 1 <= taps <= DELTA_MAX_TAPS and conv.req_of_token.numel() == T
+          and conv.cu_seqlens.numel() == conv.state_slots.numel() + 1 and conv.state.dtype == torch.float32
+          and conv.state.dim() == 2 and conv.state.stride(1) == 1
+          and conv.saved_off + channels * (taps - 1) <= conv.state.shape[1], "ssd_prepare: shapes do not fit")
+    _check(_lib().tl_ssd_prepare(_ptr(p), c_int64(p.stride(0)), c_int(conv_off), c_int(dt_off), _ptr(conv.w), _ptr(conv_b),
+                                 _ptr(a_log), _ptr(dt_bias), _ptr(conv.state), c_int64(conv.state.stride(0)),
+                                 c_int64(conv.saved_off), _ptr(conv.req_of_token), _ptr(conv.cu_seqlens),
+                                 _ptr(conv.state_slots), _ptr(x), c_int64(x.stride(0)), c_int(dt_col), c_int(a_col), c_int(T),
+                                 c_int(channels), c_int(heads), c_int(taps), c_int(1 if conv.save_single else 0), _stream()),
+           "ssd_prepare")
+
+
+def linear_recurrence(x: torch.Tensor, q_off: int, k_off: int, v_off: int, state: torch.Tensor, cu_seqlens: torch.Tensor,
+                      state_slots: torch.Tensor, out: torch.Tensor, heads: int, groups: int, dim: int, vdim: int,
+                      decay: Optional[torch.Tensor] = None, a_off: int = -1, c_off: int = -1,
+                      skip: Optional[torch.Tensor] = None, silu: bool = False, single: bool = False) -> torch.Tensor:
+    """Walks every request's tokens of this step through S <- a S + k (c v)^T; o = S^T q + D v, S [heads, dim, vdim] at the
+    start of the request's state row.  Row t of x (float32) holds q and k (groups x dim, from q_off and k_off; head n
+    reads group n // (heads / groups)), v (heads x vdim, from v_off), c (per head, from c_off; negative: 1) and a (per
+    head, from a_off; negative: `decay`[head], float32).  skip: D per head, or None.  silu: q, k and v are SiLU's inputs.
+    single: no request brings more than one token."""
+    _dev(x, state, cu_seqlens, state_slots, out, decay, skip)
+    _rows_2d(x, "linear_recurrence operands")
+    _i32(cu_seqlens, state_slots)
+    R, T = state_slots.numel(), x.shape[0]
+    _need(0 < dim <= LINEAR_MAX_DIM and heads > 0 and groups > 0 and heads % groups == 0 and vdim > 0,
+          f"linear_recurrence: heads a multiple of groups, at most {LINEAR_MAX_DIM} rows a head")
+    _f32_vec(out, T * heads * vdim, "linear_recurrence output")
+    _f32_vec(decay, heads, "linear_recurrence decay")
+    _f32_vec(skip, heads, "linear_recurrence skip")
+    _need(x.dtype == torch.float32 and min(q_off, k_off, v_off) >= 0 and max(q_off, k_off) + groups * dim <= x.shape[1]
+          and v_off + heads * vdim <= x.shape[1] and max(a_off, c_off) + heads <= x.shape[1]
+          and (a_off >= 0 or decay is not None), "linear_recurrence: columns do not fit")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
+          and heads * dim * vdim <= state.shape[1] and cu_seqlens.numel() == R + 1,
+          "linear_recurrence: the state is float32 [slots, >= heads * dim * vdim]")
+    decode = (single and vdim % 4 == 0 and vdim <= LINEAR_DECODE_MAX_VDIM and state.stride(0) % 4 == 0
+              and state.data_ptr() % 16 == 0)
+    _check(_lib().tl_linear_recurrence(_ptr(x), c_int64(x.stride(0)), c_int(q_off), c_int(k_off), c_int(v_off), c_int(c_off),
+                                       c_int(a_off), _ptr(decay), _ptr(skip), _ptr(state), c_int64(state.stride(0)),
+                                       _ptr(cu_seqlens), _ptr(state_slots), _ptr(out), c_int(R), c_int(heads), c_int(groups),
+                                       c_int(dim), c_int(vdim), c_int(1 if silu else 0), c_int(1 if decode else 0), _stream()),
+           "linear_recurrence")
+    return out
+
+
+def group_norm_gate(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, out: torch.Tensor, groups: int, eps: float,
+                    gate_kind: str = "sigmoid", gate_first: bool = False, scale: float = 1.0) -> torch.Tensor:
+    """Rows in `groups` equal parts, each divided by its own root mean square, times weight (one number a column) and
+    scale; the gate act(gate) multiplies the row ahead of the norm (`gate_first`) or behind it, act "sigmoid" or "silu"
+    (g * sigmoid(g)).  o float32 [T, width] contiguous, gate float32 [T, width] (a view into wider rows is fine)."""
+    _dev(o, weight, gate, out)
+    T, width = out.shape
+    _f32_vec(o, T * width, "group_norm_gate input")
+    _f32_vec(weight, width, "group_norm_gate weight")
+    _rows_2d(gate, "group_norm_gate gate")
+    _need(gate_kind in ("sigmoid", "silu"), f"group_norm_gate: unknown gate {gate_kind!r}")
+    _need(gate.dtype == torch.float32 and tuple(gate.shape) == (T, width) and out.is_contiguous() and width % groups == 0,
+          "group_norm_gate: gate and output are [T, width], the parts equal")
+    _check(_lib().tl_group_norm_gate(_ptr(o), _ptr(weight), _ptr(gate), c_int64(gate.stride(0)), _ptr(out), c_int(T),
+                                     c_int(width), c_int(groups), c_float(eps), c_int(1 if gate_kind == "silu" else 0),
+                                     c_int(1 if gate_first else 0), c_float(scale), c_int(_dt(out)), _stream()),
+           "group_norm_gate")
+    return out
+
+
 def tanh_rows(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     """out = tanh(x); x float32 [T, n] (a row stride is fine), out contiguous [T, n] of the engine's type."""
     _dev(x, out)
@@ -2084,15 +2198,24 @@ def row_dot_sigmoid(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> torc
 MOE_MAX_ROUTED = 1024       # experts the router kernel takes (csrc/moe.hip)
 
 
+MOE_SCORES = ("softmax", "sigmoid")
+
+
 def moe_route(z: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, groups: int = 1, keep: int = 1,
-              scale: float = 1.0, bias: Optional[torch.Tensor] = None) -> None:
+              scale: float = 1.0, bias: Optional[torch.Tensor] = None, score: str = "softmax",
+              correction: Optional[torch.Tensor] = None, group_top2: bool = False, normalize: bool = True) -> None:
     """A router over the logits z (float32 [T, E], rows may be wider apart; `bias`, float32 [E], is added to every
     row if given): scores s = softmax(z) over all experts;
     the experts lie in `groups` equal runs of neighbours, a run's score is its largest, and only experts of the
     `keep` best runs may be chosen (groups <= 1: all may); ids[t] (int32 [T, top]) names the `top` largest scores
     among those, largest first (equal scores: the lower index first), and weights[t] (float32 [T, top]) =
-    their scores / (their sum + 1e-20) * scale."""
-    _dev(z, ids, weights)
+    their scores / (their sum + 1e-20) * scale.
+    Options: `score` "sigmoid" (s = sigmoid(z)); `correction` (float32 [E]) is added to the scores wherever experts or
+    runs are chosen, never to the weights; `group_top2`: a run's score is the sum of its two largest; `normalize` False:
+    the weights are the scores * scale."""
+    _dev(z, ids, weights, correction)
+    _f32_vec(correction, z.shape[1], "moe_route correction")
+    _need(score in MOE_SCORES, f"moe_route: scores {score!r} are not built")
     _rows_2d(z, "moe_route logits")
     T, E = z.shape
     top = ids.shape[1] if ids.dim() == 2 else 0
@@ -2108,7 +2231,9 @@ def moe_route(z: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, groups:
         _need(E % groups == 0 and 0 < keep <= groups and top <= keep * (E // groups),
               "moe_route: equal groups, 1 to `groups` of them kept, holding at least `top` experts")
     _check(_lib().tl_moe_route(_ptr(z), c_int64(z.stride(0)), _ptr(bias), _ptr(ids), _ptr(weights), c_int(T), c_int(E), c_int(top),
-                               c_int(groups), c_int(keep), c_float(scale), _stream()), "moe_route")
+                               c_int(groups), c_int(keep), c_float(scale), c_int(MOE_SCORES.index(score)),
+                               _ptr(correction), c_int(1 if group_top2 else 0), c_int(1 if normalize else 0), _stream()),
+           "moe_route")
 
 
 def activate_rows(x: torch.Tensor, out: torch.Tensor, act: Optional[str]) -> torch.Tensor:
@@ -2162,6 +2287,21 @@ def embedding_pairs(tokens: torch.Tensor, positions: torch.Tensor, req_of_token:
 
 
 # ------------------------------------------- the general step between the q/k/v product and the attention kernel
+@dataclass
+class ShortConv:
+    """A short causal convolution per channel inside another step: taps w [channels, taps] (float32, the last column the
+    current token's), saved inputs in the `state` rows at saved_off, [channel][taps - 1], oldest first.  save_single (no
+    request of the step brings more than one token): the step brings the saved inputs up to date itself; else
+    `conv_state_update` has to follow."""
+    w: torch.Tensor
+    state: torch.Tensor
+    saved_off: int
+    req_of_token: torch.Tensor
+    cu_seqlens: torch.Tensor
+    state_slots: torch.Tensor
+    save_single: bool = False
+
+
 ATTN_PREPARE_MAX_DIM = 256      # numbers a unit (one map of one head) may have, and the padded head size D
 
 
@@ -2169,7 +2309,8 @@ def attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], norm_w: Optional
                  cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], slot_mapping: Optional[torch.Tensor],
                  q_out: torch.Tensor, k_caches, v_cache: Optional[torch.Tensor], heads: int, kv_heads: int, maps: int,
                  dim: int, vdim: int, v_off: int, rot: int = 0, pairing: str = "half", whole_norm: bool = False,
-                 unit_norm: bool = False, eps: float = 1e-6, q_temp=None) -> None:
+                 unit_norm: bool = False, eps: float = 1e-6, q_temp=None, conv: Optional["ShortConv"] = None,
+                 head_w: Optional[torch.Tensor] = None) -> None:
     """From the float32 product p [T, >= v_off + kv_heads * vdim] = [q: heads * maps units of dim | k: kv_heads * maps
     units | v: kv_heads heads of vdim, from column v_off]: bias added (float32 over [q | k | v]), an RMS norm over ALL of
     a token's q numbers (and all of its k numbers) with weights norm_w (float32 over [q | k], `whole_norm`), the first
@@ -2177,7 +2318,11 @@ def attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], norm_w: Optional
     (`unit_norm`), queries times 1 + coef * ln(floor((pos + 1) / every) + 1) (`q_temp` = (coef, every)).  Queries leave
     as q_out [maps, T, heads * D] rounded to the engine's type, keys of map m go to k_caches[m] and values to v_cache
     (pages [blocks, kv_heads, block, D]) at the tokens' slots; D is q_out's head size, what lies beyond dim or vdim is
-    written as zeros.  slot_mapping None (or a negative slot) stores nothing."""
+    written as zeros.  slot_mapping None (or a negative slot) stores nothing.
+    conv: behind the bias every channel of q, k and v runs through a short causal convolution, its inputs ahead of a
+    request's first token of the step kept in the request's state row (v_off is then q's and k's columns: the channels
+    are the columns).  head_w (float32 [2 * dim], queries' weights then keys'): every unit is divided by its own root
+    mean square and multiplied by them, ahead of the rotation."""
     k_caches = tuple(k_caches) if k_caches is not None else ()
     _dev(p, bias, norm_w, positions, cos, sin, slot_mapping, q_out, v_cache, *k_caches)
     _rows_2d(p, "attn_prepare input")
@@ -2218,6 +2363,25 @@ def attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], norm_w: Optional
     coef, every = (float(q_temp[0]), int(q_temp[1])) if q_temp else (0.0, 0)
     _need(every >= 0, "attn_prepare: the temperature's step is positive")
     store = slot_mapping is not None
+    cv = (c_void_p(0), c_int(0), c_int(0), c_void_p(0), c_int64(0), c_int64(0), c_void_p(0), c_void_p(0), c_void_p(0))
+    if conv is not None:
+        channels = q_size + k_size + v_size
+        _dev(conv.w, conv.state, conv.req_of_token, conv.cu_seqlens, conv.state_slots)
+        _i32(conv.req_of_token, conv.cu_seqlens, conv.state_slots)
+        taps = conv.w.shape[1]
+        _f32_vec(conv.w, channels * taps, "attn_prepare convolution taps")
+        _need(not whole_norm and v_off == q_size + k_size, "attn_prepare: the convolution takes adjacent q, k and v columns "
+              "and no norm over whole projections")
+        _need(1 <= taps <= DELTA_MAX_TAPS and conv.req_of_token.numel() == T
+              and conv.cu_seqlens.numel() == conv.state_slots.numel() + 1 and conv.state.dtype == torch.float32
+              and conv.state.dim() == 2 and conv.state.stride(1) == 1
+              and conv.saved_off + channels * (taps - 1) <= conv.state.shape[1], "attn_prepare: the convolution's shapes do not fit")
+        cv = (_ptr(conv.w), c_int(taps), c_int(1 if conv.save_single else 0), _ptr(conv.state), c_int64(conv.state.stride(0)),
+              c_int64(conv.saved_off), _ptr(conv.req_of_token), _ptr(conv.cu_seqlens), _ptr(conv.state_slots))
+    if head_w is not None:
+        _dev(head_w)
+        _need(not whole_norm, "attn_prepare: one norm ahead of the rotation, per head or over the whole projection")
+        _f32_vec(head_w, 2 * dim, "attn_prepare head norm weights")
     _check(_lib().tl_attn_prepare(_ptr(p), c_int64(p.stride(0)), _ptr(bias), _ptr(norm_w), _ptr(positions), _ptr(cos),
                                   _ptr(sin), _ptr(slot_mapping), _ptr(q_out), c_int64(q_out.stride(1)),
                                   c_int64(q_out.stride(0)), _ptr(k_caches[0] if store else None),
@@ -2225,7 +2389,8 @@ def attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], norm_w: Optional
                                   c_int(T), c_int(heads), c_int(kv_heads), c_int(maps), c_int(dim), c_int(vdim), c_int(D),
                                   c_int(v_off), c_int(rot), c_int(ROPE_PAIRINGS.index(pairing)),
                                   c_int(1 if whole_norm else 0), c_int(1 if unit_norm else 0), c_float(eps), c_float(coef),
-                                  c_int(every), c_int(block_size), c_int(_dt(q_out)), _stream()), "attn_prepare")
+                                  c_int(every), c_int(block_size), *cv, _ptr(head_w), c_int(_dt(q_out)), _stream()),
+           "attn_prepare")
 
 
 ATTN_GATES = {None: 0, "head": 1, "element": 2}

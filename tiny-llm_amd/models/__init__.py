@@ -1,2 +1,2 @@
-from . import llama, lufazen, fofapel, gesutar, vevapel  # noqa: F401  (register LlamaForCausalLM, Lufazen, Fofapel, Gesutar, Vevapel)
+from . import llama, lufazen, fofapel, gesutar, vevapel, mogutar  # noqa: F401  (register LlamaForCausalLM, Lufazen, Fofapel, Gesutar, Vevapel, Mogutar)
 from .decoder import Decoder

@@ -19,8 +19,8 @@ import torch
 
 from ..kernels import ops
 from .norm import LazyNorm
-from .base import (CacheSpec, CacheTensor, LayerCache, Mixer, POSITION_ENCODINGS, WeightSpec, project_into_residual,
-                   register_mixer)
+from .base import (CacheSpec, CacheTensor, LayerCache, Mixer, POSITION_ENCODINGS, StateSpec, WeightSpec,
+                   project_into_residual, register_mixer)
 
 
 class Attention(Mixer):
@@ -43,6 +43,7 @@ class Attention(Mixer):
         ops.check_linear_sizes(dtype, self.hidden_size, f"{prefix}: hidden_size")
         ops.check_linear_sizes(dtype, self.num_heads * self.head_dim, f"{prefix}: num_heads * head_dim")
         self.window = int(window or 0)
+        self.keep, self.softcap = 0, 0.0
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(self.head_dim)
         pos = dict(position or {"kind": "none"})
         kind = pos.pop("kind")
@@ -99,13 +100,15 @@ class Attention(Mixer):
         """attn <- attention of the step's query rows q [T, heads * head_dim] over the cache, by the kernel that
         takes this step's shape.  sink: one more term exp(0) in every softmax's denominator.  `self.window`: 0
         (every earlier key), n > 0 (the last n positions) or -n (the row's own run of n positions, runs counted
-        from position 0: a chunked mask)."""
+        from position 0: a chunked mask); the request's first `self.keep` positions are seen in any case.
+        `self.softcap` > 0: scores s become softcap * tanh(s / softcap)."""
+        mask = {"sink": sink, "keep": self.keep if self.window else 0, "softcap": self.softcap}
         T, device = q.shape[0], q.device
         group = self.num_heads // self.num_kv_heads
         flash = ops.flash_attention_supported(self.dtype, self.num_heads, self.num_kv_heads, self.head_dim)
         # the keys one row walks at most: a window bounds them whatever the context (the kernels begin at the
         # window's first key tile)
-        span = min(ctx.max_seq_len, abs(self.window) + 63) if self.window else ctx.max_seq_len
+        span = min(ctx.max_seq_len, abs(self.window) + 63 + -(-self.keep // 64) * 64) if self.window else ctx.max_seq_len
         if flash and ctx.max_q_len > 1:
             # prompt portions: many query rows share each staged key tile
             waves = ops.prefill_tile_waves(T, self.num_heads, self.num_kv_heads)
@@ -118,7 +121,7 @@ class Attention(Mixer):
                                       torch.float32, device)
             ops.flash_prefill(q, cache.k, cache.v, ctx.block_tables[cache.group], tiles, ctx.positions, attn,
                               self.num_heads, self.num_kv_heads, self.head_dim, self.scale, self.window, waves,
-                              n_splits, scratch, sink=sink)
+                              n_splits, scratch, **mask)
         elif flash:
             # decoding: one token per request, its keys split over the waves of a workgroup (and over
             # workgroups when the context is long)
@@ -127,7 +130,7 @@ class Attention(Mixer):
             n_splits, scratch = self._splits(span, T, device)
             ops.flash_attention(q, cache.k, cache.v, ctx.block_tables[cache.group], tiles, ctx.positions, attn,
                                 self.num_heads, self.num_kv_heads, self.head_dim, self.scale, self.window,
-                                n_splits, scratch, fused_rope=fused_rope, sink=sink)
+                                n_splits, scratch, fused_rope=fused_rope, **mask)
         elif ops.attention_f32_supported(self.dtype, self.num_heads, self.num_kv_heads, self.head_dim) \
                 and q.stride(0) % 4 == 0:
             # true float32 on the matrix cores; one fixed merge tree, so the same bits whatever the batch
@@ -140,11 +143,11 @@ class Attention(Mixer):
                                       torch.float32, device)
             ops.attention_f32(q, cache.k, cache.v, ctx.block_tables[cache.group], tiles, ctx.positions, attn,
                               self.num_heads, self.num_kv_heads, self.head_dim, self.scale, self.window, n_chunks,
-                              scratch, sink=sink)
+                              scratch, **mask)
         else:
             ops.paged_attention(q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.req_of_token,
                                 ctx.positions, attn, self.num_heads, self.num_kv_heads, self.head_dim,
-                                self.scale, self.window, sink=sink)
+                                self.scale, self.window, **mask)
         return attn
 
     def _splits(self, span: int, T: int, device):
@@ -264,8 +267,15 @@ class GatedAttention(Attention):
         q (and k) divided by the root mean square over ALL of the token's q (k) numbers, times a weight each
                                                                                         `qk_norm="whole"`
         q, k rotated on the first rotary_dim dims (`position`, either pairing); `qk_norm="unit"`: each head by itself
+        q, k and v, each channel by itself, through a causal convolution of `conv_taps` taps behind the biases, ahead of
+        everything else (y_t = sum_j w_j u_(t - taps + 1 + j), zeros ahead of the request's first token; its last taps - 1
+        inputs are per-request state)
+        q (and k) divided by the root mean square over each head, times a weight per dim that the heads share, ahead of
+        the rotation                                                                    `qk_norm="head"`
         q times 1 + coef ln(floor((pos + 1) / every) + 1)                              `q_temp=(coef, every)`
-        keys seen: all earlier ones, the last `window`, or those of the row's own run of `chunk` positions
+        keys seen: all earlier ones, the last `window` (and the request's first `keep_first`), or those of the row's own
+        run of `chunk` positions
+        scores s become softcap * tanh(s / softcap)                                    `softcap`
         `maps=2`: two score maps per head (q and k hold [map 1 | map 2] head by head) over the same values,
                   o = a1 - lambda a2, lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff (a scalar of the layer)
         o divided by its root mean square over the head, no weight (`sub_norm`), times `out_scale`
@@ -287,8 +297,9 @@ class GatedAttention(Attention):
                  value_dim: int = None, position: dict = None, window: int = 0, chunk: int = 0, scale: float = None,
                  bias: bool = False, out_bias: bool = None, qk_norm: str = None, eps: float = 1e-6, q_temp=None,
                  maps: int = 1, diff: float = 0.0, sub_norm: bool = False, out_scale: float = 1.0, gate: str = None,
+                 conv_taps: int = 0, keep_first: int = 0, softcap: float = 0.0,
                  names: Dict[str, str] = None, bias_suffix: str = ".b", norm_suffix: str = ".norm",
-                 max_position: int = 0):
+                 conv_suffix: str = ".conv", max_position: int = 0):
         dim, vdim = int(head_dim), int(value_dim if value_dim is not None else head_dim)
         if dim <= 0 or vdim <= 0:
             raise ValueError(f"{prefix}: head_dim and value_dim must be positive")
@@ -305,8 +316,14 @@ class GatedAttention(Attention):
             scale = 1.0 / math.sqrt(dim)
         self.scale = float(scale)
         self.qk_dim, self.value_dim, self.chunk = dim, vdim, int(chunk or 0)
-        if qk_norm not in (None, "unit", "whole"):
-            raise ValueError(f"{prefix}: qk_norm is None, 'unit' or 'whole', got {qk_norm!r}")
+        if qk_norm not in (None, "unit", "whole", "head"):
+            raise ValueError(f"{prefix}: qk_norm is None, 'unit', 'whole' or 'head', got {qk_norm!r}")
+        self.keep, self.softcap, self.taps = int(keep_first or 0), float(softcap or 0.0), int(conv_taps or 0)
+        if self.keep < 0 or self.softcap < 0 or (self.keep and not window):
+            raise ValueError(f"{prefix}: keep_first and softcap are not negative, and kept tokens lie behind a window")
+        if self.taps and (not (1 <= self.taps <= ops.DELTA_MAX_TAPS) or qk_norm == "whole"):
+            raise ValueError(f"{prefix}: a convolution of 1 to {ops.DELTA_MAX_TAPS} taps, and no norm over the whole projection "
+                             f"behind it, got {conv_taps} and {qk_norm!r}")
         if maps not in (1, 2):
             raise ValueError(f"{prefix}: one or two score maps, got {maps}")
         if gate not in ops.ATTN_GATES:
@@ -325,7 +342,7 @@ class GatedAttention(Attention):
         n = {k: k for k in ("q", "k", "v", "g", "o", "lq1", "lk1", "lq2", "lk2")}
         n.update(names or {})
         self.names = {k: f"{prefix}.{v}" for k, v in n.items()}
-        self.bias_suffix, self.norm_suffix = bias_suffix, norm_suffix
+        self.bias_suffix, self.norm_suffix, self.conv_suffix = bias_suffix, norm_suffix, conv_suffix
         H, G = self.num_heads, self.num_kv_heads
         self.q_cols, self.k_cols, self.v_cols = H * self.maps * dim, G * self.maps * dim, G * vdim
         self.q_size = H * D                             # one map's query rows as the attention kernels see them
@@ -336,7 +353,7 @@ class GatedAttention(Attention):
         self.out_cols = H * vdim
         self.out_tail = 8 if self.out_bias else 0       # a column of ones for the bias, zeros up to a multiple of 8
         ops.check_linear_sizes(dtype, self.out_cols, f"{prefix}: num_heads * value_dim")
-        self.w_in = self.b_in = self.norm_w = self.w_o = None
+        self.w_in = self.b_in = self.norm_w = self.head_w = self.conv_w = self.w_o = None
         self.lam = 0.0
 
     def weights(self) -> List[WeightSpec]:
@@ -349,6 +366,11 @@ class GatedAttention(Attention):
         if self.qk_norm == "whole":
             out += [WeightSpec(n["q"] + self.norm_suffix, (self.q_cols,), role="vector", init="ones"),
                     WeightSpec(n["k"] + self.norm_suffix, (self.k_cols,), role="vector", init="ones")]
+        if self.qk_norm == "head":
+            out += [WeightSpec(n[k] + self.norm_suffix, (self.qk_dim,), role="vector", init="ones") for k in ("q", "k")]
+        if self.taps:
+            out += [WeightSpec(n[k] + self.conv_suffix, (cols, self.taps), role="vector", init="normal")
+                    for k, cols in (("q", self.q_cols), ("k", self.k_cols), ("v", self.v_cols))]
         if self.maps == 2:
             out += [WeightSpec(n[k], (self.qk_dim,), role="vector", init="normal") for k in ("lq1", "lk1", "lq2", "lk2")]
         if self.gate:
@@ -373,6 +395,10 @@ class GatedAttention(Attention):
             self.b_in = torch.cat([f32(tensors[n[k] + bs]) for k in ("q", "k", "v")]).contiguous()
         if self.qk_norm == "whole":
             self.norm_w = torch.cat([f32(tensors[n[k] + self.norm_suffix]) for k in ("q", "k")]).contiguous()
+        if self.qk_norm == "head":
+            self.head_w = torch.cat([f32(tensors[n[k] + self.norm_suffix]) for k in ("q", "k")]).contiguous()
+        if self.taps:
+            self.conv_w = torch.cat([f32(tensors[n[k] + self.conv_suffix]) for k in ("q", "k", "v")]).contiguous()
         w_o = tensors[n["o"]]
         if self.out_bias:
             wide = torch.zeros((self.hidden_size, self.out_cols + self.out_tail), dtype=self.dtype, device=dev)
@@ -390,7 +416,14 @@ class GatedAttention(Attention):
         t = (self.num_kv_heads, self.head_dim)
         kind = "window" if self.window > 0 else "full"
         names = ("k", "k2", "v") if self.maps == 2 else ("k", "v")
-        return CacheSpec(tuple(CacheTensor(name, t, 1) for name in names), kind, max(self.window, 0))
+        return CacheSpec(tuple(CacheTensor(name, t, 1) for name in names), kind, max(self.window, 0), self.keep)
+
+    def state_spec(self) -> Optional[StateSpec]:
+        if self.taps <= 1:
+            return None
+        # the convolutions' last inputs, [channel][taps - 1]; rows a multiple of four floats
+        channels = self.q_cols + self.k_cols + self.v_cols
+        return StateSpec((-(-channels * (self.taps - 1) // 4) * 4,), torch.float32)
 
     def forward(self, h, ctx, cache: LayerCache, state, residual):
         T, dev, H = h.shape[0], h.device, self.num_heads
@@ -401,12 +434,20 @@ class GatedAttention(Attention):
         pairing = getattr(self.position, "pairing", "half")
         q = ops.scratch("q_prepared", (self.maps, T, self.q_size), self.dtype, dev)
         write = cache.write
+        conv = None
+        channels = self.v_off + self.v_cols
+        if self.taps:
+            # a step of single tokens brings the saved inputs up to date in the same kernel
+            conv = ops.ShortConv(self.conv_w, state if state is not None else ops.scratch("no_state", (1, 4), torch.float32, dev),
+                                 0, ctx.req_of_token, ctx.cu_seqlens_q, ctx.state_slots, ctx.max_q_len == 1)
         k_caches = [cache.tensors["k"]] + ([cache.tensors["k2"]] if self.maps == 2 else [])
         ops.attn_prepare(p, self.b_in, self.norm_w, ctx.positions, cos, sin,
                          ctx.slot_mappings[cache.group] if write else None, q, k_caches if write else None,
                          cache.tensors["v"] if write else None, H, self.num_kv_heads, self.maps, self.qk_dim,
                          self.value_dim, self.v_off, rot, pairing, self.qk_norm == "whole", self.qk_norm == "unit",
-                         self.eps, self.q_temp)
+                         self.eps, self.q_temp, conv, self.head_w)
+        if self.taps > 1 and ctx.max_q_len > 1:
+            ops.conv_state_update(p, 0, channels, state, 0, ctx.cu_seqlens_q, ctx.state_slots, self.taps, self.b_in)
         outs = []
         for m in range(self.maps):
             # float32 whatever the engine's type: the maps' difference, the head's norm and the gates follow in float32

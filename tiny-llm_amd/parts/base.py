@@ -66,11 +66,12 @@ class CacheTensor:
 @dataclass(frozen=True)
 class CacheSpec:
     """What a mixer keeps per token, as a list of paged tensors.
-    kind "full" keeps every position, "window" the last `window` positions.
+    kind "full" keeps every position, "window" the last `window` positions and, for good, the first `keep`.
     Layers whose specs are equal share one block-id space and one block table per request."""
     tensors: Tuple[CacheTensor, ...]
     kind: str = "full"
     window: int = 0
+    keep: int = 0
 
     @classmethod
     def keys_and_values(cls, num_kv_heads: int, head_dim: int, kind: str = "full", window: int = 0) -> "CacheSpec":
@@ -79,7 +80,7 @@ class CacheSpec:
         return cls((CacheTensor("k", t, 1), CacheTensor("v", t, 1)), kind, int(window))
 
     def group_key(self):
-        return (self.kind, self.window, self.tensors)
+        return (self.kind, self.window, self.keep, self.tensors)
 
 
 @dataclass(frozen=True)

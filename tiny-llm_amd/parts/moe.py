@@ -17,6 +17,9 @@ and is added.  Tensor names below the prefix: e<i>.up|down, router, shared.up|do
 makes the experts gated units down(silu(gate(h)) * up(h)) (tensors e<i>.gate|up|down); `router_bias` adds a bias per
 expert to the router's logits (tensor router<bias_suffix>).  With one group and scale 1 the weights are the softmax
 over the chosen logits alone: exp(z_j) / sum over the chosen of exp(z_i), whatever the other experts' logits are.
+`score="sigmoid"` (s = sigmoid(z)); `correction` (tensor correction: a number per expert added to the scores wherever
+experts or runs are chosen, left out of the weights); `group_score="top2"` (a run's score is the sum of its two largest
+choice scores); `normalize=False` (an expert weighs s_j * scale).
 """
 from __future__ import annotations
 
@@ -142,7 +145,8 @@ class RoutedMoE(FeedForward):
 
     def __init__(self, prefix, dtype, device, *, hidden_size: int, num_experts: int, top: int, intermediate_size: int,
                  groups: int = 1, keep: int = 1, scale: float = 1.0, activation: str = "relu2",
-                 shared: Optional[dict] = None, router_bias: bool = False, bias_suffix: str = ".b"):
+                 shared: Optional[dict] = None, router_bias: bool = False, bias_suffix: str = ".b",
+                 score: str = "softmax", correction: bool = False, group_score: str = "max", normalize: bool = True):
         """shared: None, or {"intermediate_size": F} (optionally "activation") for the shared expert."""
         super().__init__(prefix, dtype, device)
         self.hidden_size, self.num_experts, self.top = int(hidden_size), int(num_experts), int(top)
@@ -160,7 +164,12 @@ class RoutedMoE(FeedForward):
             raise ValueError(f"{prefix}: activation {activation!r} is not built; known: relu2, swiglu")
         self.activation = activation
         self.router_bias, self.bias_suffix = bool(router_bias), bias_suffix
-        self.b_router = None
+        self.b_router = self.correction_w = None
+        if score not in ops.MOE_SCORES or group_score not in ("max", "top2"):
+            raise ValueError(f"{prefix}: scores are one of {ops.MOE_SCORES} and a group's score 'max' or 'top2', got "
+                             f"{score!r} and {group_score!r}")
+        self.correction = bool(correction)
+        self.route_options = {"score": score, "group_top2": group_score == "top2", "normalize": bool(normalize)}
         ops.check_linear_sizes(dtype, self.hidden_size, f"{prefix}: hidden_size")
         ops.check_linear_sizes(dtype, self.intermediate_size, f"{prefix}: expert intermediate_size")
         self.shared = None
@@ -180,12 +189,16 @@ class RoutedMoE(FeedForward):
         out.append(WeightSpec(f"{p}.router", (self.num_experts, W)))
         if self.router_bias:
             out.append(WeightSpec(f"{p}.router{self.bias_suffix}", (self.num_experts,), role="vector", init="zeros"))
+        if self.correction:
+            out.append(WeightSpec(f"{p}.correction", (self.num_experts,), role="vector", init="zeros"))
         if self.shared is not None:
             out += self.shared.weights()
         return out
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         p, E = self.prefix, self.num_experts
+        if self.correction:
+            self.correction_w = tensors[f"{p}.correction"].to(torch.float32).contiguous()
         if self.gated:      # an expert's first product gives (gate_0, up_0, gate_1, up_1, ...): rows interleaved, as in
             # the dense gated layer, so that a product's epilogue sees each pair in one lane
             self.w_up = torch.stack([torch.stack([tensors[f"{p}.e{e}.gate"], tensors[f"{p}.e{e}.up"]], dim=1)
@@ -218,7 +231,8 @@ class RoutedMoE(FeedForward):
             Fs = self.shared.intermediate_size
             first = ops.scratch("moe_first", (T, self.shared_off + Fs), torch.float32, dev)
             ops.linear(h, self.w_first, first)
-            ops.moe_route(first[:, :E], ids, wts, self.groups, self.keep, self.scale, self.b_router)
+            ops.moe_route(first[:, :E], ids, wts, self.groups, self.keep, self.scale, self.b_router,
+                          correction=self.correction_w, **self.route_options)
             zs = ops.activate_rows(first[:, self.shared_off:], ops.scratch("ffn_gated", (T, Fs), self.dtype, dev),
                                    self.shared.activation)
             if residual is None:
@@ -228,7 +242,8 @@ class RoutedMoE(FeedForward):
         else:
             logits = ops.scratch("moe_router", (T, E), torch.float32, dev)
             ops.linear(h, self.w_router, logits)
-            ops.moe_route(logits, ids, wts, self.groups, self.keep, self.scale, self.b_router)
+            ops.moe_route(logits, ids, wts, self.groups, self.keep, self.scale, self.b_router,
+                          correction=self.correction_w, **self.route_options)
             base = residual                     # the experts are added to the stream itself (or stand alone)
         rows = T * top
         out = base if base is not None else ops.scratch("sublayer_out", (T, self.hidden_size), torch.float32, dev)

@@ -70,6 +70,7 @@ class RMSNorm(Norm):
         self.init = init if not self.offset else "zeros"
         self.tensor_name = f"{prefix}.{weight_name}" if weight_name else prefix
         self.weight: Optional[torch.Tensor] = None
+        self._weight_f32: Optional[torch.Tensor] = None     # for `add_normed`, of a weight kept in another type
 
     def weights(self) -> List[WeightSpec]:
         return [WeightSpec(self.tensor_name, (self.hidden_size,), role="vector", init=self.init)]
@@ -78,12 +79,17 @@ class RMSNorm(Norm):
         w = tensors[self.tensor_name]
         # offset + w is formed in float32: in bfloat16 the sum would lose what the stored weight says
         self.weight = (w.to(torch.float32) + self.offset).contiguous() if self.offset else w.contiguous()
+        self._weight_f32 = None
 
     def add_normed(self, y: torch.Tensor, x: torch.Tensor, scale: Optional[torch.Tensor] = None,
                    copy: Optional[torch.Tensor] = None) -> torch.Tensor:
         """x += scale * norm(y) for a norm that sits on a sublayer's output (y float32, one kernel);
         `copy` receives the new x in its own element type."""
-        w = self.weight if self.weight.dtype == torch.float32 else self.weight.to(torch.float32)
+        w = self.weight
+        if w.dtype != torch.float32:        # converted once, not at every step
+            if self._weight_f32 is None or self._weight_f32.device != w.device:
+                self._weight_f32 = w.to(torch.float32)
+            w = self._weight_f32
         return ops.norm_scale_add(y, w, self.eps, x, scale, copy)
 
     def lazy(self, x: torch.Tensor, rows: Optional[torch.Tensor] = None, prepared=None):

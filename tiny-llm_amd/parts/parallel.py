@@ -4,11 +4,12 @@ results, each times a constant of its own.
 A branch is any registered mixer that takes `out_scale` (it applies the constant itself, in float32,
 before its output product) and adds into the `residual` it is given: the first branch's output product
 writes the sum's buffer, every further one adds to it, so the sum costs no kernel of its own.  At most one
-branch may keep a paged cache and at most one a per-request state; they become the part's own.
+branch may keep a paged cache, which becomes the part's own; the branches' per-request states lie side by side
+in the part's state rows, and a branch is handed its own columns of them.
 """
 from __future__ import annotations
 
-from typing import Dict, List, Optional, Sequence
+from typing import Dict, List, Optional, Sequence, Tuple
 
 import torch
 
@@ -29,10 +30,22 @@ class ParallelMixer(Mixer):
             self.branches.append(MIXERS.get(b["kind"])(f"{prefix}.{b['name']}", dtype, device, **params))
         with_cache = [m for m in self.branches if m.cache_spec() is not None]
         with_state = [m for m in self.branches if m.state_spec() is not None]
-        if len(with_cache) > 1 or len(with_state) > 1:
-            raise ValueError(f"{prefix}: at most one branch may keep a cache and at most one a state")
+        if len(with_cache) > 1:
+            raise ValueError(f"{prefix}: at most one branch may keep a cache")
         self._cache_branch = with_cache[0] if with_cache else None
-        self._state_branch = with_state[0] if with_state else None
+        # one stateful branch: its state is the part's, whatever its shape; several: rows of one type side by side, each
+        # from a multiple of four elements (16-byte rows)
+        self._state_spec: Optional[StateSpec] = with_state[0].state_spec() if with_state else None
+        self._state_cols: Dict[int, Optional[Tuple[int, int]]] = {id(m): None for m in with_state}
+        if len(with_state) > 1:
+            specs = [m.state_spec() for m in with_state]
+            if any(len(s.shape) != 1 or s.dtype != specs[0].dtype for s in specs):
+                raise ValueError(f"{prefix}: branches that keep states side by side keep rows of one type")
+            at = 0
+            for m, s in zip(with_state, specs):
+                self._state_cols[id(m)] = (at, at + s.shape[0])
+                at = -(-(at + s.shape[0]) // 4) * 4
+            self._state_spec = StateSpec((at,), specs[0].dtype)
 
     @property
     def graph_safe(self) -> bool:
@@ -50,13 +63,18 @@ class ParallelMixer(Mixer):
         return self._cache_branch.cache_spec() if self._cache_branch is not None else None
 
     def state_spec(self) -> Optional[StateSpec]:
-        return self._state_branch.state_spec() if self._state_branch is not None else None
+        return self._state_spec
+
+    def _state_of(self, branch, state):
+        if id(branch) not in self._state_cols:
+            return None
+        cols = self._state_cols[id(branch)]
+        return state if cols is None else state[:, cols[0]:cols[1]]
 
     def forward(self, h, ctx, cache, state, residual):
         y = residual
         for m in self.branches:
-            y = m.forward(h, ctx, cache if m is self._cache_branch else None,
-                          state if m is self._state_branch else None, y)
+            y = m.forward(h, ctx, cache if m is self._cache_branch else None, self._state_of(m, state), y)
         return y
 
 
