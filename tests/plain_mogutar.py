@@ -3,7 +3,7 @@ equations with torch on the CPU (float64 unless told otherwise).  It shares no c
 engine: it reads config.json's own keys and the checkpoint's tensor names, keeps whole sequences
 (no cache, no pages, no state slots) and runs one request at a time.
 
-Notation: x [T, W] is the residual stream; weights are [out, in] and applied as h @ W.T; N is an RMS norm with
+Notation: x [T, W] is the residual stream; weights are [out, in]; N is an RMS norm with
 a weight; a layer is x <- x + N1(mixer(x)), then x <- x + N2(experts(x)), then x <- x + Ns(token input of x).
 """
 from __future__ import annotations
@@ -15,6 +15,17 @@ import torch
 
 
 # --------------------------------------------------------------------------- small pieces
+_round_to = None        # what `forward` was asked to round the products' operands to: (type, scale)
+
+
+def product(h, w):
+    """W h for every row of h; the operand is rounded first if the model runs with rounded operands."""
+    if _round_to is not None:
+        to, scale = _round_to
+        h = (h * scale).to(to).to(h.dtype) / scale
+    return h @ w.T
+
+
 def unit_rms(x, eps):
     """x / sqrt(mean(x^2) + eps) over the last axis."""
     return x / torch.sqrt((x * x).mean(dim=-1, keepdim=True) + eps)
@@ -98,7 +109,7 @@ def attention(h, w, m, eps, positions):
     scores inside a window that also keeps the first tokens."""
     T = h.shape[0]
     H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q, k, v = (causal_conv(h @ w[n].T + w[n + ".b"], w[n + ".conv"]) for n in ("q", "k", "v"))
+    q, k, v = (causal_conv(product(h, w[n]) + w[n + ".b"], w[n + ".conv"]) for n in ("q", "k", "v"))
     q = rms_norm(q.reshape(T, H, D), w["q.norm"], eps)
     k = rms_norm(k.reshape(T, G, D), w["k.norm"], eps)
     v = v.reshape(T, G, V)
@@ -109,7 +120,7 @@ def attention(h, w, m, eps, positions):
     allowed = window_with_first(positions, mask["size"], mask.get("keep_first", 0)) if mask \
         else positions[None, :] <= positions[:, None]
     o = attend(q, k, v, allowed, m["scale"], m.get("softcap"))
-    return o.reshape(T, H * V) @ w["o"].T
+    return product(o.reshape(T, H * V), w["o"])
 
 
 # ------------------------------------------------------------------- the two recurrences
@@ -128,7 +139,7 @@ def mamba2(h, w, m, eps, positions=None):
     T = h.shape[0]
     H, V, N, G = m["heads"], m["vdim"], m["state"], m["groups"]
     inner = H * V
-    p = h @ w["in"].T
+    p = product(h, w["in"])
     z, xbc, dt = p[:, :inner], p[:, inner:2 * inner + 2 * G * N], p[:, 2 * inner + 2 * G * N:]
     xbc = silu(causal_conv(xbc, w["conv"], w["conv.b"]))
     x = xbc[:, :inner].reshape(T, H, V)
@@ -138,17 +149,17 @@ def mamba2(h, w, m, eps, positions=None):
     y = decayed_scan(torch.exp(-torch.exp(w["A_log"]) * dt), C, B, dt[:, :, None] * x) + w["D"][None, :, None] * x
     y = y.reshape(T, inner) * silu(z)
     y = unit_rms(y.reshape(T, m["norm_groups"], -1), eps).reshape(T, inner) * w["norm"]
-    return y @ w["o"].T
+    return product(y, w["o"])
 
 
 def lightning(h, w, m, eps, positions=None):
     T = h.shape[0]
     H, N, V = m["heads"], m["dim"], m["vdim"]
-    q, k = silu(h @ w["q"].T).reshape(T, H, N), silu(h @ w["k"].T).reshape(T, H, N)
-    v = silu(h @ w["v"].T).reshape(T, H, V)
+    q, k = silu(product(h, w["q"])).reshape(T, H, N), silu(product(h, w["k"])).reshape(T, H, N)
+    v = silu(product(h, w["v"])).reshape(T, H, V)
     a = torch.tensor(m["decay"], dtype=h.dtype).expand(T, H)
     o = rms_norm(decayed_scan(a, q, k, v).reshape(T, H * V), w["norm"], eps)
-    return (o * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
+    return product(o * torch.sigmoid(product(h, w["g"])), w["o"])
 
 
 def sub(weights: Dict[str, torch.Tensor], prefix: str) -> Dict[str, torch.Tensor]:
@@ -179,48 +190,56 @@ def choose(s, correction, top: int, groups: int, keep: int):
 
 
 def expert(h, w, prefix):
-    return (silu(h @ w[prefix + ".gate"].T) * (h @ w[prefix + ".up"].T)) @ w[prefix + ".down"].T
+    return product(silu(product(h, w[prefix + ".gate"])) * product(h, w[prefix + ".up"]), w[prefix + ".down"])
 
 
 def moe(h, w, mlp):
     r = mlp["router"]
     g = r.get("groups") or {"count": 1, "keep": 1}
-    s = torch.sigmoid(h @ w["router"].T)
+    s = torch.sigmoid(product(h, w["router"]))
+    ids = [choose(s[t], w["correction"], r["top"], g["count"], g["keep"]) for t in range(h.shape[0])]
     out = torch.zeros_like(h)
-    for t in range(h.shape[0]):
-        for e in choose(s[t], w["correction"], r["top"], g["count"], g["keep"]):
-            out[t] = out[t] + s[t, e] * expert(h[t:t + 1], w, f"e{e}")[0]
+    for e in range(s.shape[1]):
+        rows = [t for t in range(h.shape[0]) if e in ids[t]]
+        if rows:
+            out[rows] += s[rows, e][:, None] * expert(h[rows], w, f"e{e}")
     return out
 
 
 # ----------------------------------------------------------------- per-layer token input
 def token_input(h, table_rows, w):
     """table_rows [T, dim]: the token's part of the side table for this layer."""
-    return (gelu_tanh(h @ w["gate"].T) * table_rows) @ w["proj"].T
+    return product(gelu_tanh(product(h, w["gate"])) * table_rows, w["proj"])
 
 
 # --------------------------------------------------------------------------- model
-def forward(cfg, weights, tokens, dtype=torch.float64, trace: Optional[List[torch.Tensor]] = None, round_inputs=None):
+def forward(cfg, weights, tokens, dtype=torch.float64, trace: Optional[List[torch.Tensor]] = None, round_operands=None,
+            round_scale: float = 1.0):
     """Logits [T, vocab] of one sequence; `trace` collects the residual stream after every layer.
-    round_inputs (a torch dtype): what every sublayer reads is rounded to it and back, the one rounding that
-    any engine with products in that type must make; what it does to the logits says how far two correct
-    implementations in that type may lie apart."""
+    round_operands (a torch dtype): what enters a matrix product is rounded to it and back, the roundings that
+    any engine with products in that type must make; what they do to the logits says how far two correct
+    implementations in that type may lie apart.  round_scale shifts the grid they are rounded to (another sample of the
+    same noise)."""
+    global _round_to
     w = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in weights.items()}
     eps = cfg["norm"]["eps"]
     ids = torch.tensor(list(tokens), dtype=torch.long)
     positions = torch.arange(len(ids))
-    cut = (lambda h: h.to(round_inputs).to(dtype)) if round_inputs is not None else (lambda h: h)
     x = w["embed"][ids]
     side = cfg.get("token_side")
-    for i, layer in enumerate(cfg["layers"]):
-        p = f"l{i}."
-        y = MIXERS[layer["type"]](cut(x), sub(w, p + "mix."), layer["mixer"], eps, positions)
-        x = x + rms_norm(y, w[p + "norm1"], eps)
-        if layer.get("mlp"):
-            x = x + rms_norm(moe(cut(x), sub(w, p + "mlp."), layer["mlp"]), w[p + "norm2"], eps)
-        if side:
-            rows = w["side.embed"][ids, i * side["dim"]:(i + 1) * side["dim"]]
-            x = x + rms_norm(token_input(cut(x), rows, sub(w, p + "side.")), w[p + "side.norm"], eps)
-        if trace is not None:
-            trace.append(x.clone())
-    return rms_norm(x, w["final.norm"], eps) @ w["head"].T
+    _round_to = None if round_operands is None else (round_operands, round_scale)
+    try:
+        for i, layer in enumerate(cfg["layers"]):
+            p = f"l{i}."
+            y = MIXERS[layer["type"]](x, sub(w, p + "mix."), layer["mixer"], eps, positions)
+            x = x + rms_norm(y, w[p + "norm1"], eps)
+            if layer.get("mlp"):
+                x = x + rms_norm(moe(x, sub(w, p + "mlp."), layer["mlp"]), w[p + "norm2"], eps)
+            if side:
+                rows = w["side.embed"][ids, i * side["dim"]:(i + 1) * side["dim"]]
+                x = x + rms_norm(token_input(x, rows, sub(w, p + "side.")), w[p + "side.norm"], eps)
+            if trace is not None:
+                trace.append(x.clone())
+        return product(rms_norm(x, w["final.norm"], eps), w["head"])
+    finally:
+        _round_to = None
