@@ -13,7 +13,7 @@ Llama-3-8B shape; 64 requests of 1,024 tokens that nearly fill the cache at the 
 `--only` picks a part (for profiling), or one of the measurements that are not part of the line:
 `attention` (the attention kernels alone at contexts up to 131,072 tokens), `long_context` (the Llama-3-8B
 shape with 8 requests of 32,000 tokens and one of 131,000), `decode_shapes` (decode steps at the two larger
-shapes by batch), `host` (a step's wall time against its time on the GPU), `vevapel`, `gesutar` and `fofapel` (those designs, as `lufazen`), `lufazen` (the Lufazen design,
+shapes by batch), `host` (a step's wall time against its time on the GPU), `mogutar`, `vevapel`, `gesutar` and `fofapel` (those designs, as `lufazen`), `lufazen` (the Lufazen design,
 recurrent and latent-attention layers, at two sizes beside a Llama of equal size: prefill, decode, time by kernel).
 """
 import argparse
@@ -904,6 +904,58 @@ def vevapel_figures(args):
     return design_beside_llama(args, "vevapel", vevapel_config, bounds, beside=(("lufazen", lufazen_config),))
 
 
+def mogutar_config(layers, width, ff, heads, vocab=32000, window=512):
+    """Layers in the order parallel, lightning.  Parallel: attention in a window of 512 tokens that keeps the first 4
+    (heads of 128, four query heads a kv head, 4 taps on q, k and v, capped scores, YaRN on half of a head) beside a
+    state-space mixer of width / 64 heads of 64 values with states of 128 rows (B and C shared by groups of heads, 4 taps);
+    lightning: `heads` heads of 128 x 128; every layer with 16 routed experts of ff / 8 in four groups of which two are
+    kept, four a token (half of a dense layer's hidden units a token), and a token input of 64 numbers."""
+    out = []
+    mlp = {"kind": "moe", "router": {"experts": 16, "top": 4, "groups": {"count": 4, "keep": 2}}, "expert": {"ff": ff // 8}}
+    for i in range(layers):
+        if i % 2 == 0:
+            left = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "conv": 4,
+                    "mask": {"size": window, "keep_first": 4}, "scale": 128 ** -0.5, "softcap": 30.0,
+                    "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}}}
+            right = {"heads": width // 64, "groups": 2, "state": 128, "vdim": 64, "conv": 4, "norm_groups": 2}
+            mixer = {"left": left, "right": right, "left_scale": 1.0, "right_scale": 1.0}
+            out.append({"type": "parallel", "mixer": mixer, "mlp": mlp})
+        else:
+            decay = [1.0 - 2.0 ** -(2 + 6.0 * h / heads) for h in range(heads)]
+            out.append({"type": "lightning", "mixer": {"heads": heads, "dim": 128, "vdim": 128, "decay": decay}, "mlp": mlp})
+    return {"architecture": "Mogutar", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "token_side": {"dim": 64},
+            "layers": out, "max_position": 8192}
+
+
+def mogutar_figures(args):
+    """The Mogutar design at two sizes beside the closest design of the tree, Fofapel (windowed attention beside a
+    recurrence in every layer, experts), and a Llama, each of equal layers, width, feed-forward size, heads of 128 and
+    vocabulary, as `lufazen_figures`; bounds for the kernels that this design runs."""
+    def bounds(dtype, heads, width, ff):
+        e = ELT[dtype]
+        T, ctx, B, win = PREFILL_TOKENS, PROMPT_LEN, 8, 512
+        kv, sh = max(1, heads // 4), width // 64
+        return {
+            "window attention prefill (flops of scores and values inside the window)":
+                round(2.0 * heads * T * min(win, T / 2) * 2 * 128 / (PEAK_TFLOPS[dtype] * 1e12) * 1e6, 1),
+            "window attention decode b8 (the cached keys and values of the window once)":
+                round(B * min(ctx, win) * 2 * kv * 128 * e / (HBM_GBS * 1e9) * 1e6, 2),
+            "state-space recurrence decode b8 (the states read and written)":
+                round(2.0 * B * sh * 128 * 64 * 4 / (HBM_GBS * 1e9) * 1e6, 2),
+            "state-space recurrence prefill (5 flops per state element and token, float32 vector units at 157 TFLOP/s)":
+                round(5.0 * T * sh * 128 * 64 / (157.3e12) * 1e6, 1),
+            "lightning recurrence decode b8 (the states read and written)":
+                round(2.0 * B * heads * 128 * 128 * 4 / (HBM_GBS * 1e9) * 1e6, 2),
+            "lightning recurrence prefill (5 flops per state element and token, float32 vector units at 157 TFLOP/s)":
+                round(5.0 * T * heads * 128 * 128 / (157.3e12) * 1e6, 1),
+            "experts decode b8 (the weights of all 16 experts once)":
+                round(16 * 3 * width * (ff // 8) * e / (HBM_GBS * 1e9) * 1e6, 2),
+            "experts prefill (flops of four experts a token)":
+                round(2.0 * T * 4 * 3 * width * (ff // 8) / (PEAK_TFLOPS[dtype] * 1e12) * 1e6, 1),
+        }
+    return design_beside_llama(args, "mogutar", mogutar_config, bounds, beside=(("fofapel", fofapel_config),))
+
+
 def design_beside_llama(args, design, config_of, bounds_of, beside=()):
     """`beside`: (name, config function) of further designs of the tree to measure at the same sizes."""
     import torch
@@ -965,6 +1017,9 @@ def run(args):
         return
     if args.only == "vevapel":
         print(json.dumps({"vevapel_beside_lufazen_and_llama": vevapel_figures(args)}), flush=True)
+        return
+    if args.only == "mogutar":
+        print(json.dumps({"mogutar_beside_fofapel_and_llama": mogutar_figures(args)}), flush=True)
         return
     if args.only == "attention":
         print(json.dumps({"decode_attention": attention_sweep()}), flush=True)
@@ -1041,7 +1096,8 @@ def main():
     ap.add_argument("--block-size", type=int, default=16)
     ap.add_argument("--only", default="all",
                     choices=["all", "headline", "decode", "prefill", "fp32", "kernels", "peaks", "llama3_8b", "llama3_8b_prefill", "llama2_13b", "host",
-                             "attention", "long_context", "decode_shapes", "lufazen", "fofapel", "gesutar", "vevapel"],
+                             "attention", "long_context", "decode_shapes", "lufazen", "fofapel", "gesutar", "vevapel",
+                             "mogutar"],
                     help="all: everything in one line; headline: the bfloat16 TinyLlama figures only; decode / prefill: "
                          "one of them (profiling); fp32: the float32 figures as the headline; kernels: decode with the time of "
                          "a step by kernel (torch's profiler); peaks / llama3_8b / "
@@ -1050,7 +1106,8 @@ def main():
                          "8 requests of 32,000 tokens and one of 131,000; decode_shapes: decode steps at the two larger shapes by batch; "
                          "lufazen: prefill and decode of the Lufazen design at two sizes beside a Llama of equal size, by kernel; "
                          "fofapel, gesutar: the same for the Fofapel and the Gesutar design; "
-                         "vevapel: the Vevapel design beside Lufazen and a Llama of equal size")
+                         "vevapel: the Vevapel design beside Lufazen and a Llama of equal size; "
+                         "mogutar: the Mogutar design beside Fofapel and a Llama of equal size")
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         if int(os.environ.get("RANK", "0")) == 0:
