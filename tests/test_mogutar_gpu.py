@@ -497,10 +497,11 @@ def test_windowed_attention_of_a_prompts_portion(kernel, window, keep):
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("dim,vdim,rot,taps,yarn", [(24, 16, 8, 3, (4.0, 64.0, 16.0, 1.0)), (16, 40, 16, 4, None), (6, 11, 2, 2, None),
                                                     (80, 8, 0, 6, None), (8, 8, 4, 1, (1.5, 2048.0, 32.0, 1.0))])
-def test_attn_prepare_with_convolution_and_head_norm(dtype, dim, vdim, rot, taps, yarn):
+def test_conv_attn_prepare(dtype, dim, vdim, rot, taps, yarn):
     """Bias, the short convolution over time on q, k and v with the request's saved inputs, the norm per head with its
     weights and then the rotation (with YaRN's frequencies and magnitude); three requests of unequal length in state slots
     out of order, cut into steps of several tokens and of single ones (which bring the saved inputs up to date themselves)."""
+    from tiny_llm_amd.engine.step import tile_lists
     from tiny_llm_amd.kernels import ops
     from tiny_llm_amd.parts.rotary import angle_tables
     g = torch.Generator().manual_seed(3)
@@ -510,7 +511,7 @@ def test_attn_prepare_with_convolution_and_head_norm(dtype, dim, vdim, rot, taps
     channels = qc + kc + vc
     bias, head_w = torch.randn(channels, generator=g), 1.0 + 0.3 * torch.randn(2 * dim, generator=g)
     conv_w = torch.randn(channels, taps, generator=g)
-    lens, slots = [9, 5, 12], [2, 0, 3]
+    lens, slots = [9, 5, 31], [2, 0, 3]
     ps = [torch.randn(n, channels + 3, generator=g) for n in lens]
     want = []
     for p in ps:
@@ -534,22 +535,22 @@ def test_attn_prepare_with_convolution_and_head_norm(dtype, dim, vdim, rot, taps
     rel = 1e-5 if dtype == torch.float32 else 2.0 ** -8         # a bfloat16 result is its value rounded once
     close = lambda got, w: bool(((got - w).abs() <= rel * (w.abs() + 1.0)).all())
     at = [0, 0, 0]
-    for take in ([3, 1, 2], [1, 1, 1], [1, 0, 1], [4, 2, 5], [0, 1, 3]):
+    for take in ([3, 1, 2], [1, 1, 1], [1, 0, 1], [4, 2, 19], [0, 1, 8]):
         live = [r for r in (1, 2, 0) if take[r]]
         p = torch.cat([ps[r][at[r]:at[r] + take[r]] for r in live]).cuda()
         T = p.shape[0]
         counts = [take[r] for r in live]
         pos = torch.tensor([at[r] + i for r in live for i in range(take[r])], dtype=torch.int32, device="cuda")
         cu = torch.tensor([0] + list(np.cumsum(counts)), dtype=torch.int32, device="cuda")
-        rot_of = torch.tensor([i for i, n in enumerate(counts) for _ in range(n)], dtype=torch.int32, device="cuda")
         sl = torch.tensor([slots[r] for r in live], dtype=torch.int32, device="cuda")
         single = max(counts) == 1
         pages = [torch.full((10, G, block, D), float("nan"), dtype=dtype, device="cuda") for _ in range(2)]
         q = torch.full((1, T, H * D), float("nan"), dtype=dtype, device="cuda")
         where = torch.randperm(40, generator=g)[:T].to(torch.int32)
-        conv = ops.ShortConv(conv_w.cuda(), state, off, rot_of, cu, sl, single)
-        ops.attn_prepare(p, bias.cuda(), None, pos, cos, sin, where.cuda(), q, pages[:1], pages[1], H, G, 1, dim, vdim, qc + kc,
-                         rot, "half", eps=eps, conv=conv, head_w=head_w.cuda())
+        runs = None if single else tuple(torch.tensor(x, dtype=torch.int32, device="cuda") for x in tile_lists(counts, ops.CONV_RUN))
+        conv = ops.ShortConv(conv_w.cuda(), state, off, cu, sl, runs)
+        ops.conv_attn_prepare(p, bias.cuda(), pos, cos, sin, where.cuda(), q[0], pages[0], pages[1], H, G, dim, vdim, conv,
+                              head_w.cuda(), rot, "half", eps)
         if not single and taps > 1:
             ops.conv_state_update(p, 0, channels, state, off, cu, sl, taps, bias.cuda())
         t = 0
@@ -659,7 +660,11 @@ class _Ctx:
         self.cu_seqlens_q = torch.tensor([0] + list(np.cumsum(counts)), dtype=torch.int32, device="cuda")
         self.req_of_token = torch.tensor([i for i, n in enumerate(counts) for _ in range(n)], dtype=torch.int32, device="cuda")
         self.state_slots = torch.tensor(slots, dtype=torch.int32, device="cuda")
-        self.max_q_len, self.num_requests = max(counts), len(counts)
+        self.max_q_len, self.num_requests, self.counts = max(counts), len(counts), counts
+
+    def attention_tiles(self, width):
+        from tiny_llm_amd.engine.step import tile_lists
+        return tuple(torch.tensor(t, dtype=torch.int32, device="cuda") for t in tile_lists(self.counts, width))
 
 
 def _mixer(kind, sizes, dtype, W, eps):
@@ -684,7 +689,7 @@ RECURRENT = [("state_space", (4, 2, 24, 16, 4, 2)), ("state_space", (3, 1, 5, 9,
 @pytest.mark.parametrize("kind,sizes", RECURRENT)
 def test_recurrent_state_over_slots_and_tiny_portions(kind, sizes):
     """The recurrent mixers alone: three requests of unequal length in slots out of order, fed in portions of 1 to 70
-    tokens (single tokens take the one-token kernel), against the plain scan over each whole sequence; a slot of another
+    tokens (single tokens take the one-token kernel, steps with a long portion the chunked form), against the plain scan over each whole sequence; a slot of another
     request stays untouched.  The state is a slice of wider rows, as it is beside another branch."""
     g = torch.Generator().manual_seed(9)
     W, eps = 40, 1e-5

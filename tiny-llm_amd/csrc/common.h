@@ -131,6 +131,59 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
   return t;
 }
 
+// A short causal convolution per channel: y_n = sum_j w[c, j] u_(n - (taps - 1) + j) over a request's inputs u.  The inputs
+// ahead of the request's first token of a step come from its state row, [channel][taps - 1] from saved_off, oldest first.
+// single: no request brings more than one token (row i is request i's); whoever has read a channel's saved inputs then
+// leaves the next token's in their place.
+constexpr int kConvMaxTaps = 16;
+struct ShortConv {
+  const float* w;         // [channels, taps]
+  int taps, single;
+  float* state;
+  int64_t state_stride, saved_off;
+  const int32_t* cu;      // first token row of every request (single: not read)
+  const int32_t* slots;
+};
+// One channel of a run of up to RUN consecutive tokens of a request, the run's first token being its token n0 of this step
+// (row t0 + n0 of `col`).  TAPS >= taps; the inputs are requested together: load() first, value(tt) behind.
+template <int RUN, int TAPS>
+struct ConvRun {
+  float x[RUN + TAPS - 1], wt[TAPS];
+  __device__ __forceinline__ void load(const ShortConv& cv, const float* __restrict__ col, int64_t stride, int t0, int n0,
+                                       int n_tok, int ch, float bias, const float* __restrict__ saved) {
+    const float* w = cv.w + (int64_t)ch * cv.taps;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wt[j] = j >= TAPS - cv.taps ? w[j - (TAPS - cv.taps)] : 0.f;
+    if (n0 >= TAPS - 1) {         // every input lies in this step (rows beyond the run's tokens repeat its last)
+#pragma unroll
+      for (int j = 0; j < RUN + TAPS - 1; ++j)
+        x[j] = col[(int64_t)(t0 + n0 + min(j - (TAPS - 1), n_tok - 1)) * stride];
+#pragma unroll
+      for (int j = 0; j < RUN + TAPS - 1; ++j) x[j] += bias;
+      return;
+    }
+#pragma unroll
+    for (int j = 0; j < RUN + TAPS - 1; ++j) {
+      const int m = n0 - (TAPS - 1) + j;
+      x[j] = 0.f;
+      if (m >= 0) x[j] = col[(int64_t)(t0 + min(m, n0 + n_tok - 1)) * stride] + bias;
+      else if (-m <= cv.taps - 1) x[j] = saved[(cv.taps - 1) + m];
+    }
+  }
+  __device__ __forceinline__ float value(int tt) const {
+    float acc = 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) acc = fmaf(wt[j], x[tt + j], acc);
+    return acc;
+  }
+  // the saved inputs behind the run's first token
+  __device__ __forceinline__ void save_first(const ShortConv& cv, float* __restrict__ saved) const {
+#pragma unroll
+    for (int j = 1; j < TAPS; ++j)
+      if (j > TAPS - cv.taps) saved[j - 1 - (TAPS - cv.taps)] = x[j];
+  }
+};
+
 static inline int tl_launch_status() {
   return hipGetLastError() == hipSuccess ? TL_OK : TL_ERR_LAUNCH;
 }

@@ -114,74 +114,16 @@ __global__ void head_gate_kernel(const T* __restrict__ a, int64_t a_stride, cons
 // token's slot, pages [blocks, nkv, block_size, D]; D >= dim, vdim, and what lies beyond dim (vdim) is written as
 // zeros, so that an attention kernel over heads of D computes the same scores and leaves the values' columns first.
 // A negative slot (padding) stores nothing.
-// Two more options, which make the kernel hold a unit's numbers in LDS between the steps (STAGED):
-//   every channel of q, k and v runs through a short causal convolution behind the bias, a <- sum_j w[c, j] a_(t - (taps - 1) + j):
-//     a request's values ahead of its first token of the step come from its state row, [channel][taps - 1] from
-//     saved_off, oldest first (channels count [q | k | v]); save_single: no request brings more than one token,
-//     and whoever has read a channel's saved values leaves the next token's in their place   (conv.w)
-//   a <- a / sqrt(mean over the unit of a^2 + eps) * head_w, ahead of the rotation; head_w holds `dim` weights for
-//     queries, then `dim` for keys, shared by the heads                                        (head_w)
-struct ShortConv {
-  const float* w;         // [channels, taps], or null
-  int taps, save_single;
-  float* state;
-  int64_t state_stride, saved_off;
-  const int32_t* req_of_token;
-  const int32_t* cu;
-  const int32_t* slots;
-};
-constexpr int kMaxTaps = 16;
-// Channel `ch` (column col of p, bias b) of the convolution at row t of a request that begins at row t0 in this step.
-__device__ __forceinline__ float short_conv(const ShortConv& cv, const float* __restrict__ p, int64_t p_stride, int t, int t0,
-                                            int col, float b, int ch, float* saved_row, bool save) {
-  float* saved = saved_row + (int64_t)ch * (cv.taps - 1);
-  const float* w = cv.w + (int64_t)ch * cv.taps;
-  auto input = [&](int j) {
-    const int m = t - t0 - (cv.taps - 1) + j;
-    return m >= 0 ? p[(int64_t)(t0 + m) * p_stride + col] + b : saved[(cv.taps - 1) + m];
-  };
-  float acc = 0.f;
-  if (cv.taps <= 4) {         // requested together
-    float in[4], wt[4];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      in[j] = j < cv.taps ? input(j) : 0.f;
-      wt[j] = j < cv.taps ? w[j] : 0.f;
-    }
-#pragma unroll
-    for (int j = 0; j < 4; ++j) acc = fmaf(wt[j], in[j], acc);
-    if (save) {
-#pragma unroll
-      for (int j = 1; j < 4; ++j)
-        if (j < cv.taps) saved[j - 1] = in[j];
-    }
-    return acc;
-  }
-  float in[kMaxTaps];
-#pragma unroll
-  for (int j = 0; j < kMaxTaps; ++j) {
-    in[j] = j < cv.taps ? input(j) : 0.f;
-    if (j < cv.taps) acc = fmaf(w[j], in[j], acc);
-  }
-  if (save) {
-#pragma unroll
-    for (int j = 1; j < kMaxTaps; ++j)
-      if (j < cv.taps) saved[j - 1] = in[j];
-  }
-  return acc;
-}
-
 constexpr int kPrepThreads = 256, kPrepWaves = kPrepThreads / TL_WAVE, kPrepPerLane = 4;     // units of up to 256
-template <typename T, bool STAGED>
+template <typename T>
 __global__ __launch_bounds__(kPrepThreads) void attn_prepare_kernel(
     const float* __restrict__ p, int64_t p_stride, const float* __restrict__ bias, const float* __restrict__ norm_w,
     const int32_t* __restrict__ positions, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
     const int32_t* __restrict__ slot_mapping, T* __restrict__ q_out, int64_t q_stride, int64_t q_map_stride,
     T* __restrict__ k_cache0, T* __restrict__ k_cache1, T* __restrict__ v_cache, int heads, int nkv, int maps, int dim,
     int vdim, int D, int v_off, int rot, int interleaved, int whole_norm, int unit_norm, float eps, float temp_coef,
-    int temp_every, int block_size, const ShortConv conv, const float* __restrict__ head_w) {
+    int temp_every, int block_size) {
   __shared__ float red[kPrepWaves];
-  __shared__ float stage[STAGED ? kPrepWaves : 1][STAGED ? kPrepPerLane * TL_WAVE : 1];
   const int t = blockIdx.x, tid = threadIdx.x, wave = tid / TL_WAVE, lane = tid % TL_WAVE;
   const float* row = p + (int64_t)t * p_stride;
   const int q_units = heads * maps, k_units = nkv * maps;
@@ -208,15 +150,6 @@ __global__ __launch_bounds__(kPrepThreads) void attn_prepare_kernel(
   const float* cs = rot ? cos_t + (int64_t)pos * half : nullptr;
   const float* sn = rot ? sin_t + (int64_t)pos * half : nullptr;
   const int64_t page_row = slot >= 0 ? (int64_t)(slot / block_size) * nkv * block_size + slot % block_size : 0;
-  int t0 = 0;
-  float* saved_row = nullptr;
-  bool save = false;
-  if (STAGED && conv.w) {
-    const int r = conv.req_of_token[t];
-    t0 = conv.cu[r];
-    saved_row = conv.state + (int64_t)conv.slots[r] * conv.state_stride + conv.saved_off;
-    save = conv.save_single && t == t0 && conv.cu[r + 1] == t + 1;
-  }
   for (int u = blockIdx.y * kPrepWaves + wave; u < q_units + k_units; u += gridDim.y * kPrepWaves) {
     const bool is_key = u >= q_units;
     if (is_key && slot < 0) continue;
@@ -231,36 +164,12 @@ __global__ __launch_bounds__(kPrepThreads) void attn_prepare_kernel(
     };
     float out[kPrepPerLane];
     float ss = 0.f;
-    if constexpr (STAGED) {
-      float hs = 0.f;
-#pragma unroll
-      for (int i = 0; i < kPrepPerLane; ++i) {
-        const int d = lane + i * TL_WAVE;
-        out[i] = 0.f;
-        if (d < dim) {
-          out[i] = conv.w ? short_conv(conv, p, p_stride, t, t0, c0 + d, bias ? bias[c0 + d] : 0.f, c0 + d, saved_row, save)
-                          : value(d);
-          hs += out[i] * out[i];
-        }
-      }
-      const float hr = head_w ? 1.f / sqrtf(wave_sum(hs) / (float)dim + eps) : 1.f;
-#pragma unroll
-      for (int i = 0; i < kPrepPerLane; ++i) {
-        const int d = lane + i * TL_WAVE;
-        if (d < dim) stage[wave][d] = head_w ? out[i] * hr * head_w[(is_key ? dim : 0) + d] : out[i];
-      }
-      // one wave's LDS operations are carried out in order; the fences keep the compiler to it
-      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-      __builtin_amdgcn_wave_barrier();
-      __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-    }
-    auto prepared = [&](int d) { return STAGED ? stage[wave][d] : value(d); };
 #pragma unroll
     for (int i = 0; i < kPrepPerLane; ++i) {
       const int d = lane + i * TL_WAVE;
       out[i] = 0.f;
       if (d < dim) {
-        float a = prepared(d);
+        float a = value(d);
         if (d < rot) {
           int j, partner;
           bool first;
@@ -273,7 +182,7 @@ __global__ __launch_bounds__(kPrepThreads) void attn_prepare_kernel(
             j = first ? d : d - half;
             partner = first ? d + half : d - half;
           }
-          const float b = prepared(partner);
+          const float b = value(partner);
           a = first ? a * cs[j] - b * sn[j] : a * cs[j] + b * sn[j];
         }
         out[i] = a;
@@ -292,22 +201,137 @@ __global__ __launch_bounds__(kPrepThreads) void attn_prepare_kernel(
       const int d = lane + i * TL_WAVE;
       if (d < D) dst[d] = from_f32<T>(d < dim ? out[i] * f : 0.f);
     }
-    if constexpr (STAGED) {       // the area is read before the wave's next unit is written over it
-      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-      __builtin_amdgcn_wave_barrier();
-      __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-    }
   }
   if (slot < 0) return;
   for (int c = blockIdx.y * kPrepThreads + tid; c < nkv * D; c += gridDim.y * kPrepThreads) {
     const int g = c / D, d = c - g * D;
     float a = 0.f;
     if (d < vdim) {
-      const int col = v_off + g * vdim + d, ch = q_size + k_size + g * vdim + d;
-      const float b = bias ? bias[ch] : 0.f;
-      a = STAGED && conv.w ? short_conv(conv, p, p_stride, t, t0, col, b, ch, saved_row, save) : row[col] + b;
+      const int col = v_off + g * vdim + d;
+      a = row[col] + (bias ? bias[q_size + k_size + g * vdim + d] : 0.f);
     }
     v_cache[(page_row + (int64_t)g * block_size) * D + d] = from_f32<T>(a);
+  }
+}
+
+// The same step for attention whose q, k and v run through a short causal convolution over time behind their biases, and
+// whose queries and keys are normed per head ahead of the rotation:
+//   a <- conv(p + bias) per channel;   q, k: a <- a / sqrt(mean over the head of a^2 + eps) * head_w (or no norm);
+//   q, k: a <- rotate(a) on the first `rot` dims
+// A wave takes one head of q, k or v for a run of up to RUN consecutive tokens of a request (its inputs are requested once,
+// and the run's sums and rotations have each other's latencies to hide behind).  head_w: `dim` weights for queries, then
+// `dim` for keys.  Channels count [q | k | v], as the columns of p do.
+template <typename T, int RUN, int PER, int TAPS>
+__global__ __launch_bounds__(kPrepThreads) void conv_attn_prepare_kernel(
+    const float* __restrict__ p, int64_t p_stride, const float* __restrict__ bias, const float* __restrict__ head_w,
+    const int32_t* __restrict__ positions, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
+    const int32_t* __restrict__ slot_mapping, T* __restrict__ q_out, int64_t q_stride, T* __restrict__ k_cache,
+    T* __restrict__ v_cache, int heads, int nkv, int dim, int vdim, int D, int rot, int interleaved, float eps,
+    int block_size, const ShortConv conv, const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
+    const int32_t* __restrict__ tile_ntok) {
+  __shared__ float stage[kPrepWaves][RUN][PER * TL_WAVE];
+  const int tile = blockIdx.x, wave = threadIdx.x / TL_WAVE, lane = threadIdx.x % TL_WAVE;
+  const int u = blockIdx.y * kPrepWaves + wave;
+  if (u >= heads + 2 * nkv) return;                // whole waves; the kernel has no workgroup barrier
+  const int req = RUN == 1 ? tile : tile_req[tile], tok0 = RUN == 1 ? tile : tile_tok0[tile];
+  const int n_tok = RUN == 1 ? 1 : tile_ntok[tile];
+  if (n_tok <= 0) return;                          // a padding tile
+  const int t0 = RUN == 1 ? tok0 : conv.cu[req];
+  const bool is_q = u < heads, is_v = u >= heads + nkv;
+  const int head = is_q ? u : is_v ? u - heads - nkv : u - heads;
+  const int width = is_v ? vdim : dim;
+  const int c0 = is_q ? head * dim : is_v ? (heads + nkv) * dim + head * vdim : (heads + head) * dim;
+  float* saved_row = conv.taps > 1 ? conv.state + (int64_t)conv.slots[req] * conv.state_stride + conv.saved_off : nullptr;
+  const int pos0 = positions[tok0];                // the tokens of a run are consecutive
+  ConvRun<RUN, TAPS> cv[PER];
+  float hw[PER], cs[RUN][PER], sn[RUN][PER];
+  int partner[PER];
+  bool first[PER];
+  const int half = rot / 2;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int d = lane + i * TL_WAVE, ch = c0 + min(d, width - 1);
+    cv[i].load(conv, p + ch, p_stride, t0, tok0 - t0, n_tok, ch, bias ? bias[ch] : 0.f,
+               saved_row + (int64_t)ch * (conv.taps - 1));
+    hw[i] = (head_w && !is_v) ? head_w[(is_q ? 0 : dim) + min(d, dim - 1)] : 1.f;
+    partner[i] = d;
+    first[i] = true;
+    if (!is_v && d < rot) {
+      int j;
+      if (interleaved) {
+        j = d / 2;
+        first[i] = (d & 1) == 0;
+        partner[i] = first[i] ? d + 1 : d - 1;
+      } else {
+        first[i] = d < half;
+        j = first[i] ? d : d - half;
+        partner[i] = first[i] ? d + half : d - half;
+      }
+#pragma unroll
+      for (int tt = 0; tt < RUN; ++tt) {
+        const int64_t row = (int64_t)(pos0 + min(tt, n_tok - 1)) * half;
+        cs[tt][i] = cos_t[row + j];
+        sn[tt][i] = sin_t[row + j];
+      }
+    }
+  }
+  float a[RUN][PER];
+#pragma unroll
+  for (int tt = 0; tt < RUN; ++tt)
+#pragma unroll
+    for (int i = 0; i < PER; ++i) a[tt][i] = lane + i * TL_WAVE < width ? cv[i].value(tt) : 0.f;
+  if (RUN == 1 && conv.taps > 1) {
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (lane + i * TL_WAVE < width) cv[i].save_first(conv, saved_row + (int64_t)(c0 + lane + i * TL_WAVE) * (conv.taps - 1));
+  }
+  if (!is_v) {
+    if (head_w) {
+#pragma unroll
+      for (int tt = 0; tt < RUN; ++tt) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < PER; ++i) ss += a[tt][i] * a[tt][i];
+        const float r = 1.f / sqrtf(wave_sum(ss) / (float)dim + eps);
+#pragma unroll
+        for (int i = 0; i < PER; ++i) a[tt][i] *= r * hw[i];
+      }
+    }
+    if (rot) {
+#pragma unroll
+      for (int tt = 0; tt < RUN; ++tt)
+#pragma unroll
+        for (int i = 0; i < PER; ++i) stage[wave][tt][lane + i * TL_WAVE] = a[tt][i];
+      // one wave's LDS operations are carried out in order; the fences keep the compiler to it
+      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+      __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+#pragma unroll
+      for (int tt = 0; tt < RUN; ++tt)
+#pragma unroll
+        for (int i = 0; i < PER; ++i)
+          if (lane + i * TL_WAVE < rot) {
+            const float b = stage[wave][tt][partner[i]];
+            a[tt][i] = first[i] ? a[tt][i] * cs[tt][i] - b * sn[tt][i] : a[tt][i] * cs[tt][i] + b * sn[tt][i];
+          }
+    }
+  }
+#pragma unroll
+  for (int tt = 0; tt < RUN; ++tt) {
+    if (tt >= n_tok) break;
+    T* dst;
+    if (is_q) {
+      dst = q_out + (int64_t)(tok0 + tt) * q_stride + (int64_t)head * D;
+    } else {
+      const int slot = slot_mapping ? slot_mapping[tok0 + tt] : -1;
+      if (slot < 0) continue;
+      dst = (is_v ? v_cache : k_cache) + (((int64_t)(slot / block_size) * nkv + head) * block_size + slot % block_size) * D;
+    }
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int d = lane + i * TL_WAVE;
+      if (d < D) dst[d] = from_f32<T>(a[tt][i]);      // zero beyond the head's numbers
+    }
   }
 }
 
@@ -407,18 +431,13 @@ int tl_head_gate(const void* a, int64_t a_stride, const float* g, int64_t g_stri
 
 // p: float32 [n_tokens, p_stride]; bias [q | k | v] and norm_w [q | k] float32 or null; cos_t / sin_t [positions,
 // rot / 2] (null when rot == 0); q_out: `maps` arrays of [n_tokens, q_stride], q_map_stride elements apart; caches
-// [blocks, nkv, block_size, D], k_cache1 for the second map.  conv_w (null: none): float32 [q | k | v channels, taps],
-// the saved values in `state` rows at saved_off; head_w: float32 [2 * dim] or null.
+// [blocks, nkv, block_size, D], k_cache1 for the second map.
 int tl_attn_prepare(const float* p, int64_t p_stride, const float* bias, const float* norm_w, const int32_t* positions,
                     const float* cos_t, const float* sin_t, const int32_t* slot_mapping, void* q_out, int64_t q_stride,
                     int64_t q_map_stride, void* k_cache0, void* k_cache1, void* v_cache, int n_tokens, int heads, int nkv,
                     int maps, int dim, int vdim, int D, int v_off, int rot, int interleaved, int whole_norm, int unit_norm,
-                    float eps, float temp_coef, int temp_every, int block_size, const float* conv_w, int taps,
-                    int save_single, float* state, int64_t state_stride, int64_t saved_off, const int32_t* req_of_token,
-                    const int32_t* cu, const int32_t* slots, const float* head_w, int dtype, hipStream_t stream) {
+                    float eps, float temp_coef, int temp_every, int block_size, int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return TL_OK;
-  if (conv_w && (taps < 1 || taps > kMaxTaps || !state || !req_of_token || !cu || !slots || whole_norm)) return TL_ERR_ARG;
-  if (head_w && whole_norm) return TL_ERR_ARG;
   if (heads <= 0 || nkv <= 0 || maps < 1 || maps > 2 || dim <= 0 || vdim <= 0 || D < dim || D < vdim ||
       D > kPrepPerLane * TL_WAVE || rot < 0 || rot > dim || (rot & 1) || block_size <= 0 || !p || !positions || !q_out ||
       v_off < (heads + nkv) * maps * dim || temp_every < 0)
@@ -431,19 +450,64 @@ int tl_attn_prepare(const float* p, int64_t p_stride, const float* bias, const f
   const int units = (heads + nkv) * maps, most = (units + kPrepWaves - 1) / kPrepWaves;
   const int share = n_tokens >= 256 ? 1 : (256 / n_tokens < most ? 256 / n_tokens : most);
   dim3 g(n_tokens, share), b(kPrepThreads);
-  const ShortConv conv{conv_w, taps, save_single, state, state_stride, saved_off, req_of_token, cu, slots};
-#define TL_PREPARE(T, STAGED)                                                                                            \
-  hipLaunchKernelGGL((attn_prepare_kernel<T, STAGED>), g, b, 0, stream, p, p_stride, bias, norm_w, positions, cos_t,     \
-                     sin_t, slot_mapping, (T*)q_out, q_stride, q_map_stride, (T*)k_cache0, (T*)k_cache1, (T*)v_cache,    \
-                     heads, nkv, maps, dim, vdim, D, v_off, rot, interleaved, whole_norm, unit_norm, eps, temp_coef,     \
-                     temp_every, block_size, conv, head_w)
-  const bool staged = conv_w || head_w;
-  if (dtype == 0 && staged) TL_PREPARE(float, true);
-  else if (dtype == 0) TL_PREPARE(float, false);
-  else if (dtype == 1 && staged) TL_PREPARE(bf16_t, true);
-  else if (dtype == 1) TL_PREPARE(bf16_t, false);
+  if (dtype == 0)
+    hipLaunchKernelGGL(attn_prepare_kernel<float>, g, b, 0, stream, p, p_stride, bias, norm_w, positions, cos_t, sin_t,
+                       slot_mapping, (float*)q_out, q_stride, q_map_stride, (float*)k_cache0, (float*)k_cache1,
+                       (float*)v_cache, heads, nkv, maps, dim, vdim, D, v_off, rot, interleaved, whole_norm, unit_norm, eps,
+                       temp_coef, temp_every, block_size);
+  else if (dtype == 1)
+    hipLaunchKernelGGL(attn_prepare_kernel<bf16_t>, g, b, 0, stream, p, p_stride, bias, norm_w, positions, cos_t, sin_t,
+                       slot_mapping, (bf16_t*)q_out, q_stride, q_map_stride, (bf16_t*)k_cache0, (bf16_t*)k_cache1,
+                       (bf16_t*)v_cache, heads, nkv, maps, dim, vdim, D, v_off, rot, interleaved, whole_norm, unit_norm,
+                       eps, temp_coef, temp_every, block_size);
+  else
+    return TL_ERR_ARG;
+  return tl_launch_status();
+}
+
+// Tokens a wave of tl_conv_attn_prepare takes in a run (what its tile lists cut a request's tokens into).
+constexpr int kConvRun = 8;
+int tl_conv_run(void) { return kConvRun; }
+
+// p: float32 [n_tokens, p_stride], columns [q | k | v]; bias (over them) and head_w [2 * dim] float32 or null; caches
+// [blocks, nkv, block_size, D].  single: every request brings one token (row i is request i's), no tile lists; else the
+// lists cut every request's tokens into runs of at most tl_conv_run() and conv_state_update has to follow.
+int tl_conv_attn_prepare(const float* p, int64_t p_stride, const float* bias, const float* head_w, const int32_t* positions,
+                         const float* cos_t, const float* sin_t, const int32_t* slot_mapping, void* q_out, int64_t q_stride,
+                         void* k_cache, void* v_cache, int heads, int nkv, int dim, int vdim, int D, int rot, int interleaved,
+                         float eps, int block_size, const float* conv_w, int taps, float* state, int64_t state_stride,
+                         int64_t saved_off, const int32_t* cu, const int32_t* slots, int single, const int32_t* tile_req,
+                         const int32_t* tile_tok0, const int32_t* tile_ntok, int n_tiles, int dtype, hipStream_t stream) {
+  if (n_tiles <= 0) return TL_OK;
+  if (heads <= 0 || nkv <= 0 || dim <= 0 || vdim <= 0 || D < dim || D < vdim || D > kPrepPerLane * TL_WAVE || rot < 0 ||
+      rot > dim || (rot & 1) || block_size <= 0 || !p || !positions || !q_out || (rot > 0 && (!cos_t || !sin_t)) ||
+      (slot_mapping && (!k_cache || !v_cache)) || (interleaved != 0 && interleaved != 1) || !conv_w || taps < 1 ||
+      taps > kConvMaxTaps || (taps > 1 && !state) || !slots || (!single && (!tile_req || !tile_tok0 || !tile_ntok || !cu)) ||
+      heads + 2 * nkv > 4 * 65535)
+    return TL_ERR_ARG;
+  const ShortConv conv{conv_w, taps, single, state, state_stride, saved_off, cu, slots};
+  dim3 g(n_tiles, (heads + 2 * nkv + kPrepWaves - 1) / kPrepWaves), b(kPrepThreads);
+#define TL_CAP(T, RUN, PER, TAPS)                                                                                        \
+  hipLaunchKernelGGL((conv_attn_prepare_kernel<T, RUN, PER, TAPS>), g, b, 0, stream, p, p_stride, bias, head_w,           \
+                     positions, cos_t, sin_t, slot_mapping, (T*)q_out, q_stride, (T*)k_cache, (T*)v_cache, heads, nkv,    \
+                     dim, vdim, D, rot, interleaved, eps, block_size, conv, tile_req, tile_tok0, tile_ntok)
+#define TL_CAP_TAPS(T, RUN, PER)                \
+  if (taps <= 4) TL_CAP(T, RUN, PER, 4);        \
+  else TL_CAP(T, RUN, PER, kConvMaxTaps);
+#define TL_CAP_PER(T, RUN)                                \
+  if (D <= TL_WAVE) { TL_CAP_TAPS(T, RUN, 1) }            \
+  else if (D <= 2 * TL_WAVE) { TL_CAP_TAPS(T, RUN, 2) }   \
+  else { TL_CAP_TAPS(T, RUN, 4) }
+#define TL_CAP_RUN(T)                             \
+  if (single) { TL_CAP_PER(T, 1) }                \
+  else { TL_CAP_PER(T, kConvRun) }
+  if (dtype == 0) { TL_CAP_RUN(float) }
+  else if (dtype == 1) { TL_CAP_RUN(bf16_t) }
   else return TL_ERR_ARG;
-#undef TL_PREPARE
+#undef TL_CAP_RUN
+#undef TL_CAP_PER
+#undef TL_CAP_TAPS
+#undef TL_CAP
   return tl_launch_status();
 }
 

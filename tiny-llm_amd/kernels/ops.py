@@ -1858,46 +1858,43 @@ def time_mix_recurrence(x: torch.Tensor, r_off: int, k_off: int, v_off: int, w_o
 
 # ---------------------------- linear recurrences with one decay per head and token (csrc/linear_recurrence.hip)
 LINEAR_MAX_DIM = 256            # rows of a head's state
+LINEAR_CHUNK = 64               # tokens of a chunk of the chunked form
+LINEAR_CHUNK_TOKENS = 48        # from this many tokens of a request in a step on the chunked form is used
 LINEAR_DECODE_MAX_VDIM = 256    # value columns the one-token kernel takes
 
 
 def ssd_prepare(p: torch.Tensor, conv_off: int, dt_off: int, conv: ShortConv, conv_b: Optional[torch.Tensor],
                 a_log: torch.Tensor, dt_bias: torch.Tensor, x: torch.Tensor, dt_col: int, a_col: int) -> None:
     """x[t] = [silu(conv(p[t, conv_off ..]) + conv_b): channels | c = softplus(p[t, dt_off + h] + dt_bias[h]), from column
-    dt_col | exp(-exp(a_log[h]) c), from a_col]; p and x float32."""
-    _dev(p, conv_b, a_log, dt_bias, x, conv.w, conv.state, conv.req_of_token, conv.cu_seqlens, conv.state_slots)
+    dt_col | ln a = -exp(a_log[h]) c, from a_col]; p and x float32."""
+    _dev(p, conv_b, a_log, dt_bias, x)
     _rows_2d(p, "ssd_prepare input")
     _rows_2d(x, "ssd_prepare output")
-    _i32(conv.req_of_token, conv.cu_seqlens, conv.state_slots)
-    T, heads = p.shape[0], a_log.numel()
-    channels, taps = conv.w.shape
-    _f32_vec(conv.w, channels * taps, "ssd_prepare taps")
+    T, heads, channels = p.shape[0], a_log.numel(), conv.w.shape[0]
     _f32_vec(conv_b, channels, "ssd_prepare convolution bias")
     _f32_vec(a_log, heads, "A_log")
     _f32_vec(dt_bias, heads, "dt_bias")
     _need(p.dtype == x.dtype == torch.float32 and x.shape[0] == T and conv_off + channels <= p.shape[1]
-          and dt_off + heads <= p.shape[1] and channels <= dt_col and dt_col + heads <= a_col and a_col + heads <= x.shape[1]
-          and 1 <= taps <= DELTA_MAX_TAPS and conv.req_of_token.numel() == T
-          and conv.cu_seqlens.numel() == conv.state_slots.numel() + 1 and conv.state.dtype == torch.float32
-          and conv.state.dim() == 2 and conv.state.stride(1) == 1
-          and conv.saved_off + channels * (taps - 1) <= conv.state.shape[1], "ssd_prepare: shapes do not fit")
-    _check(_lib().tl_ssd_prepare(_ptr(p), c_int64(p.stride(0)), c_int(conv_off), c_int(dt_off), _ptr(conv.w), _ptr(conv_b),
-                                 _ptr(a_log), _ptr(dt_bias), _ptr(conv.state), c_int64(conv.state.stride(0)),
-                                 c_int64(conv.saved_off), _ptr(conv.req_of_token), _ptr(conv.cu_seqlens),
-                                 _ptr(conv.state_slots), _ptr(x), c_int64(x.stride(0)), c_int(dt_col), c_int(a_col), c_int(T),
-                                 c_int(channels), c_int(heads), c_int(taps), c_int(1 if conv.save_single else 0), _stream()),
-           "ssd_prepare")
+          and dt_off + heads <= p.shape[1] and channels <= dt_col and dt_col + heads <= a_col and a_col + heads <= x.shape[1],
+          "ssd_prepare: shapes do not fit")
+    w, taps, (state, stride, saved, cu, slots), lists, n_tiles = conv.args(channels, T, "ssd_prepare")
+    _check(_lib().tl_ssd_prepare(_ptr(p), c_int64(p.stride(0)), c_int(conv_off), c_int(dt_off), w, _ptr(conv_b), _ptr(a_log),
+                                 _ptr(dt_bias), state, stride, saved, cu, slots, _ptr(x), c_int64(x.stride(0)), c_int(dt_col),
+                                 c_int(a_col), c_int(channels), c_int(heads), taps, *lists, n_tiles, _stream()), "ssd_prepare")
 
 
 def linear_recurrence(x: torch.Tensor, q_off: int, k_off: int, v_off: int, state: torch.Tensor, cu_seqlens: torch.Tensor,
                       state_slots: torch.Tensor, out: torch.Tensor, heads: int, groups: int, dim: int, vdim: int,
                       decay: Optional[torch.Tensor] = None, a_off: int = -1, c_off: int = -1,
-                      skip: Optional[torch.Tensor] = None, silu: bool = False, single: bool = False) -> torch.Tensor:
+                      skip: Optional[torch.Tensor] = None, silu: bool = False, single: bool = False,
+                      tiles=None) -> torch.Tensor:
     """Walks every request's tokens of this step through S <- a S + k (c v)^T; o = S^T q + D v, S [heads, dim, vdim] at the
     start of the request's state row.  Row t of x (float32) holds q and k (groups x dim, from q_off and k_off; head n
-    reads group n // (heads / groups)), v (heads x vdim, from v_off), c (per head, from c_off; negative: 1) and a (per
-    head, from a_off; negative: `decay`[head], float32).  skip: D per head, or None.  silu: q, k and v are SiLU's inputs.
-    single: no request brings more than one token."""
+    reads group n // (heads / groups)), v (heads x vdim, from v_off), c (per head, from c_off; negative: 1) and ln a
+    (per head, from a_off; negative: a is `decay`[head], float32).  skip: D per head, or None.  silu: q, k and v are SiLU's
+    inputs.  single: no request brings more than one token.  tiles (req, tok0, ntok): every request's tokens cut into
+    chunks of at most LINEAR_CHUNK, request after request; the step then runs chunk by chunk on the matrix cores (float32
+    either way; meant for steps that bring many tokens of a request)."""
     _dev(x, state, cu_seqlens, state_slots, out, decay, skip)
     _rows_2d(x, "linear_recurrence operands")
     _i32(cu_seqlens, state_slots)
@@ -1913,6 +1910,20 @@ def linear_recurrence(x: torch.Tensor, q_off: int, k_off: int, v_off: int, state
     _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
           and heads * dim * vdim <= state.shape[1] and cu_seqlens.numel() == R + 1,
           "linear_recurrence: the state is float32 [slots, >= heads * dim * vdim]")
+    if tiles is not None:
+        _, tok0, ntok = tiles
+        _i32(tok0, ntok)
+        n_tiles = tok0.numel()
+        _need(ntok.numel() == n_tiles > 0, "linear_recurrence: chunk lists of one length")
+        u = scratch("recurrence_chunks", (n_tiles * heads * dim * vdim,), torch.float32, x.device)
+        decays = scratch("recurrence_decays", (n_tiles * heads,), torch.float32, x.device)
+        _check(_lib().tl_linear_recurrence_chunks(_ptr(x), c_int64(x.stride(0)), c_int(q_off), c_int(k_off), c_int(v_off),
+                                                  c_int(c_off), c_int(a_off), _ptr(decay), _ptr(skip), _ptr(state),
+                                                  c_int64(state.stride(0)), _ptr(cu_seqlens), _ptr(state_slots), _ptr(tok0),
+                                                  _ptr(ntok), _ptr(u), _ptr(decays), _ptr(out), c_int(n_tiles), c_int(R),
+                                                  c_int(heads), c_int(groups), c_int(dim), c_int(vdim),
+                                                  c_int(1 if silu else 0), _stream()), "linear_recurrence (chunks)")
+        return out
     decode = (single and vdim % 4 == 0 and vdim <= LINEAR_DECODE_MAX_VDIM and state.stride(0) % 4 == 0
               and state.data_ptr() % 16 == 0)
     _check(_lib().tl_linear_recurrence(_ptr(x), c_int64(x.stride(0)), c_int(q_off), c_int(k_off), c_int(v_off), c_int(c_off),
@@ -2287,19 +2298,48 @@ def embedding_pairs(tokens: torch.Tensor, positions: torch.Tensor, req_of_token:
 
 
 # ------------------------------------------- the general step between the q/k/v product and the attention kernel
+CONV_RUN = 8        # tokens of a run (csrc/qk_prepare.hip kConvRun)
+
+
 @dataclass
 class ShortConv:
     """A short causal convolution per channel inside another step: taps w [channels, taps] (float32, the last column the
-    current token's), saved inputs in the `state` rows at saved_off, [channel][taps - 1], oldest first.  save_single (no
-    request of the step brings more than one token): the step brings the saved inputs up to date itself; else
-    `conv_state_update` has to follow."""
+    current token's), saved inputs in the `state` rows at saved_off, [channel][taps - 1], oldest first.  runs: (req, tok0,
+    ntok) lists that cut every request's tokens into runs of at most CONV_RUN, with `conv_state_update` to follow; None: every
+    request of the step brings one token (row i is request i's), and the step brings the saved inputs up to date itself."""
     w: torch.Tensor
-    state: torch.Tensor
+    state: Optional[torch.Tensor]
     saved_off: int
-    req_of_token: torch.Tensor
     cu_seqlens: torch.Tensor
     state_slots: torch.Tensor
-    save_single: bool = False
+    runs: Optional[tuple] = None
+
+    def args(self, channels: int, tokens: int, what: str):
+        """The kernels' arguments (w, taps, the state's, single and the lists, n_tiles), checked."""
+        _dev(self.w, self.state, self.cu_seqlens, self.state_slots)
+        _i32(self.cu_seqlens, self.state_slots)
+        taps = self.w.shape[1]
+        R = self.state_slots.numel()
+        _f32_vec(self.w, channels * taps, f"{what}: convolution taps")
+        _need(1 <= taps <= DELTA_MAX_TAPS and self.cu_seqlens.numel() == R + 1, f"{what}: 1 to {DELTA_MAX_TAPS} taps, a row start per request")
+        st = self.state
+        if taps > 1:
+            _need(st is not None and st.dtype == torch.float32 and st.dim() == 2 and st.stride(1) == 1
+                  and self.saved_off + channels * (taps - 1) <= st.shape[1], f"{what}: the convolution's state does not fit")
+        else:
+            st = None
+        n_tiles = tokens
+        lists = (None, None, None)
+        if self.runs is None:
+            _need(tokens == R, f"{what}: without runs every request brings one token")
+        else:
+            lists = self.runs
+            _i32(*lists)
+            n_tiles = lists[0].numel()
+            _need(all(t.numel() == n_tiles for t in lists), f"{what}: run lists of one length")
+        state_args = (_ptr(st), c_int64(st.stride(0) if st is not None else 0), c_int64(self.saved_off), _ptr(self.cu_seqlens),
+                      _ptr(self.state_slots))
+        return _ptr(self.w), c_int(taps), state_args, (c_int(1 if self.runs is None else 0), *(_ptr(t) for t in lists)), c_int(n_tiles)
 
 
 ATTN_PREPARE_MAX_DIM = 256      # numbers a unit (one map of one head) may have, and the padded head size D
@@ -2309,8 +2349,7 @@ def attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], norm_w: Optional
                  cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], slot_mapping: Optional[torch.Tensor],
                  q_out: torch.Tensor, k_caches, v_cache: Optional[torch.Tensor], heads: int, kv_heads: int, maps: int,
                  dim: int, vdim: int, v_off: int, rot: int = 0, pairing: str = "half", whole_norm: bool = False,
-                 unit_norm: bool = False, eps: float = 1e-6, q_temp=None, conv: Optional["ShortConv"] = None,
-                 head_w: Optional[torch.Tensor] = None) -> None:
+                 unit_norm: bool = False, eps: float = 1e-6, q_temp=None) -> None:
     """From the float32 product p [T, >= v_off + kv_heads * vdim] = [q: heads * maps units of dim | k: kv_heads * maps
     units | v: kv_heads heads of vdim, from column v_off]: bias added (float32 over [q | k | v]), an RMS norm over ALL of
     a token's q numbers (and all of its k numbers) with weights norm_w (float32 over [q | k], `whole_norm`), the first
@@ -2318,11 +2357,7 @@ def attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], norm_w: Optional
     (`unit_norm`), queries times 1 + coef * ln(floor((pos + 1) / every) + 1) (`q_temp` = (coef, every)).  Queries leave
     as q_out [maps, T, heads * D] rounded to the engine's type, keys of map m go to k_caches[m] and values to v_cache
     (pages [blocks, kv_heads, block, D]) at the tokens' slots; D is q_out's head size, what lies beyond dim or vdim is
-    written as zeros.  slot_mapping None (or a negative slot) stores nothing.
-    conv: behind the bias every channel of q, k and v runs through a short causal convolution, its inputs ahead of a
-    request's first token of the step kept in the request's state row (v_off is then q's and k's columns: the channels
-    are the columns).  head_w (float32 [2 * dim], queries' weights then keys'): every unit is divided by its own root
-    mean square and multiplied by them, ahead of the rotation."""
+    written as zeros.  slot_mapping None (or a negative slot) stores nothing."""
     k_caches = tuple(k_caches) if k_caches is not None else ()
     _dev(p, bias, norm_w, positions, cos, sin, slot_mapping, q_out, v_cache, *k_caches)
     _rows_2d(p, "attn_prepare input")
@@ -2363,25 +2398,6 @@ def attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], norm_w: Optional
     coef, every = (float(q_temp[0]), int(q_temp[1])) if q_temp else (0.0, 0)
     _need(every >= 0, "attn_prepare: the temperature's step is positive")
     store = slot_mapping is not None
-    cv = (c_void_p(0), c_int(0), c_int(0), c_void_p(0), c_int64(0), c_int64(0), c_void_p(0), c_void_p(0), c_void_p(0))
-    if conv is not None:
-        channels = q_size + k_size + v_size
-        _dev(conv.w, conv.state, conv.req_of_token, conv.cu_seqlens, conv.state_slots)
-        _i32(conv.req_of_token, conv.cu_seqlens, conv.state_slots)
-        taps = conv.w.shape[1]
-        _f32_vec(conv.w, channels * taps, "attn_prepare convolution taps")
-        _need(not whole_norm and v_off == q_size + k_size, "attn_prepare: the convolution takes adjacent q, k and v columns "
-              "and no norm over whole projections")
-        _need(1 <= taps <= DELTA_MAX_TAPS and conv.req_of_token.numel() == T
-              and conv.cu_seqlens.numel() == conv.state_slots.numel() + 1 and conv.state.dtype == torch.float32
-              and conv.state.dim() == 2 and conv.state.stride(1) == 1
-              and conv.saved_off + channels * (taps - 1) <= conv.state.shape[1], "attn_prepare: the convolution's shapes do not fit")
-        cv = (_ptr(conv.w), c_int(taps), c_int(1 if conv.save_single else 0), _ptr(conv.state), c_int64(conv.state.stride(0)),
-              c_int64(conv.saved_off), _ptr(conv.req_of_token), _ptr(conv.cu_seqlens), _ptr(conv.state_slots))
-    if head_w is not None:
-        _dev(head_w)
-        _need(not whole_norm, "attn_prepare: one norm ahead of the rotation, per head or over the whole projection")
-        _f32_vec(head_w, 2 * dim, "attn_prepare head norm weights")
     _check(_lib().tl_attn_prepare(_ptr(p), c_int64(p.stride(0)), _ptr(bias), _ptr(norm_w), _ptr(positions), _ptr(cos),
                                   _ptr(sin), _ptr(slot_mapping), _ptr(q_out), c_int64(q_out.stride(1)),
                                   c_int64(q_out.stride(0)), _ptr(k_caches[0] if store else None),
@@ -2389,8 +2405,58 @@ def attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], norm_w: Optional
                                   c_int(T), c_int(heads), c_int(kv_heads), c_int(maps), c_int(dim), c_int(vdim), c_int(D),
                                   c_int(v_off), c_int(rot), c_int(ROPE_PAIRINGS.index(pairing)),
                                   c_int(1 if whole_norm else 0), c_int(1 if unit_norm else 0), c_float(eps), c_float(coef),
-                                  c_int(every), c_int(block_size), *cv, _ptr(head_w), c_int(_dt(q_out)), _stream()),
-           "attn_prepare")
+                                  c_int(every), c_int(block_size), c_int(_dt(q_out)), _stream()), "attn_prepare")
+
+
+def conv_attn_prepare(p: torch.Tensor, bias: Optional[torch.Tensor], positions: torch.Tensor, cos: Optional[torch.Tensor],
+                      sin: Optional[torch.Tensor], slot_mapping: Optional[torch.Tensor], q_out: torch.Tensor,
+                      k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], heads: int, kv_heads: int, dim: int,
+                      vdim: int, conv: ShortConv, head_w: Optional[torch.Tensor] = None, rot: int = 0, pairing: str = "half",
+                      eps: float = 1e-6) -> None:
+    """`attn_prepare` for attention whose q, k and v run through a short causal convolution: from the float32 product p
+    [T, >= channels], columns [q: heads x dim | k: kv_heads x dim | v: kv_heads x vdim], bias added (float32 over them), every
+    channel convolved over time (`conv`), q and k divided by the head's root mean square and multiplied by head_w (float32
+    [2 * dim], queries' weights, then keys'; None: no norm), then rotated on the first `rot` dims.  Queries leave as q_out
+    [T, heads * D], keys and values go to the pages, zeros beyond dim and vdim as in `attn_prepare`."""
+    _dev(p, bias, head_w, positions, cos, sin, slot_mapping, q_out, k_cache, v_cache)
+    _rows_2d(p, "conv_attn_prepare input")
+    _rows_2d(q_out, "conv_attn_prepare queries")
+    T = p.shape[0]
+    channels = (heads + kv_heads) * dim + kv_heads * vdim
+    _need(p.dtype == torch.float32 and heads > 0 and kv_heads > 0 and heads % kv_heads == 0 and p.shape[1] >= channels,
+          "conv_attn_prepare: the product is float32 with q, k and v side by side, heads a multiple of kv heads")
+    _need(q_out.shape[0] == T and q_out.shape[1] % heads == 0, "conv_attn_prepare: queries leave as [T, heads * D]")
+    D = q_out.shape[1] // heads
+    _need(0 < dim <= D and 0 < vdim <= D and D <= ATTN_PREPARE_MAX_DIM, f"conv_attn_prepare: dim and vdim within D = {D} <= "
+          f"{ATTN_PREPARE_MAX_DIM}")
+    _f32_vec(bias, channels, "conv_attn_prepare bias")
+    _f32_vec(head_w, 2 * dim, "conv_attn_prepare head norm weights")
+    _need(pairing in ROPE_PAIRINGS and rot % 2 == 0 and 0 <= rot <= dim, "conv_attn_prepare: a known pairing on an even number "
+          "of dims within the head")
+    _i32(positions)
+    _need(positions.numel() == T, "conv_attn_prepare: one position per row")
+    if rot:
+        _need(cos is not None and sin is not None and cos.dtype == sin.dtype == torch.float32 and cos.is_contiguous()
+              and sin.is_contiguous() and cos.shape == sin.shape and cos.shape[1] == rot // 2,
+              "conv_attn_prepare: angle tables are float32 [positions, rot / 2]")
+    block_size = 1
+    if slot_mapping is not None:
+        _i32(slot_mapping)
+        _need(slot_mapping.numel() == T and k_cache is not None and v_cache is not None, "conv_attn_prepare: one slot per row, "
+              "a key cache and a value cache")
+        for c in (k_cache, v_cache):
+            _need(c.dtype == q_out.dtype and c.dim() == 4 and c.is_contiguous() and c.shape[1] == kv_heads
+                  and c.shape[3] == D and c.shape == v_cache.shape, "conv_attn_prepare: caches are contiguous "
+                  "[blocks, kv_heads, block, D] of the queries' type")
+        block_size = v_cache.shape[2]
+    store = slot_mapping is not None
+    w, taps, state_args, lists, n_tiles = conv.args(channels, T, "conv_attn_prepare")
+    _check(_lib().tl_conv_attn_prepare(_ptr(p), c_int64(p.stride(0)), _ptr(bias), _ptr(head_w), _ptr(positions), _ptr(cos),
+                                       _ptr(sin), _ptr(slot_mapping), _ptr(q_out), c_int64(q_out.stride(0)),
+                                       _ptr(k_cache if store else None), _ptr(v_cache if store else None), c_int(heads),
+                                       c_int(kv_heads), c_int(dim), c_int(vdim), c_int(D), c_int(rot),
+                                       c_int(ROPE_PAIRINGS.index(pairing)), c_float(eps), c_int(block_size), w, taps,
+                                       *state_args, *lists, n_tiles, c_int(_dt(q_out)), _stream()), "conv_attn_prepare")
 
 
 ATTN_GATES = {None: 0, "head": 1, "element": 2}

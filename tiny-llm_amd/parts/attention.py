@@ -321,9 +321,13 @@ class GatedAttention(Attention):
         self.keep, self.softcap, self.taps = int(keep_first or 0), float(softcap or 0.0), int(conv_taps or 0)
         if self.keep < 0 or self.softcap < 0 or (self.keep and not window):
             raise ValueError(f"{prefix}: keep_first and softcap are not negative, and kept tokens lie behind a window")
-        if self.taps and (not (1 <= self.taps <= ops.DELTA_MAX_TAPS) or qk_norm == "whole"):
-            raise ValueError(f"{prefix}: a convolution of 1 to {ops.DELTA_MAX_TAPS} taps, and no norm over the whole projection "
-                             f"behind it, got {conv_taps} and {qk_norm!r}")
+        if not (0 <= self.taps <= ops.DELTA_MAX_TAPS):
+            raise ValueError(f"{prefix}: a convolution of 1 to {ops.DELTA_MAX_TAPS} taps, got {conv_taps}")
+        # the convolution and the norm per head are steps of a kernel of their own, which has no more than them
+        self.convolved = bool(self.taps) or qk_norm == "head"
+        if self.convolved and (maps != 1 or q_temp or qk_norm not in (None, "head")):
+            raise ValueError(f"{prefix}: a convolution or a norm per head ahead of the rotation goes with one score map, no query "
+                             f"temperature and no other norm")
         if maps not in (1, 2):
             raise ValueError(f"{prefix}: one or two score maps, got {maps}")
         if gate not in ops.ATTN_GATES:
@@ -399,6 +403,8 @@ class GatedAttention(Attention):
             self.head_w = torch.cat([f32(tensors[n[k] + self.norm_suffix]) for k in ("q", "k")]).contiguous()
         if self.taps:
             self.conv_w = torch.cat([f32(tensors[n[k] + self.conv_suffix]) for k in ("q", "k", "v")]).contiguous()
+        elif self.convolved:        # one tap of one: the value itself
+            self.conv_w = torch.ones((self.v_off + self.v_cols, 1), dtype=torch.float32, device=dev)
         w_o = tensors[n["o"]]
         if self.out_bias:
             wide = torch.zeros((self.hidden_size, self.out_cols + self.out_tail), dtype=self.dtype, device=dev)
@@ -434,20 +440,24 @@ class GatedAttention(Attention):
         pairing = getattr(self.position, "pairing", "half")
         q = ops.scratch("q_prepared", (self.maps, T, self.q_size), self.dtype, dev)
         write = cache.write
-        conv = None
-        channels = self.v_off + self.v_cols
-        if self.taps:
-            # a step of single tokens brings the saved inputs up to date in the same kernel
-            conv = ops.ShortConv(self.conv_w, state if state is not None else ops.scratch("no_state", (1, 4), torch.float32, dev),
-                                 0, ctx.req_of_token, ctx.cu_seqlens_q, ctx.state_slots, ctx.max_q_len == 1)
         k_caches = [cache.tensors["k"]] + ([cache.tensors["k2"]] if self.maps == 2 else [])
-        ops.attn_prepare(p, self.b_in, self.norm_w, ctx.positions, cos, sin,
-                         ctx.slot_mappings[cache.group] if write else None, q, k_caches if write else None,
-                         cache.tensors["v"] if write else None, H, self.num_kv_heads, self.maps, self.qk_dim,
-                         self.value_dim, self.v_off, rot, pairing, self.qk_norm == "whole", self.qk_norm == "unit",
-                         self.eps, self.q_temp, conv, self.head_w)
-        if self.taps > 1 and ctx.max_q_len > 1:
-            ops.conv_state_update(p, 0, channels, state, 0, ctx.cu_seqlens_q, ctx.state_slots, self.taps, self.b_in)
+        slots = ctx.slot_mappings[cache.group] if write else None
+        if self.convolved:
+            # a step of single tokens brings the convolutions' saved inputs up to date in the same kernel
+            single = ctx.max_q_len == 1 and T == ctx.num_requests
+            conv = ops.ShortConv(self.conv_w, state, 0, ctx.cu_seqlens_q, ctx.state_slots,
+                                 None if single else ctx.attention_tiles(ops.CONV_RUN))
+            ops.conv_attn_prepare(p, self.b_in, ctx.positions, cos, sin, slots, q[0], k_caches[0] if write else None,
+                                  cache.tensors["v"] if write else None, H, self.num_kv_heads, self.qk_dim, self.value_dim, conv,
+                                  self.head_w, rot, pairing, self.eps)
+            if self.taps > 1 and not single:
+                ops.conv_state_update(p, 0, self.v_off + self.v_cols, state, 0, ctx.cu_seqlens_q, ctx.state_slots, self.taps,
+                                      self.b_in)
+        else:
+            ops.attn_prepare(p, self.b_in, self.norm_w, ctx.positions, cos, sin, slots, q, k_caches if write else None,
+                             cache.tensors["v"] if write else None, H, self.num_kv_heads, self.maps, self.qk_dim,
+                             self.value_dim, self.v_off, rot, pairing, self.qk_norm == "whole", self.qk_norm == "unit",
+                             self.eps, self.q_temp)
         outs = []
         for m in range(self.maps):
             # float32 whatever the engine's type: the maps' difference, the head's norm and the gates follow in float32

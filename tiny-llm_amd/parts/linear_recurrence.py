@@ -34,6 +34,11 @@ def _pad(n: int, m: int) -> int:
     return -(-n // m) * m
 
 
+def _chunks(ctx):
+    """The step's tokens in the recurrence's chunks, if some request may bring many."""
+    return ctx.attention_tiles(ops.LINEAR_CHUNK) if ctx.max_q_len >= ops.LINEAR_CHUNK_TOKENS else None
+
+
 def _project_out(part, z, residual):
     if residual is None:
         out = ops.scratch("sublayer_out", (z.shape[0], part.hidden_size), torch.float32, z.device)
@@ -101,9 +106,10 @@ class StateSpace(Mixer):
         T, dev, H = h.shape[0], h.device, self.num_heads
         p = ops.scratch("ssd_in", (T, self.in_width), torch.float32, dev)
         ops.linear(h, self.w_in, p)
-        single = ctx.max_q_len == 1              # no request brings more than one token
+        single = ctx.max_q_len == 1 and T == ctx.num_requests       # every request brings one token
         x = ops.scratch("ssd_operands", (T, self.x_width), torch.float32, dev)
-        conv = ops.ShortConv(self.conv_w, state, self.s_floats, ctx.req_of_token, ctx.cu_seqlens_q, ctx.state_slots, single)
+        conv = ops.ShortConv(self.conv_w, state, self.s_floats, ctx.cu_seqlens_q, ctx.state_slots,
+                             None if single else ctx.attention_tiles(ops.CONV_RUN))
         ops.ssd_prepare(p, self.inner, self.inner + self.channels, conv, self.conv_b, self.a_log, self.dt_bias, x, self.dt_col,
                         self.a_col)
         if self.taps > 1 and not single:
@@ -113,7 +119,7 @@ class StateSpace(Mixer):
         b_off = self.inner
         ops.linear_recurrence(x, b_off + self.groups * self.dim, b_off, 0, state, ctx.cu_seqlens_q, ctx.state_slots, y, H,
                               self.groups, self.dim, self.vdim, a_off=self.a_col, c_off=self.dt_col, skip=self.skip,
-                              single=single)
+                              single=single, tiles=_chunks(ctx))
         z = ops.scratch("recurrence_gated", (T, self.inner), self.dtype, dev)
         ops.group_norm_gate(y, self.w_norm, p[:, :self.inner], z, self.norm_groups, self.eps, "silu", True, self.out_scale)
         return _project_out(self, z, residual)
@@ -170,7 +176,7 @@ class DecayedAttention(Mixer):
         ops.linear(h, self.w_in, p)
         o = ops.scratch("recurrence_out", (T, self.inner), torch.float32, dev)
         ops.linear_recurrence(p, 0, self.qk_size, self.v_off, state, ctx.cu_seqlens_q, ctx.state_slots, o, H, H, self.dim,
-                              self.vdim, decay=self.decay, silu=True, single=ctx.max_q_len == 1)
+                              self.vdim, decay=self.decay, silu=True, single=ctx.max_q_len == 1, tiles=_chunks(ctx))
         z = ops.scratch("recurrence_gated", (T, self.inner), self.dtype, dev)
         ops.group_norm_gate(o, self.w_norm, p[:, self.g_off:self.g_off + self.inner], z, 1, self.eps, "sigmoid", False,
                             self.out_scale)
