@@ -32,11 +32,13 @@ __device__ __forceinline__ int first_visible_key(int pos, int window) {
 
 // Which keys a row at position `pos` sees, and what happens to their scores: the keys from first_visible_key up to its
 // own, and, of the ones in front of those, the request's first `keep` (tokens a sliding window keeps for good);
-// cap > 0: a score s (scale applied) becomes cap * tanh(s / cap).
+// cap > 0: a score s (scale applied) becomes cap * tanh(s / cap).  out_scale: a constant on the result (float32, ahead of
+// its rounding).
 struct KeyMask {
   int window;
   int keep;
   float cap;
+  float out_scale;
 };
 __device__ __forceinline__ bool key_visible(int j, int pos, int row_lo, int keep) {
   return j <= pos && (j >= row_lo || j < keep);
@@ -136,7 +138,7 @@ __global__ __launch_bounds__(TL_WAVE) void paged_attention_kernel(
 #pragma unroll
   for (int i = 0; i < kDPL; ++i) {
     const int d = lane + i * TL_WAVE;
-    if (d < hd) store_result(out, orow + d, o[i] / l, sink);
+    if (d < hd) store_result(out, orow + d, o[i] * mask.out_scale / l, sink);
   }
 }
 
@@ -587,7 +589,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
     }
     if (n_splits == 1) {
       const float Ls = with_sink(L, M, sink);
-      store_result(out, (int64_t)t * out_stride + (int64_t)h * HD + d, Ls > 0.f ? acc / Ls : 0.f, sink);
+      store_result(out, (int64_t)t * out_stride + (int64_t)h * HD + d, Ls > 0.f ? acc * mask.out_scale / Ls : 0.f, sink);
     } else {
       part_o[(((int64_t)split * n_tokens + t) * nq + h) * HD + d] = acc;
       if (d == 0) {
@@ -870,7 +872,7 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_kernel(
     const int t = tok0 + t_local, h = kvh * G + h_local;
     if (gridDim.z == 1) {
       const float Ls = with_sink(Lrun[u], Mrun[u], sink);
-      out[(int64_t)t * out_stride + (int64_t)h * HD + d] = Ls > 0.f ? Orun[u] / Ls : 0.f;
+      out[(int64_t)t * out_stride + (int64_t)h * HD + d] = Ls > 0.f ? Orun[u] * mask.out_scale / Ls : 0.f;
     } else {
       float* pr = part + (((int64_t)blockIdx.z * n_tokens + t) * nq + h) * (HD + 2);
       pr[d] = Orun[u];
@@ -965,7 +967,7 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
 #pragma unroll
   for (int dt = 0; dt < HDT; ++dt)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) orow[dt * 16 + kk * 4 + r] = Ls > 0.f ? Orun[dt][r] / Ls : 0.f;
+    for (int r = 0; r < 4; ++r) orow[dt * 16 + kk * 4 + r] = Ls > 0.f ? Orun[dt][r] * mask.out_scale / Ls : 0.f;
 }
 
 // Merges the chunks that attention_f32_kernel left in `part` [chunks][tokens][heads][hd + 2], in
@@ -974,7 +976,7 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
 __global__ __launch_bounds__(TL_WAVE) void attention_f32_combine_kernel(const float* __restrict__ part,
                                                                        float* __restrict__ out, int64_t out_stride,
                                                                        int n_tokens, int nq, int hd, int n_chunks,
-                                                                       int sink) {
+                                                                       int sink, float out_scale) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   for (int d = lane; d < hd; d += TL_WAVE) {
     float M = kNegBig, L = 0.f, O = 0.f, wa, wb;
@@ -984,7 +986,7 @@ __global__ __launch_bounds__(TL_WAVE) void attention_f32_combine_kernel(const fl
       O = merge_f32_value(O, pr[d], wa, wb);
     }
     const float Ls = with_sink(L, M, sink);
-    out[(int64_t)t * out_stride + (int64_t)h * hd + d] = Ls > 0.f ? O / Ls : 0.f;
+    out[(int64_t)t * out_stride + (int64_t)h * hd + d] = Ls > 0.f ? O * out_scale / Ls : 0.f;
   }
 }
 
@@ -1347,7 +1349,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
       continue;
     }
     const float ls = with_sink(l, m_run[rt], sink);
-    const float inv = ls > 0.f ? 1.f / ls : 0.f;
+    const float inv = ls > 0.f ? mask.out_scale / ls : 0.f;
     const int64_t oat = (int64_t)tok[rt] * out_stride + (int64_t)head * HD + g * 4;
     if (sink & kFlagOutF32) {
       float* orow = reinterpret_cast<float*>(out) + oat;
@@ -1379,7 +1381,8 @@ template <int FC_BATCH>
 __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __restrict__ part_o,
                                                                 const float* __restrict__ part_ml,
                                                                 bf16_t* __restrict__ out, int64_t out_stride,
-                                                                int n_tokens, int nq, int hd, int n_splits, int sink) {
+                                                                int n_tokens, int nq, int hd, int n_splits, int sink,
+                                                                float out_scale) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int64_t row = (int64_t)t * nq + h, step = (int64_t)n_tokens * nq;      // split s: row + s * step
   // maxima are in units of log2 e; a split without keys has l = 0 and O = 0
@@ -1408,7 +1411,7 @@ __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __r
         }
       }
       const float Ls = with_sink(L, M, sink);
-      store_result(out, (int64_t)t * out_stride + (int64_t)h * hd + d, Ls > 0.f ? acc / Ls : 0.f, sink);
+      store_result(out, (int64_t)t * out_stride + (int64_t)h * hd + d, Ls > 0.f ? acc * out_scale / Ls : 0.f, sink);
     }
     return;
   }
@@ -1440,7 +1443,7 @@ __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __r
       }
     }
     const float Ls = with_sink(L, M, sink);
-    store_result(out, (int64_t)t * out_stride + (int64_t)h * hd + d, Ls > 0.f ? acc / Ls : 0.f, sink);
+    store_result(out, (int64_t)t * out_stride + (int64_t)h * hd + d, Ls > 0.f ? acc * out_scale / Ls : 0.f, sink);
   }
 }
 
@@ -1506,14 +1509,14 @@ extern "C" {
 int tl_paged_attention(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                        const int32_t* block_tables, int max_blocks, const int32_t* req_of_token,
                        const int32_t* positions, void* out, int64_t out_stride, int n_tokens, int nq,
-                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, int sink, int dtype,
+                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int dtype,
                        hipStream_t stream) {
   if (n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || hd <= 0 || hd > kMaxHd || block_size <= 0 || max_blocks <= 0 ||
       nq > 65535)
     return TL_ERR_ARG;
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
-  const KeyMask mask{window, keep, softcap};
+  const KeyMask mask{window, keep, softcap, out_scale};
   dim3 g(n_tokens, nq), b(TL_WAVE);
   if (dtype == 0)
     hipLaunchKernelGGL(paged_attention_kernel<float>, g, b, 0, stream, (const float*)q, q_stride,
@@ -1536,7 +1539,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
                      const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                      const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, float* out,
                      int64_t out_stride, float* part, int n_tiles, int n_tokens, int nq, int nkv, int hd,
-                     int block_size, float scale, int window, int keep, float softcap, int sink, int n_chunks, hipStream_t stream) {
+                     int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int n_chunks, hipStream_t stream) {
   if (n_tiles <= 0 || n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || nq / nkv > 16 || hd <= 0 || hd % 16 || hd > 128 || block_size <= 0 ||
       max_blocks <= 0 || n_chunks < 1 || nkv > 65535 || n_chunks > 65535 || q_stride % 4 ||
@@ -1546,7 +1549,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
   if (!tile_req && (tile_tok0 || tile_ntok || n_tiles != n_tokens)) return TL_ERR_ARG;
   if (tile_req && (!tile_tok0 || !tile_ntok)) return TL_ERR_ARG;
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
-  const KeyMask mask{window, keep, softcap};
+  const KeyMask mask{window, keep, softcap, out_scale};
   const size_t smem = (size_t)(A32_WAVES * FA_KT * A32_VS + A32_CHUNK * 16 * (hd + 4) + A32_CHUNK * 16 * 2) * sizeof(float);
   // Many query tiles (prompts): a wave a tile, four neighbouring tiles a workgroup; few (decode steps, small
   // steps): a workgroup a tile, its waves sharing the key tiles out.  The same bits either way.
@@ -1593,7 +1596,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
 #undef TL_A32_CASE
   if (n_chunks > 1)
     hipLaunchKernelGGL(attention_f32_combine_kernel, dim3(n_tokens, nq), dim3(TL_WAVE), 0, stream, part, out,
-                       out_stride, n_tokens, nq, hd, n_chunks, sink);
+                       out_stride, n_tokens, nq, hd, n_chunks, sink, out_scale);
   return tl_launch_status();
 }
 
@@ -1604,7 +1607,7 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
                      const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                      const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
                      int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq, int nkv,
-                     int hd, int block_size, float scale, int window, int keep, float softcap, int sink, int tile_waves, int n_splits,
+                     int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int tile_waves, int n_splits,
                      hipStream_t stream) {
   if (n_tiles <= 0) return TL_OK;
   if (tile_waves != 8 && tile_waves != 4) return TL_ERR_ARG;
@@ -1618,7 +1621,7 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
       out_stride % 4)
     return TL_ERR_ARG;
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
-  const KeyMask mask{window, keep, softcap};
+  const KeyMask mask{window, keep, softcap, out_scale};
   int bs_shift = -1;      // log2 of the page size where it is a power of two
   for (int sh = 0; sh < 31; ++sh)
     if ((1 << sh) == block_size) bs_shift = sh;
@@ -1643,7 +1646,7 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
 #undef TL_PREFILL_LAUNCH
 #define TL_COMBINE(B)                                                                                          \
   hipLaunchKernelGGL(flash_combine_kernel<B>, dim3(n_tokens, nq), dim3(TL_WAVE), 0, stream, part_o, part_ml, \
-                     (bf16_t*)out, out_stride, n_tokens, nq, hd, n_splits, sink)
+                     (bf16_t*)out, out_stride, n_tokens, nq, hd, n_splits, sink, out_scale)
   if (n_splits > 8) TL_COMBINE(16);
   else if (n_splits > 4) TL_COMBINE(8);
   else if (n_splits > 2) TL_COMBINE(4);
@@ -1663,7 +1666,7 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
                                const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                                const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
                                int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq,
-                               int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, int sink, int n_splits,
+                               int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int n_splits,
                                const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
   if (n_tiles <= 0 || n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || nq / nkv > 16 || hd <= 0 || hd % 16 || hd > 128 || block_size <= 0 ||
@@ -1678,7 +1681,7 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
   FusedRope fused{fuse_store ? rope_cos : nullptr, fuse_store ? rope_sin : nullptr, (bf16_t*)k_cache, (bf16_t*)v_cache,
                   nq * hd, (nq + nkv) * hd};
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
-  const KeyMask mask{window, keep, softcap};
+  const KeyMask mask{window, keep, softcap, out_scale};
   int rc = TL_ERR_ARG;
 #define TL_FLASH_CASE(HDT)                                                                                       \
   case HDT:                                                                                                      \
@@ -1695,7 +1698,7 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
   if (rc != TL_OK) return rc;
 #define TL_COMBINE(B)                                                                                          \
   hipLaunchKernelGGL(flash_combine_kernel<B>, dim3(n_tokens, nq), dim3(TL_WAVE), 0, stream, part_o, part_ml, \
-                     (bf16_t*)out, out_stride, n_tokens, nq, hd, n_splits, sink)
+                     (bf16_t*)out, out_stride, n_tokens, nq, hd, n_splits, sink, out_scale)
   if (n_splits > 8) TL_COMBINE(16);
   else if (n_splits > 4) TL_COMBINE(8);
   else if (n_splits > 2) TL_COMBINE(4);
@@ -1712,20 +1715,20 @@ int tl_flash_attention(const void* q, int64_t q_stride, const void* k_cache, con
                        const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
   return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                              positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
-                             scale, window, 0, 0.f, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+                             scale, window, 0, 0.f, 1.f, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
 }
 
 // The same with the rest of the mask: the request's first `keep` tokens stay visible behind a window, and softcap > 0
-// caps the scores, cap * tanh(score / cap).
+// caps the scores, cap * tanh(score / cap); the result is multiplied by out_scale.
 int tl_flash_attention_masked(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                        const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                        const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
                        int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq,
-                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, int sink, int n_splits,
+                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int n_splits,
                        const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
   return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                              positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
-                             scale, window, keep, softcap, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+                             scale, window, keep, softcap, out_scale, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
 }
 
 // ------------------------------------------------ the entry point that allocates nothing
@@ -1778,7 +1781,7 @@ int tl_flash_attention_static(const void* q, int64_t q_stride, const void* k_cac
   }
   return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                              positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
-                             scale, window, 0, 0.f, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+                             scale, window, 0, 0.f, 1.f, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
 }
 
 }  // extern "C"

@@ -565,14 +565,14 @@ __global__ __launch_bounds__(kThreads, NB <= 8 ? 3 : 2) void chunk_output_kernel
 template <typename T, int KEEP>
 __global__ __launch_bounds__(kThreads) void group_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w,
                                                                    const float* __restrict__ gate, int64_t gate_stride,
-                                                                   T* __restrict__ z, int width, int part, float eps,
+                                                                   T* __restrict__ z, int64_t z_stride, int width, int part, float eps,
                                                                    int gate_kind, int gate_first, float scale) {
   __shared__ float red[kThreads / TL_WAVE];
   const int t = blockIdx.x, c0 = blockIdx.y * part;
   const float* src = o + (int64_t)t * width + c0;
   const float* gp = gate + (int64_t)t * gate_stride + c0;
   const float* wp = w + c0;
-  T* dst = z + (int64_t)t * width + c0;
+  T* dst = z + (int64_t)t * z_stride + c0;
   auto act = [&](float g) {
     const float s = 1.f / (1.f + expf(-g));
     return gate_kind ? g * s : s;
@@ -741,9 +741,9 @@ int tl_linear_recurrence_chunks(const float* x, int64_t x_stride, int q_off, int
   return tl_launch_status();
 }
 
-// o: float32 [n_tokens, width]; w: float32 [width]; gate: float32, rows gate_stride apart; z: [n_tokens, width] in dtype.
-int tl_group_norm_gate(const float* o, const float* w, const float* gate, int64_t gate_stride, void* z, int n_tokens,
-                       int width, int groups, float eps, int gate_kind, int gate_first, float scale, int dtype,
+// o: float32 [n_tokens, width]; w: float32 [width]; gate: float32, rows gate_stride apart; z: [n_tokens, width] in dtype, rows z_stride apart.
+int tl_group_norm_gate(const float* o, const float* w, const float* gate, int64_t gate_stride, void* z,
+                       int64_t z_stride, int n_tokens, int width, int groups, float eps, int gate_kind, int gate_first, float scale, int dtype,
                        hipStream_t stream) {
   if (n_tokens <= 0) return TL_OK;
   if (width <= 0 || groups <= 0 || groups > 65535 || width % groups || gate_kind < 0 || gate_kind > 1 || !o || !w || !gate || !z)
@@ -751,7 +751,7 @@ int tl_group_norm_gate(const float* o, const float* w, const float* gate, int64_
   const int part = width / groups;
   dim3 g(n_tokens, groups), b(kThreads);
 #define TL_GNG(T, K)                                                                                                     \
-  hipLaunchKernelGGL((group_norm_gate_kernel<T, K>), g, b, 0, stream, o, w, gate, gate_stride, (T*)z, width, part, eps,   \
+  hipLaunchKernelGGL((group_norm_gate_kernel<T, K>), g, b, 0, stream, o, w, gate, gate_stride, (T*)z, z_stride, width, part, eps, \
                      gate_kind, gate_first, scale)
 #define TL_GNG_K(T)                         \
   if (part <= 2 * kThreads) TL_GNG(T, 2);   \

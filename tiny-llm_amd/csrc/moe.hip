@@ -293,20 +293,53 @@ __global__ __launch_bounds__(kThreads) void moe_gather_kernel(const bf16_t* __re
   }
 }
 
-// out[t, c] = base[t, c] * base_scale[t] + coef * sum_j row_w[t * top + j] * y[row_pos[t * top + j], c]
-__global__ void moe_combine_at_kernel(const float* __restrict__ y, const int32_t* __restrict__ row_pos,
-                                      const float* __restrict__ base, const float* __restrict__ base_scale,
-                                      const float* __restrict__ row_w, float* __restrict__ out, int64_t total, int N,
-                                      int top, float coef) {
-  const int64_t i = (int64_t)blockIdx.x * kThreads + threadIdx.x;
-  if (i >= total) return;
-  const int64_t t = i / N;
-  const int c = (int)(i - t * N);
-  float acc = 0.f;
-  for (int j = 0; j < top; ++j)
-    acc = fmaf(row_w ? row_w[t * top + j] : 1.f, y[(int64_t)row_pos[t * top + j] * N + c], acc);
-  const float b = base ? base[i] * (base_scale ? base_scale[t] : 1.f) : 0.f;
-  out[i] = fmaf(coef, acc, b);
+// out[t, c] = base[t, c] * base_scale[t] + coef * sum_j row_w[t * top + j] * y[row_pos[t * top + j], c] (row_pos null: the
+// rows of y lie in the table's order).  A workgroup takes VEC * kThreads columns of one token: which rows it adds is then
+// the same for all its threads, and up to four rows' vectors are requested together.
+template <int VEC>
+__global__ __launch_bounds__(kThreads) void moe_combine_rows_kernel(const float* __restrict__ y,
+                                                                    const int32_t* __restrict__ row_pos,
+                                                                    const float* __restrict__ base,
+                                                                    const float* __restrict__ base_scale,
+                                                                    const float* __restrict__ row_w, float* __restrict__ out,
+                                                                    int N, int top, float coef) {
+  typedef float vec __attribute__((ext_vector_type(VEC)));
+  const int t = blockIdx.x, c = (blockIdx.y * kThreads + threadIdx.x) * VEC;
+  if (c >= N) return;
+  const int64_t at = (int64_t)t * N + c;
+  vec b = {}, acc = {};
+  if (base) b = *(const vec*)(base + at);
+  for (int j0 = 0; j0 < top; j0 += 4) {
+    vec v[4];
+    float w[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j0 + j < top) {
+        const int i = t * top + j0 + j;
+        w[j] = row_w ? row_w[i] : 1.f;
+        v[j] = *(const vec*)(y + (int64_t)(row_pos ? row_pos[i] : i) * N + c);
+      }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j0 + j < top) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) acc[e] = fmaf(w[j], v[j][e], acc[e]);
+      }
+  }
+  const float bs = base_scale ? base_scale[t] : 1.f;
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) acc[e] = fmaf(coef, acc[e], base ? b[e] * bs : 0.f);
+  *(vec*)(out + at) = acc;
+}
+
+static void launch_combine(const float* y, const int32_t* row_pos, const float* base, const float* base_scale,
+                           const float* row_w, float* out, int n_tokens, int N, int top, float coef, hipStream_t stream) {
+  const bool vec = N % 4 == 0 && !(((uintptr_t)y | (uintptr_t)base | (uintptr_t)out) & 15);
+  dim3 g(n_tokens, (N / (vec ? 4 : 1) + kThreads - 1) / kThreads), b(kThreads);
+  if (vec)
+    hipLaunchKernelGGL(moe_combine_rows_kernel<4>, g, b, 0, stream, y, row_pos, base, base_scale, row_w, out, N, top, coef);
+  else
+    hipLaunchKernelGGL(moe_combine_rows_kernel<1>, g, b, 0, stream, y, row_pos, base, base_scale, row_w, out, N, top, coef);
 }
 
 // A workgroup ranks its rows inside every expert in LDS, takes one range per expert from the shared cursors and
@@ -389,21 +422,6 @@ __global__ __launch_bounds__(kThreads) void grouped_rows_gemm_bf16_kernel(
         if (c < N) orow[c] = from_f32<TO>(acc[rb][cb][i]);
       }
   }
-}
-
-// out[t, c] = base[t, c] * base_scale[t] + coef * sum_j row_w[t * top + j] * y[t * top + j, c]   (the experts in the
-// table's order)
-__global__ void moe_combine_kernel(const float* __restrict__ y, const float* __restrict__ base,
-                                   const float* __restrict__ base_scale, const float* __restrict__ row_w,
-                                   float* __restrict__ out, int64_t total, int N, int top, float coef) {
-  const int64_t i = (int64_t)blockIdx.x * kThreads + threadIdx.x;
-  if (i >= total) return;
-  const int64_t t = i / N;
-  const int c = (int)(i - t * N);
-  float acc = 0.f;
-  for (int j = 0; j < top; ++j) acc = fmaf(row_w ? row_w[t * top + j] : 1.f, y[(t * top + j) * N + c], acc);
-  const float b = base ? base[i] * (base_scale ? base_scale[t] : 1.f) : 0.f;
-  out[i] = fmaf(coef, acc, b);
 }
 
 // ------------------------------------------------------------------------------- a router
@@ -603,20 +621,16 @@ int tl_moe_gather(const void* a, int64_t a_stride, int a_div, void* dst, int32_t
 int tl_moe_combine_at(const float* y, const int32_t* row_pos, const float* base, const float* base_scale,
                       const float* row_w, float* out, int n_tokens, int N, int top, float coef, hipStream_t stream) {
   if (n_tokens <= 0) return TL_OK;
-  if (N <= 0 || top <= 0 || !y || !out || !row_pos) return TL_ERR_ARG;
-  const int64_t total = (int64_t)n_tokens * N;
-  hipLaunchKernelGGL(moe_combine_at_kernel, dim3((unsigned)ceil_div64(total, kThreads)), dim3(kThreads), 0, stream, y,
-                     row_pos, base, base_scale, row_w, out, total, N, top, coef);
+  if (N <= 0 || top <= 0 || !y || !out || !row_pos || (int64_t)n_tokens * top > 0x7fffffff || N > 65535 * kThreads) return TL_ERR_ARG;
+  launch_combine(y, row_pos, base, base_scale, row_w, out, n_tokens, N, top, coef, stream);
   return tl_launch_status();
 }
 
 int tl_moe_combine(const float* y, const float* base, const float* base_scale, const float* row_w, float* out,
                    int n_tokens, int N, int top, float coef, hipStream_t stream) {
   if (n_tokens <= 0) return TL_OK;
-  if (N <= 0 || top <= 0 || !y || !out) return TL_ERR_ARG;
-  const int64_t total = (int64_t)n_tokens * N;
-  hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)ceil_div64(total, kThreads)), dim3(kThreads), 0, stream, y, base,
-                     base_scale, row_w, out, total, N, top, coef);
+  if (N <= 0 || top <= 0 || !y || !out || (int64_t)n_tokens * top > 0x7fffffff || N > 65535 * kThreads) return TL_ERR_ARG;
+  launch_combine(y, nullptr, base, base_scale, row_w, out, n_tokens, N, top, coef, stream);
   return tl_launch_status();
 }
 

@@ -117,6 +117,61 @@ __global__ void gelu_table_rows_kernel(const float* __restrict__ gate, int64_t g
   z[i] = from_f32<T>(v);
 }
 
+// The product in front of it and gelu_table_rows_kernel in one, for few rows: a workgroup a column, eight rows at a time;
+// its threads stride over the inner size in vectors (a row's sum is formed in one order whatever else the step holds).
+constexpr int kGateRows = 8;
+template <typename T>
+__global__ __launch_bounds__(kThreads) void token_gate_kernel(const T* __restrict__ h, int64_t h_stride,
+                                                              const T* __restrict__ w, const int32_t* __restrict__ tokens,
+                                                              const T* __restrict__ table, int64_t table_stride, int off,
+                                                              T* __restrict__ z, int n_rows, int K, int dim, int wide, int vec) {
+  typedef T tvec __attribute__((ext_vector_type(8)));
+  __shared__ float red[kWaves][kGateRows];
+  const int j = blockIdx.x, tid = threadIdx.x, lane = tid % TL_WAVE, t0 = blockIdx.y * kGateRows;
+  const int n = min(kGateRows, n_rows - t0);
+  float acc[kGateRows], e = 0.f;
+#pragma unroll
+  for (int r = 0; r < kGateRows; ++r) acc[r] = 0.f;
+  if (j < dim) {
+    if (tid < n) e = to_f32(table[(int64_t)tokens[t0 + tid] * table_stride + off + j]);
+    const T* wr = w + (int64_t)j * K;
+    const T* hr[kGateRows];
+#pragma unroll
+    for (int r = 0; r < kGateRows; ++r) hr[r] = h + (int64_t)(t0 + min(r, n - 1)) * h_stride;
+    if (vec) {
+      for (int k = tid * 8; k < K; k += kThreads * 8) {
+        const tvec wv = *(const tvec*)(wr + k);
+        tvec hv[kGateRows];
+#pragma unroll
+        for (int r = 0; r < kGateRows; ++r) hv[r] = *(const tvec*)(hr[r] + k);
+#pragma unroll
+        for (int r = 0; r < kGateRows; ++r)
+#pragma unroll
+          for (int c = 0; c < 8; ++c) acc[r] = fmaf((float)hv[r][c], (float)wv[c], acc[r]);
+      }
+    } else {
+      for (int k = tid; k < K; k += kThreads) {
+        const float wv = to_f32(wr[k]);
+#pragma unroll
+        for (int r = 0; r < kGateRows; ++r) acc[r] = fmaf(to_f32(hr[r][k]), wv, acc[r]);
+      }
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < kGateRows; ++r) {
+    const float s = wave_sum(acc[r]);
+    if (lane == 0) red[tid / TL_WAVE][r] = s;
+  }
+  __syncthreads();
+  if (tid < n) {
+    float g = 0.f;
+#pragma unroll
+    for (int w4 = 0; w4 < kWaves; ++w4) g += red[w4][tid];
+    const float act = 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+    z[(int64_t)(t0 + tid) * wide + j] = from_f32<T>(j < dim ? act * e : 0.f);
+  }
+}
+
 __global__ void softcap_kernel(float* __restrict__ x, int64_t total, float cap) {
   const int64_t i = (int64_t)blockIdx.x * kThreads + threadIdx.x;
   if (i < total) x[i] = cap * tanhf(x[i] / cap);
@@ -220,6 +275,25 @@ int tl_gelu_table_rows(const float* gate, int64_t gate_stride, const int32_t* to
                        table_stride, off, (bf16_t*)z, total, dim, wide);
   else
     return TL_ERR_ARG;
+  return tl_launch_status();
+}
+
+// h: [n_rows, K], w: [>= dim, K], table, z as tl_gelu_table_rows; all in dtype.
+int tl_token_gate(const void* h, int64_t h_stride, const void* w, const int32_t* tokens, const void* table,
+                  int64_t table_stride, int off, void* z, int n_rows, int K, int dim, int wide, int dtype, hipStream_t stream) {
+  if (n_rows <= 0) return TL_OK;
+  if (dim <= 0 || wide < dim || K <= 0 || off < 0 || off + dim > table_stride || !h || !w || !tokens || !table || !z ||
+      (n_rows + kGateRows - 1) / kGateRows > 65535)
+    return TL_ERR_ARG;
+  dim3 g(wide, (n_rows + kGateRows - 1) / kGateRows), b(kThreads);
+  const int vec = K % 8 == 0 && h_stride % 8 == 0 && !(((uintptr_t)h | (uintptr_t)w) & 15);
+#define TL_GATE(T)                                                                                                      \
+  hipLaunchKernelGGL(token_gate_kernel<T>, g, b, 0, stream, (const T*)h, h_stride, (const T*)w, tokens, (const T*)table, \
+                     table_stride, off, (T*)z, n_rows, K, dim, wide, vec)
+  if (dtype == 0) TL_GATE(float);
+  else if (dtype == 1) TL_GATE(bf16_t);
+  else return TL_ERR_ARG;
+#undef TL_GATE
   return tl_launch_status();
 }
 

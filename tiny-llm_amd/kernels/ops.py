@@ -616,10 +616,12 @@ def _attn_types_ok(q, k_cache, v_cache, out) -> bool:
 def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                     block_tables: torch.Tensor, req_of_token: torch.Tensor, positions: torch.Tensor,
                     out: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, scale: float,
-                    window: int = 0, sink: bool = False, keep: int = 0, softcap: float = 0.0) -> torch.Tensor:
+                    window: int = 0, sink: bool = False, keep: int = 0, softcap: float = 0.0,
+                    out_scale: float = 1.0) -> torch.Tensor:
     """Causal attention of every row of q (at its absolute position) over its
     request's cached keys 0..position (the last `window` of them if window > 0; the request's first `keep`
     stay visible behind the window).  softcap > 0: every score s becomes softcap * tanh(s / softcap).
+    out_scale: a constant on the result.
     sink: the softmax's denominator has one more term, exp(0), that carries no value."""
     _dev(q, k_cache, v_cache, block_tables, req_of_token, positions, out)
     _rows_2d(q, "q")
@@ -646,7 +648,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         _ptr(q), c_int64(q.stride(0)), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
         c_int(block_tables.shape[1]), _ptr(req_of_token), _ptr(positions), _ptr(out), c_int64(out.stride(0)),
         c_int(T), c_int(num_heads), c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]),
-        c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_int(_attn_flags(sink, q, out)), c_int(_dt(q)),
+        c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), c_int(_attn_flags(sink, q, out)), c_int(_dt(q)),
         _stream()), "paged_attention")
     return out
 
@@ -664,7 +666,7 @@ def attention_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                   tiles, positions: torch.Tensor, out: torch.Tensor, num_heads: int, num_kv_heads: int,
                   head_dim: int, scale: float, window: int = 0, n_chunks: int = 1,
                   scratch: Optional[torch.Tensor] = None, sink: bool = False, keep: int = 0,
-                  softcap: float = 0.0) -> torch.Tensor:
+                  softcap: float = 0.0, out_scale: float = 1.0) -> torch.Tensor:
     """The same function as `paged_attention` in true float32 on the matrix cores.  `tiles` as for
     `flash_attention` (None: row i is the one new token of request i).  n_chunks == 1: one
     workgroup per tile and kv head walks all keys; n_chunks > 1 (at least ceil(longest context /
@@ -711,7 +713,7 @@ def attention_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         _ptr(q, 16), c_int64(q.stride(0)), _ptr(k_cache, 16), _ptr(v_cache, 16), _ptr(block_tables),
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out), c_int64(out.stride(0)), _ptr(scratch), c_int(n_tiles), c_int(T), c_int(num_heads),
-        c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_int(1 if sink else 0),
+        c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), c_int(1 if sink else 0),
         c_int(n_chunks), _stream()), "attention_f32")
     return out
 
@@ -726,7 +728,8 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     tiles, positions: torch.Tensor, out: torch.Tensor, num_heads: int, num_kv_heads: int,
                     head_dim: int, scale: float, window: int = 0, n_splits: int = 1,
                     scratch: Optional[torch.Tensor] = None, fused_rope=None, static_scratch: bool = False,
-                    sink: bool = False, keep: int = 0, softcap: float = 0.0) -> torch.Tensor:
+                    sink: bool = False, keep: int = 0, softcap: float = 0.0,
+                    out_scale: float = 1.0) -> torch.Tensor:
     """The same function as `paged_attention` on the matrix cores (bfloat16).  `tiles` =
     (tile_req, tile_tok0, tile_ntok): groups of at most 16 // (heads / kv_heads) consecutive
     tokens of one request; None for a decode step, where row i is the one new token of request i
@@ -793,7 +796,8 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         if not (q.stride(0) >= (num_heads + 2 * num_kv_heads) * head_dim):
             _fail("fused mode needs q inside its qkv rows")
     if static_scratch:
-        _need(keep == 0 and softcap == 0.0, "flash_attention: the static entry point takes no kept tokens and no soft cap")
+        _need(keep == 0 and softcap == 0.0 and out_scale == 1.0, "flash_attention: the static entry point takes no kept tokens, "
+              "no soft cap and no constant on the result")
         code = _lib().tl_flash_attention_static(
             _ptr(q, 16), c_int64(q.stride(0)), _ptr(k_cache, 16), _ptr(v_cache, 16), _ptr(block_tables),
             c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
@@ -810,7 +814,7 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out, 8), c_int64(out.stride(0)), _ptr(part_o), _ptr(part_ml), c_int(n_tiles), c_int(T),
         c_int(num_heads), c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale),
-        c_int(window), c_int(keep), c_float(softcap), c_int(_attn_flags(sink, q, out)), c_int(n_splits), _ptr(cos), _ptr(sin),
+        c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), c_int(_attn_flags(sink, q, out)), c_int(n_splits), _ptr(cos), _ptr(sin),
         c_int(1 if fused_rope is not None else 0), _stream()), "flash_attention")
     return out
 
@@ -901,7 +905,7 @@ def flash_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                   tiles, positions: torch.Tensor, out: torch.Tensor, num_heads: int, num_kv_heads: int,
                   head_dim: int, scale: float, window: int = 0, tile_waves: int = 8, n_splits: int = 1,
                   scratch: Optional[torch.Tensor] = None, sink: bool = False, keep: int = 0,
-                  softcap: float = 0.0) -> torch.Tensor:
+                  softcap: float = 0.0, out_scale: float = 1.0) -> torch.Tensor:
     """`flash_attention` arranged for prompt portions: `tiles` are groups of at most
     tile_waves * (16 // (heads / kv_heads)) consecutive tokens of one request, and a key or value
     row is staged once per such group.  tile_waves is PREFILL_TILES (8), or 4 for steps with few
@@ -951,7 +955,7 @@ def flash_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out, 16 if out.dtype == torch.float32 else 8), c_int64(out.stride(0)), _ptr(part_o, 16), _ptr(part_ml), c_int(n_tiles), c_int(T),
         c_int(num_heads), c_int(num_kv_heads),
-        c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_int(_attn_flags(sink, q, out)), c_int(tile_waves),
+        c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), c_int(_attn_flags(sink, q, out)), c_int(tile_waves),
         c_int(n_splits),
         _stream()), "flash_prefill")
     return out
@@ -1136,6 +1140,28 @@ def gelu_table_rows(gate: torch.Tensor, tokens: torch.Tensor, table: torch.Tenso
     _check(_lib().tl_gelu_table_rows(_ptr(gate), c_int64(gate.stride(0)), _ptr(tokens), _ptr(table), c_int64(table.shape[1]),
                                      c_int(off), _ptr(out), c_int(T), c_int(dim), c_int(out.shape[1]), c_int(_dt(table)),
                                      _stream()), "gelu_table_rows")
+    return out
+
+
+TOKEN_GATE_ROWS = 32        # up to this many rows the gate's product and what follows it are one kernel
+
+
+def token_gate(h: torch.Tensor, w: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, off: int, dim: int,
+               out: torch.Tensor) -> torch.Tensor:
+    """out[t, j] = gelu(w[j] . h[t]) * table[tokens[t], off + j] for j < dim, zeros in out's further columns: `linear` and
+    `gelu_table_rows` in one launch, for few rows.  h [T, W], w [>= dim, W], table and out of one type."""
+    _dev(h, w, tokens, table, out)
+    _rows_2d(h, "token_gate input")
+    _i32(tokens)
+    T, W = h.shape
+    _need(T == tokens.numel() and w.dim() == 2 and w.is_contiguous() and w.shape[1] == W and w.shape[0] >= dim > 0 and off >= 0
+          and table.dim() == 2 and table.is_contiguous() and off + dim <= table.shape[1] and out.dim() == 2
+          and out.is_contiguous() and out.shape[0] == T and out.shape[1] >= dim
+          and h.dtype == w.dtype == table.dtype == out.dtype, "token_gate: shapes do not fit")
+    al = 16 if W % 8 == 0 and h.stride(0) % 8 == 0 else 1
+    _check(_lib().tl_token_gate(_ptr(h, al), c_int64(h.stride(0)), _ptr(w, al), _ptr(tokens), _ptr(table),
+                                c_int64(table.shape[1]), c_int(off), _ptr(out), c_int(T), c_int(W), c_int(dim),
+                                c_int(out.shape[1]), c_int(_dt(h)), _stream()), "token_gate")
     return out
 
 
@@ -1938,17 +1964,18 @@ def group_norm_gate(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, o
                     gate_kind: str = "sigmoid", gate_first: bool = False, scale: float = 1.0) -> torch.Tensor:
     """Rows in `groups` equal parts, each divided by its own root mean square, times weight (one number a column) and
     scale; the gate act(gate) multiplies the row ahead of the norm (`gate_first`) or behind it, act "sigmoid" or "silu"
-    (g * sigmoid(g)).  o float32 [T, width] contiguous, gate float32 [T, width] (a view into wider rows is fine)."""
+    (g * sigmoid(g)).  o float32 [T, width] contiguous, gate float32 [T, width] and out [T, width] (views into wider rows are fine)."""
     _dev(o, weight, gate, out)
     T, width = out.shape
     _f32_vec(o, T * width, "group_norm_gate input")
     _f32_vec(weight, width, "group_norm_gate weight")
     _rows_2d(gate, "group_norm_gate gate")
+    _rows_2d(out, "group_norm_gate output")
     _need(gate_kind in ("sigmoid", "silu"), f"group_norm_gate: unknown gate {gate_kind!r}")
-    _need(gate.dtype == torch.float32 and tuple(gate.shape) == (T, width) and out.is_contiguous() and width % groups == 0,
+    _need(gate.dtype == torch.float32 and tuple(gate.shape) == (T, width) and width % groups == 0,
           "group_norm_gate: gate and output are [T, width], the parts equal")
-    _check(_lib().tl_group_norm_gate(_ptr(o), _ptr(weight), _ptr(gate), c_int64(gate.stride(0)), _ptr(out), c_int(T),
-                                     c_int(width), c_int(groups), c_float(eps), c_int(1 if gate_kind == "silu" else 0),
+    _check(_lib().tl_group_norm_gate(_ptr(o), _ptr(weight), _ptr(gate), c_int64(gate.stride(0)), _ptr(out),
+                                     c_int64(out.stride(0)), c_int(T), c_int(width), c_int(groups), c_float(eps), c_int(1 if gate_kind == "silu" else 0),
                                      c_int(1 if gate_first else 0), c_float(scale), c_int(_dt(out)), _stream()),
            "group_norm_gate")
     return out

@@ -96,13 +96,13 @@ class Attention(Mixer):
         out, prepared = project_into_residual(attn, self.w_o, residual, next_norm)
         return out if next_norm is None else (out, prepared)
 
-    def _attend(self, q, ctx, cache: LayerCache, attn, fused_rope=None, sink: bool = False):
+    def _attend(self, q, ctx, cache: LayerCache, attn, fused_rope=None, sink: bool = False, out_scale: float = 1.0):
         """attn <- attention of the step's query rows q [T, heads * head_dim] over the cache, by the kernel that
         takes this step's shape.  sink: one more term exp(0) in every softmax's denominator.  `self.window`: 0
         (every earlier key), n > 0 (the last n positions) or -n (the row's own run of n positions, runs counted
         from position 0: a chunked mask); the request's first `self.keep` positions are seen in any case.
-        `self.softcap` > 0: scores s become softcap * tanh(s / softcap)."""
-        mask = {"sink": sink, "keep": self.keep if self.window else 0, "softcap": self.softcap}
+        `self.softcap` > 0: scores s become softcap * tanh(s / softcap).  out_scale: a constant on the result."""
+        mask = {"sink": sink, "keep": self.keep if self.window else 0, "softcap": self.softcap, "out_scale": out_scale}
         T, device = q.shape[0], q.device
         group = self.num_heads // self.num_kv_heads
         flash = ops.flash_attention_supported(self.dtype, self.num_heads, self.num_kv_heads, self.head_dim)
@@ -431,10 +431,26 @@ class GatedAttention(Attention):
         channels = self.q_cols + self.k_cols + self.v_cols
         return StateSpec((-(-channels * (self.taps - 1) // 4) * 4,), torch.float32)
 
+    # the two products and what lies between them, by themselves: a mixer of several branches may join the branches'
+    # products (parts/parallel.py)
+    splits_products = True
+
     def forward(self, h, ctx, cache: LayerCache, state, residual):
-        T, dev, H = h.shape[0], h.device, self.num_heads
+        T, dev = h.shape[0], h.device
         p = ops.scratch("qk_product", (T, self.in_width), torch.float32, dev)
         ops.linear(h, self.w_in, p)
+        z = self.mix(p, ctx, cache, state, ops.scratch("attention_gated", (T, self.out_width), self.dtype, dev))
+        if residual is None:
+            return ops.linear(z, self.w_o, ops.scratch("sublayer_out", (T, self.hidden_size), torch.float32, dev))
+        return ops.linear(z, self.w_o, residual, residual)
+
+    @property
+    def out_width(self) -> int:
+        return self.out_cols + self.out_tail
+
+    def mix(self, p, ctx, cache: LayerCache, state, z):
+        """From the first product's rows p (float32 [T, in_width]) to the output product's operand z ([T, out_width])."""
+        T, dev, H = p.shape[0], p.device, self.num_heads
         tables = self.position.rotary_tables()
         cos, sin, rot = tables if tables is not None else (None, None, 0)
         pairing = getattr(self.position, "pairing", "half")
@@ -458,19 +474,18 @@ class GatedAttention(Attention):
                              cache.tensors["v"] if write else None, H, self.num_kv_heads, self.maps, self.qk_dim,
                              self.value_dim, self.v_off, rot, pairing, self.qk_norm == "whole", self.qk_norm == "unit",
                              self.eps, self.q_temp)
+        if self.maps == 1 and self.value_dim == self.head_dim and not (self.sub_norm or self.gate or self.out_tail):
+            # nothing lies behind the weighted sum but a constant: the attention kernel leaves the operand itself
+            return self._attend(q[0], ctx, cache, z, out_scale=self.out_scale)
         outs = []
         for m in range(self.maps):
             # float32 whatever the engine's type: the maps' difference, the head's norm and the gates follow in float32
             attn = ops.scratch("attention_out" if m == 0 else "attention_out2", (T, self.q_size), torch.float32, dev)
             view = LayerCache({"k": k_caches[m], "v": cache.tensors["v"]}, cache.group, cache.write)
             outs.append(self._attend(q[m], ctx, view, attn))
-        z = ops.scratch("attention_gated", (T, self.out_cols + self.out_tail), self.dtype, dev)
         gate = p[:, self.g_off:self.g_off + self.g_cols] if self.gate else None
-        ops.attn_finish(outs[0], outs[1] if self.maps == 2 else None, gate, z, H, self.value_dim, self.lam, self.sub_norm,
-                        self.eps, self.out_scale, self.gate, self.out_tail)
-        if residual is None:
-            return ops.linear(z, self.w_o, ops.scratch("sublayer_out", (T, self.hidden_size), torch.float32, dev))
-        return ops.linear(z, self.w_o, residual, residual)
+        return ops.attn_finish(outs[0], outs[1] if self.maps == 2 else None, gate, z, H, self.value_dim, self.lam, self.sub_norm,
+                               self.eps, self.out_scale, self.gate, self.out_tail)
 
 
 register_mixer("attention", Attention)

@@ -39,7 +39,11 @@ def _chunks(ctx):
     return ctx.attention_tiles(ops.LINEAR_CHUNK) if ctx.max_q_len >= ops.LINEAR_CHUNK_TOKENS else None
 
 
-def _project_out(part, z, residual):
+def _forward(part, h, ctx, state, residual):
+    """The first product, `mix`, the output product."""
+    T, dev = h.shape[0], h.device
+    p = ops.linear(h, part.w_in, ops.scratch("recurrence_in", (T, part.in_width), torch.float32, dev))
+    z = part.mix(p, ctx, None, state, ops.scratch("recurrence_gated", (T, part.out_width), part.dtype, dev))
     if residual is None:
         out = ops.scratch("sublayer_out", (z.shape[0], part.hidden_size), torch.float32, z.device)
         return ops.linear(z, part.w_o, out)
@@ -48,6 +52,7 @@ def _project_out(part, z, residual):
 
 class StateSpace(Mixer):
     graph_safe = True
+    splits_products = True
 
     def __init__(self, prefix, dtype, device, *, hidden_size: int, num_heads: int, groups: int, state_dim: int,
                  value_dim: int, conv_taps: int, norm_groups: int, eps: float, out_scale: float = 1.0,
@@ -73,6 +78,7 @@ class StateSpace(Mixer):
         self.dt_col = _pad(self.channels, 4)
         self.a_col = self.dt_col + _pad(self.num_heads, 4)
         self.x_width = self.a_col + _pad(self.num_heads, 4)
+        self.out_width = self.inner
         self.s_floats = self.num_heads * self.dim * self.vdim
         n = {k: k for k in ("in", "conv", "dt_bias", "A_log", "D", "norm", "o")}
         n["conv_b"] = "conv.b"
@@ -103,9 +109,11 @@ class StateSpace(Mixer):
         return StateSpec((_pad(self.s_floats + self.channels * (self.taps - 1), 4),), torch.float32)
 
     def forward(self, h, ctx, cache, state, residual):
-        T, dev, H = h.shape[0], h.device, self.num_heads
-        p = ops.scratch("ssd_in", (T, self.in_width), torch.float32, dev)
-        ops.linear(h, self.w_in, p)
+        return _forward(self, h, ctx, state, residual)
+
+    def mix(self, p, ctx, cache, state, z):
+        """From the first product's rows p (float32 [T, in_width]) to the output product's operand z ([T, out_width])."""
+        T, dev, H = p.shape[0], p.device, self.num_heads
         single = ctx.max_q_len == 1 and T == ctx.num_requests       # every request brings one token
         x = ops.scratch("ssd_operands", (T, self.x_width), torch.float32, dev)
         conv = ops.ShortConv(self.conv_w, state, self.s_floats, ctx.cu_seqlens_q, ctx.state_slots,
@@ -120,13 +128,12 @@ class StateSpace(Mixer):
         ops.linear_recurrence(x, b_off + self.groups * self.dim, b_off, 0, state, ctx.cu_seqlens_q, ctx.state_slots, y, H,
                               self.groups, self.dim, self.vdim, a_off=self.a_col, c_off=self.dt_col, skip=self.skip,
                               single=single, tiles=_chunks(ctx))
-        z = ops.scratch("recurrence_gated", (T, self.inner), self.dtype, dev)
-        ops.group_norm_gate(y, self.w_norm, p[:, :self.inner], z, self.norm_groups, self.eps, "silu", True, self.out_scale)
-        return _project_out(self, z, residual)
+        return ops.group_norm_gate(y, self.w_norm, p[:, :self.inner], z, self.norm_groups, self.eps, "silu", True, self.out_scale)
 
 
 class DecayedAttention(Mixer):
     graph_safe = True
+    splits_products = True
 
     def __init__(self, prefix, dtype, device, *, hidden_size: int, num_heads: int, head_dim: int, value_dim: int,
                  decay: Sequence[float], eps: float, out_scale: float = 1.0, names: Dict[str, str] = None):
@@ -144,6 +151,7 @@ class DecayedAttention(Mixer):
         self.v_off = 2 * self.qk_size
         self.g_off = _pad(self.v_off + self.inner, 8)
         self.in_width = _pad(self.g_off + self.inner, 8)
+        self.out_width = self.inner
         self.s_floats = self.num_heads * self.dim * self.vdim
         n = {k: k for k in ("q", "k", "v", "g", "norm", "o")}
         n.update(names or {})
@@ -171,16 +179,16 @@ class DecayedAttention(Mixer):
         return StateSpec((_pad(self.s_floats, 4),), torch.float32)
 
     def forward(self, h, ctx, cache, state, residual):
-        T, dev, H = h.shape[0], h.device, self.num_heads
-        p = ops.scratch("decayed_in", (T, self.in_width), torch.float32, dev)
-        ops.linear(h, self.w_in, p)
+        return _forward(self, h, ctx, state, residual)
+
+    def mix(self, p, ctx, cache, state, z):
+        """From the first product's rows p (float32 [T, in_width]) to the output product's operand z ([T, out_width])."""
+        T, dev, H = p.shape[0], p.device, self.num_heads
         o = ops.scratch("recurrence_out", (T, self.inner), torch.float32, dev)
         ops.linear_recurrence(p, 0, self.qk_size, self.v_off, state, ctx.cu_seqlens_q, ctx.state_slots, o, H, H, self.dim,
                               self.vdim, decay=self.decay, silu=True, single=ctx.max_q_len == 1, tiles=_chunks(ctx))
-        z = ops.scratch("recurrence_gated", (T, self.inner), self.dtype, dev)
-        ops.group_norm_gate(o, self.w_norm, p[:, self.g_off:self.g_off + self.inner], z, 1, self.eps, "sigmoid", False,
-                            self.out_scale)
-        return _project_out(self, z, residual)
+        return ops.group_norm_gate(o, self.w_norm, p[:, self.g_off:self.g_off + self.inner], z, 1, self.eps, "sigmoid", False,
+                                   self.out_scale)
 
 
 register_mixer("state_space", StateSpace)

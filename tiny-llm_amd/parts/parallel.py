@@ -6,6 +6,10 @@ before its output product) and adds into the `residual` it is given: the first b
 writes the sum's buffer, every further one adds to it, so the sum costs no kernel of its own.  At most one
 branch may keep a paged cache, which becomes the part's own; the branches' per-request states lie side by side
 in the part's state rows, and a branch is handed its own columns of them.
+
+Where every branch says `splits_products` (its first product, `mix` and its output product by themselves), the branches'
+first products are ONE product over the rows of all of them, and their output products ONE product over their operands
+side by side, which forms the sum of the branches on its way.
 """
 from __future__ import annotations
 
@@ -13,6 +17,7 @@ from typing import Dict, List, Optional, Sequence, Tuple
 
 import torch
 
+from ..kernels import ops
 from .base import MIXERS, CacheSpec, Mixer, StateSpec, WeightSpec, register_mixer
 
 
@@ -23,11 +28,13 @@ class ParallelMixer(Mixer):
         super().__init__(prefix, dtype, device)
         if not branches:
             raise ValueError(f"{prefix}: a parallel mixer needs at least one branch")
+        self.w_in = self.w_o = None
         self.branches: List[Mixer] = []
         for b in branches:
             params = dict(b.get("params") or {})
             params["out_scale"] = float(b.get("scale", 1.0))
             self.branches.append(MIXERS.get(b["kind"])(f"{prefix}.{b['name']}", dtype, device, **params))
+        self.joined = all(getattr(m, "splits_products", False) for m in self.branches)
         with_cache = [m for m in self.branches if m.cache_spec() is not None]
         with_state = [m for m in self.branches if m.state_spec() is not None]
         if len(with_cache) > 1:
@@ -58,6 +65,11 @@ class ParallelMixer(Mixer):
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         for m in self.branches:
             m.bind(tensors)
+        if self.joined:
+            self.w_in = torch.cat([m.w_in for m in self.branches], dim=0).contiguous()
+            self.w_o = torch.cat([m.w_o for m in self.branches], dim=1).contiguous()
+            for m in self.branches:
+                m.w_in = m.w_o = None
 
     def cache_spec(self) -> Optional[CacheSpec]:
         return self._cache_branch.cache_spec() if self._cache_branch is not None else None
@@ -72,10 +84,27 @@ class ParallelMixer(Mixer):
         return state if cols is None else state[:, cols[0]:cols[1]]
 
     def forward(self, h, ctx, cache, state, residual):
+        if self.joined:
+            return self._forward_joined(h, ctx, cache, state, residual)
         y = residual
         for m in self.branches:
             y = m.forward(h, ctx, cache if m is self._cache_branch else None, self._state_of(m, state), y)
         return y
+
+
+    def _forward_joined(self, h, ctx, cache, state, residual):
+        T, dev = h.shape[0], h.device
+        p = ops.linear(h, self.w_in, ops.scratch("parallel_in", (T, self.w_in.shape[0]), torch.float32, dev))
+        z = ops.scratch("parallel_out", (T, self.w_o.shape[1]), self.dtype, dev)
+        at_p = at_z = 0
+        for m in self.branches:
+            m.mix(p[:, at_p:at_p + m.in_width], ctx, cache if m is self._cache_branch else None, self._state_of(m, state),
+                  z[:, at_z:at_z + m.out_width])
+            at_p += m.in_width
+            at_z += m.out_width
+        if residual is None:
+            return ops.linear(z, self.w_o, ops.scratch("sublayer_out", (T, self.w_o.shape[0]), torch.float32, dev))
+        return ops.linear(z, self.w_o, residual, residual)
 
 
 register_mixer("parallel", ParallelMixer)

@@ -47,9 +47,12 @@ class TokenInput(FeedForward):
 
     def forward(self, h, ctx, residual):
         T, dev = h.shape[0], h.device
-        g = ops.linear(h, self.w_gate, ops.scratch("token_input_gate", (T, self.wide), torch.float32, dev))
-        z = ops.gelu_table_rows(g, ctx.tokens, self.table, self.offset, self.dim,
-                                ops.scratch("token_input_gated", (T, self.wide), self.dtype, dev))
+        z = ops.scratch("token_input_gated", (T, self.wide), self.dtype, dev)
+        if T <= ops.TOKEN_GATE_ROWS:            # few rows (decoding): the product, the gelu and the table's row in one kernel
+            ops.token_gate(h, self.w_gate, ctx.tokens, self.table, self.offset, self.dim, z)
+        else:
+            g = ops.linear(h, self.w_gate, ops.scratch("token_input_gate", (T, self.wide), torch.float32, dev))
+            ops.gelu_table_rows(g, ctx.tokens, self.table, self.offset, self.dim, z)
         out = ops.linear(z, self.w_proj, ops.scratch("sublayer_out", (T, self.hidden_size), torch.float32, dev))
         return out if residual is None else add_to_residual(residual, out)
 
