@@ -770,3 +770,24 @@ def test_long_memory_of_a_recurrence(kind, sizes):
             at += c
         err = (torch.cat(got).double() - want).abs().max() / want.abs().max()
         assert err < 1e-4, (cuts[:3], float(err))
+
+
+@pytest.mark.parametrize("name", ["lightning", "parallel"])
+def test_generation_of_models_with_one_kind_of_memory(name, tmp_path_factory):
+    """A model without any paged cache (state slots alone), and one with a window and states, through the scheduler with
+    more requests than slots, captured steps and chained decode steps."""
+    folder, cfg, w, reqs, ref, block = material(name, "float32", tmp_path_factory)
+    from tiny_llm_amd import Engine, SamplingParams
+    prompts = [reqs["r0"][:17], reqs["r1"][:61], reqs["r3"][:3]]
+    eng = Engine(folder, dtype="float32", kv_block_size=block, max_num_seqs=2, max_num_batched_tokens=64, max_model_len=256)
+    out = eng.generate(prompts, SamplingParams.greedy(24, ignore_eos=True))
+    for p, o in zip(prompts, out):
+        seq = list(p)
+        for _ in range(24):
+            seq.append(int(plain.forward(cfg, w, seq)[-1].argmax()))
+        assert o == seq[len(p):]
+    steps, peak = traces.mixed(reqs, seed=5)
+    runner = make_runner(folder, "float32", block, peak)
+    for use_graph in (False, True, True):
+        check(replay(runner, steps, use_graph=use_graph), steps, ref, TOL["float32"])
+        assert all_free(runner)
