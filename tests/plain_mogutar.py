@@ -178,7 +178,7 @@ MIXERS = {"parallel": parallel, "lightning": lightning}
 # ------------------------------------------------------------------------- experts
 def choose(s, correction, top: int, groups: int, keep: int):
     """s [E], one token's scores: the indices of its experts.  Choice scores are s + correction; of `groups` equal
-    runs of neighbours only the `keep` with the largest sums of two choice scores stay in."""
+    runs of neighbours only the `keep` whose two best experts together score highest stay in."""
     c = s + correction
     if groups > 1:
         per = c.numel() // groups

@@ -574,8 +574,8 @@ def test_conv_attn_prepare(dtype, dim, vdim, rot, taps, yarn):
 @pytest.mark.parametrize("experts,top,groups,keep", [(6, 2, 2, 1), (16, 3, 4, 2), (64, 6, 8, 3), (5, 5, 1, 1), (130, 4, 10, 1), (8, 2, 8, 3),
                                                      (1, 1, 1, 1), (12, 5, 4, 4)])
 def test_router_with_sigmoid_scores_and_a_correction(experts, top, groups, keep):
-    """Sigmoid scores; the correction decides (most choice scores are negative) and stays out of the weights; a group's
-    score is the sum of its two largest choice scores (groups of one expert: that one's); weights are not renormalized."""
+    """Sigmoid scores; the correction decides (most corrected scores are negative) and stays out of the weights; a group is
+    ranked by its two best experts together (groups of one expert: that one); the weights keep their size."""
     from tiny_llm_amd.kernels import ops
     g = torch.Generator().manual_seed(experts * 7 + top)
     T = 37

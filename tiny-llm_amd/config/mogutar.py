@@ -4,7 +4,7 @@ config.json of this design is nested: `layers` (the layers in order, each with `
 `lightning`; `mixer`, its sizes and constants, for `parallel` under `left` (attention) and `right` (state space) with
 `left_scale` and `right_scale`; and `mlp`, a mixture of experts or null for none); `token_side.dim` (the numbers per
 token and layer of the per-layer token input; absent: no layer has one); `norm.eps`; `vocab`; `width`.  Every size and
-constant that can differ between models of the design comes from there; a layer has its own.
+constant is read from there; a layer has its own.
 """
 from __future__ import annotations
 

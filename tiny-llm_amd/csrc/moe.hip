@@ -431,8 +431,8 @@ __global__ __launch_bounds__(kThreads) void grouped_rows_gemm_bf16_kernel(
 // are chosen, largest first (equal scores: the lower index first); ids[t, j] names them, and
 // wts[t, j] = s_j / (sum of the chosen s + 1e-20) * scale.
 // Options: sigmoid scores s = sigmoid(z); a correction per expert that is added to the score for every choice and
-// left out of the weights (choice scores may then be negative: whatever is out counts as minus infinity); a run's
-// score as the sum of its two largest choice scores; weights s_j * scale without the division.
+// left out of the weights (corrected scores may be negative: whatever is out ranks below all of them); a run ranked by
+// its two best experts together; weights s_j * scale without the division.
 constexpr int kMaxRouted = 1024;
 
 struct Best {

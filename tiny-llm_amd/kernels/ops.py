@@ -2249,7 +2249,7 @@ def moe_route(z: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, groups:
     among those, largest first (equal scores: the lower index first), and weights[t] (float32 [T, top]) =
     their scores / (their sum + 1e-20) * scale.
     Options: `score` "sigmoid" (s = sigmoid(z)); `correction` (float32 [E]) is added to the scores wherever experts or
-    runs are chosen, never to the weights; `group_top2`: a run's score is the sum of its two largest; `normalize` False:
+    runs are chosen, never to the weights; `group_top2`: a run is ranked by its two best experts together; `normalize` False:
     the weights are the scores * scale."""
     _dev(z, ids, weights, correction)
     _f32_vec(correction, z.shape[1], "moe_route correction")

@@ -18,8 +18,8 @@ makes the experts gated units down(silu(gate(h)) * up(h)) (tensors e<i>.gate|up|
 expert to the router's logits (tensor router<bias_suffix>).  With one group and scale 1 the weights are the softmax
 over the chosen logits alone: exp(z_j) / sum over the chosen of exp(z_i), whatever the other experts' logits are.
 `score="sigmoid"` (s = sigmoid(z)); `correction` (tensor correction: a number per expert added to the scores wherever
-experts or runs are chosen, left out of the weights); `group_score="top2"` (a run's score is the sum of its two largest
-choice scores); `normalize=False` (an expert weighs s_j * scale).
+experts or runs are chosen, left out of the weights); `group_score="top2"` (a run is ranked by its two best
+experts together); `normalize=False` (an expert weighs s_j * scale).
 """
 from __future__ import annotations
 
