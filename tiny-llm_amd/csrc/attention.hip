@@ -40,6 +40,9 @@ struct KeyMask {
   float cap;
   float out_scale;
 };
+// The bfloat16 kernels are compiled for the plain mask, for one with kept tokens, and for capped scores (with or without
+// kept tokens): the plain one would pay a tenth of its time for what it does not use.
+enum MaskKind { kMaskPlain = 0, kMaskKeeps = 1, kMaskCapped = 2 };
 __device__ __forceinline__ bool key_visible(int j, int pos, int row_lo, int keep) {
   return j <= pos && (j >= row_lo || j < keep);
 }
@@ -229,7 +232,7 @@ __device__ __forceinline__ bf16x8 rotate_chunk_regs(const bf16x8 x, const bf16x8
   return r;
 }
 
-template <int HDT, int WAVES, bool CAP>
+template <int HDT, int WAVES, int KIND>
 __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
     const bf16_t* __restrict__ q, int64_t q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
@@ -238,6 +241,8 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
     int64_t out_stride, float* __restrict__ part_o, float* __restrict__ part_ml, int nq, int nkv,
     int block_size, float scale, KeyMask mask, int sink, int n_splits, int n_tokens, const FusedRope fused) {
   constexpr int HD = HDT * 16;
+  constexpr bool CAP = KIND == kMaskCapped, KEEPS = KIND != kMaskPlain;
+  const int keep = KEEPS ? mask.keep : 0;
   constexpr int KS = (HD + 31) / 32;       // k-steps of the score product
   constexpr int VS = HD + FA_VPAD;         // row stride of a wave's V tile in LDS
   constexpr int WAVE_ELEMS = FA_KT * VS;   // a wave's LDS area: its V tile, [key][dim]
@@ -301,8 +306,8 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   // With kept first keys the numbers count the n_kept tiles of those, then the window's: number n is tile n,
   // or n + skip from n_kept on (without them skip is 0 and number and tile are one).
   const int stride = WAVES * n_splits, mine = split * WAVES + wave;
-  const int n_kept = kept_key_tiles(mask.keep, first_tile), skip = mask.keep > 0 ? first_tile - n_kept : 0;
-  const int it0 = mask.keep > 0 ? 0 : first_tile / stride;
+  const int n_kept = KEEPS ? kept_key_tiles(keep, first_tile) : 0, skip = keep > 0 ? first_tile - n_kept : 0;
+  const int it0 = keep > 0 ? 0 : first_tile / stride;
   const int iters = (last_tile - skip - mine + stride - 1) / stride - it0;      // may be <= 0: no tile
   // fused mode: the one new token of the tile, at position kv_end - 1
   const int new_pos = kv_end - 1;
@@ -352,7 +357,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   const bf16_t* finite_row = q + (int64_t)tok0 * q_stride + (int64_t)kvh * G * HD;
   auto tile_at = [&](int it) {
     const int n = (it0 + it) * stride + mine;
-    return n >= n_kept ? n + skip : n;
+    return KEEPS && n >= n_kept ? n + skip : n;
   };
   auto tile_base = [&](int it) { return tile_at(it) * FA_KT; };
   auto fetch = [&](int it, int pages_raw) {
@@ -362,7 +367,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
 #pragma unroll
     for (int kt = 0; kt < 4; ++kt) {
       const int row = kt * 16 + r16, j = base + row;
-      const bool k_in = (j >= kv_begin || j < mask.keep) && j < kv_end;
+      const bool k_in = (j >= kv_begin || (KEEPS && j < keep)) && j < kv_end;
       const int64_t off = row_offset(j, __shfl(pages, row, TL_WAVE));
       kp[kt] = k_cache + (k_in ? off : 0);
     }
@@ -373,7 +378,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
 #pragma unroll
     for (int c = 0; c < VCH; ++c) {
       const int f = c * TL_WAVE + lane, row = f / VCH, ch = f % VCH, j = base + row;
-      const bool v_in = (j >= kv_begin || j < mask.keep) && j < kv_end;
+      const bool v_in = (j >= kv_begin || (KEEPS && j < keep)) && j < kv_end;
       const int64_t off = row_offset(j, __shfl(pages, row, TL_WAVE));
       const bf16_t* vp = v_in ? v_cache + off : finite_row;
       if (do_rope && j == new_pos) vp = new_v;      // not in the cache yet
@@ -385,7 +390,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   // (Two tiles in flight per wave, in two register sets, were measured to gain nothing: what a
   // compute unit can have on its way from memory is the limit, about 40 GB/s.)
   if (iters > 0) {
-    if (it0 != 0 || mask.keep > 0) next_pages = pages_at(tile_base(0));
+    if (it0 != 0 || keep > 0) next_pages = pages_at(tile_base(0));
     fetch(0, next_pages);
     if (iters > 1) next_pages = pages_at(tile_base(1));
   }
@@ -488,7 +493,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int j = kt_idx * FA_KT + kt * 16 + g * 4 + r;
-          const bool ok = row_valid && key_visible(j, pos, row_lo, mask.keep);
+          const bool ok = row_valid && j <= pos && (j >= row_lo || (KEEPS && j < keep));
           if constexpr (CAP) sc[kt][r] = capped_score(sc[kt][r], cap_in, cap_out);
           const float sv = ok ? sc[kt][r] : -INFINITY;
           sc[kt][r] = sv;
@@ -589,7 +594,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
     }
     if (n_splits == 1) {
       const float Ls = with_sink(L, M, sink);
-      store_result(out, (int64_t)t * out_stride + (int64_t)h * HD + d, Ls > 0.f ? acc * mask.out_scale / Ls : 0.f, sink);
+      store_result(out, (int64_t)t * out_stride + (int64_t)h * HD + d, Ls > 0.f ? acc * (KEEPS ? mask.out_scale : 1.f) / Ls : 0.f, sink);
     } else {
       part_o[(((int64_t)split * n_tokens + t) * nq + h) * HD + d] = acc;
       if (d == 0) {
@@ -1000,7 +1005,7 @@ __global__ __launch_bounds__(TL_WAVE) void attention_f32_combine_kernel(const fl
 constexpr int FP_RT = 1;                      // query tiles (of 16 rows) per wave
 // waves (query tiles) of a workgroup: 8, or 4 where 8 would leave compute units without work
 
-template <int HDT, int WAVES, bool CAP>
+template <int HDT, int WAVES, int KIND>
 __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
     const bf16_t* __restrict__ q, int64_t q_stride, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
@@ -1009,6 +1014,8 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
     int64_t out_stride, float* __restrict__ part_o, float* __restrict__ part_ml, int n_tiles, int n_tokens,
     int n_splits, int nq, int nkv, int block_size, int bs_shift, float scale, KeyMask mask, int sink) {
   constexpr int HD = HDT * 16;
+  constexpr bool CAP = KIND == kMaskCapped, KEEPS = KIND != kMaskPlain;
+  const int keep = KEEPS ? mask.keep : 0;
   constexpr int KS = (HD + 31) / 32;
   constexpr int KP = KS * 32 + 8;
   // two staging buffers: the next key tile is written while the current one is worked on, so a
@@ -1040,12 +1047,12 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
   // Tiles of kept first keys come in front of the window's: the loop counts n_kept + (last - first) numbers, number n
   // is tile n, or n + skip from n_kept on (first_tile, last_tile are numbers from here on; without kept keys
   // number and tile are one).
-  const int n_kept = kept_key_tiles(mask.keep, first_tile), skip = mask.keep > 0 ? first_tile - n_kept : 0;
-  if (mask.keep > 0) {
+  const int n_kept = KEEPS ? kept_key_tiles(keep, first_tile) : 0, skip = keep > 0 ? first_tile - n_kept : 0;
+  if (keep > 0) {
     last_tile -= skip;
     first_tile = 0;
   }
-  auto tile_of = [&](int n) { return n >= n_kept ? n + skip : n; };
+  auto tile_of = [&](int n) { return KEEPS && n >= n_kept ? n + skip : n; };
   if (n_splits > 1) {       // this workgroup's share of the key tiles (possibly none)
     const int per = (last_tile - first_tile + n_splits - 1) / n_splits;
     first_tile = min(first_tile + split * per, last_tile);
@@ -1128,7 +1135,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
   // probability is an exact zero): so no load is predicated, which would make it a branch.
   auto key_row = [&](int n) {
     const int j = tile_of(n) * FA_KT + lane;
-    return min(j < mask.keep ? j : max(j, kv_begin), kv_end - 1);
+    return min(KEEPS && j < keep ? j : max(j, kv_begin), kv_end - 1);
   };
   auto page_of_row = [&](int n) {
     const int j = key_row(n);
@@ -1248,7 +1255,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int j = tile_j0 + kt * 16 + g * 4 + r;
-              const bool ok = row_valid[rt] && key_visible(j, pos[rt], row_lo[rt], mask.keep);
+              const bool ok = row_valid[rt] && j <= pos[rt] && (j >= row_lo[rt] || (KEEPS && j < keep));
               const float sv = ok ? sc[rt][kt][r] : -INFINITY;
               sc[rt][kt][r] = sv;
               m_tile = fmaxf(m_tile, sv);
@@ -1328,7 +1335,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
       // start is visible to every row
       const int tile_j0 = kt_idx * FA_KT;
       const bool no_mask = all_valid && tile_j0 + FA_KT - 1 <= wave_lo_pos &&
-                           (tile_j0 >= wave_hi_lo || tile_j0 + FA_KT <= mask.keep);
+                           (tile_j0 >= wave_hi_lo || (KEEPS && tile_j0 + FA_KT <= keep));
       if (no_mask) work_on_tile(std::false_type{});
       else work_on_tile(std::true_type{});
     }
@@ -1349,7 +1356,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
       continue;
     }
     const float ls = with_sink(l, m_run[rt], sink);
-    const float inv = ls > 0.f ? mask.out_scale / ls : 0.f;
+    const float inv = ls > 0.f ? (KEEPS ? mask.out_scale : 1.f) / ls : 0.f;
     const int64_t oat = (int64_t)tok[rt] * out_stride + (int64_t)head * HD + g * 4;
     if (sink & kFlagOutF32) {
       float* orow = reinterpret_cast<float*>(out) + oat;
@@ -1447,7 +1454,7 @@ __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __r
   }
 }
 
-template <int HDT, int WAVES, bool CAP>
+template <int HDT, int WAVES, int KIND>
 static int launch_flash_w(const bf16_t* q, int64_t q_stride, const bf16_t* k_cache, const bf16_t* v_cache,
                           const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                           const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, bf16_t* out,
@@ -1460,12 +1467,12 @@ static int launch_flash_w(const bf16_t* q, int64_t q_stride, const bf16_t* k_cac
                 "a wave's merge area must fit its staging area");
   static bool configured = false;
   if (!configured) {
-    if (hipFuncSetAttribute((const void*)flash_attn_bf16_kernel<HDT, WAVES, CAP>,
+    if (hipFuncSetAttribute((const void*)flash_attn_bf16_kernel<HDT, WAVES, KIND>,
                             hipFuncAttributeMaxDynamicSharedMemorySize, (int)stage) != hipSuccess)
       return TL_ERR_LAUNCH;
     configured = true;
   }
-  hipLaunchKernelGGL((flash_attn_bf16_kernel<HDT, WAVES, CAP>), dim3(n_tiles, nkv, n_splits), dim3(WAVES * TL_WAVE), stage,
+  hipLaunchKernelGGL((flash_attn_bf16_kernel<HDT, WAVES, KIND>), dim3(n_tiles, nkv, n_splits), dim3(WAVES * TL_WAVE), stage,
                      stream, q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                      positions, out, out_stride, part_o, part_ml, nq, nkv, block_size, scale, mask, sink, n_splits,
                      n_tokens, fused);
@@ -1480,7 +1487,7 @@ static int launch_flash_w(const bf16_t* q, int64_t q_stride, const bf16_t* k_cac
 // has few: measured on whole decode steps, batch 1 and 8 gain 1 %, batch 64 would lose 2 %.
 static int flash_waves(int hd, int groups) { return hd <= 64 && groups > 64 ? 8 : 4; }
 
-template <int HDT, bool CAP>
+template <int HDT, int KIND>
 static int launch_flash(const bf16_t* q, int64_t q_stride, const bf16_t* k_cache, const bf16_t* v_cache,
                         const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                         const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, bf16_t* out,
@@ -1489,16 +1496,19 @@ static int launch_flash(const bf16_t* q, int64_t q_stride, const bf16_t* k_cache
                         hipStream_t stream) {
   if constexpr (HDT <= 4) {
     if (flash_waves(HDT * 16, n_tiles * nkv) == 8)
-      return launch_flash_w<HDT, 8, CAP>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0,
+      return launch_flash_w<HDT, 8, KIND>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0,
                                     tile_ntok, positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv,
                                     block_size, scale, mask, sink, n_splits, fused, stream);
   }
-  return launch_flash_w<HDT, 4, CAP>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
+  return launch_flash_w<HDT, 4, KIND>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                                 positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, block_size,
                                 scale, mask, sink, n_splits, fused, stream);
 }
 
 static bool mask_ok(int keep, float softcap) { return keep >= 0 && softcap >= 0.f; }
+static MaskKind mask_kind(const KeyMask& m) {
+  return m.cap > 0.f ? kMaskCapped : m.keep > 0 || m.out_scale != 1.f ? kMaskKeeps : kMaskPlain;
+}
 
 }  // namespace
 
@@ -1622,21 +1632,24 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
     return TL_ERR_ARG;
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
   const KeyMask mask{window, keep, softcap, out_scale};
+  const MaskKind kind = mask_kind(mask);
   int bs_shift = -1;      // log2 of the page size where it is a power of two
   for (int sh = 0; sh < 31; ++sh)
     if ((1 << sh) == block_size) bs_shift = sh;
-#define TL_PREFILL_LAUNCH(HDT, W, CAP)                                                                            \
-  hipLaunchKernelGGL((flash_prefill_bf16_kernel<HDT, W, CAP>), dim3(n_tiles * nkv * n_splits), dim3(W * TL_WAVE), 0,   \
+#define TL_PREFILL_LAUNCH(HDT, W, KIND)                                                                           \
+  hipLaunchKernelGGL((flash_prefill_bf16_kernel<HDT, W, KIND>), dim3(n_tiles * nkv * n_splits), dim3(W * TL_WAVE), 0,   \
                      stream, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,          \
                      block_tables, max_blocks, tile_req, tile_tok0, tile_ntok, positions, (bf16_t*)out,           \
                      out_stride, part_o, part_ml, n_tiles, n_tokens, n_splits, nq, nkv, block_size, bs_shift,     \
                      scale, mask, sink)
 #define TL_PREFILL_CASE(HDT)                        \
   case HDT:                                         \
-    if (softcap > 0.f && tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, true); \
-    else if (softcap > 0.f) TL_PREFILL_LAUNCH(HDT, 4, true);               \
-    else if (tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, false);            \
-    else TL_PREFILL_LAUNCH(HDT, 4, false);                                 \
+    if (kind == kMaskCapped && tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, kMaskCapped);     \
+    else if (kind == kMaskCapped) TL_PREFILL_LAUNCH(HDT, 4, kMaskCapped);                   \
+    else if (kind == kMaskKeeps && tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, kMaskKeeps);  \
+    else if (kind == kMaskKeeps) TL_PREFILL_LAUNCH(HDT, 4, kMaskKeeps);                     \
+    else if (tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, kMaskPlain);                        \
+    else TL_PREFILL_LAUNCH(HDT, 4, kMaskPlain);                                             \
     break;
   switch (hd / 16) {
     TL_PREFILL_CASE(1) TL_PREFILL_CASE(2) TL_PREFILL_CASE(3) TL_PREFILL_CASE(4)
@@ -1682,10 +1695,13 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
                   nq * hd, (nq + nkv) * hd};
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
   const KeyMask mask{window, keep, softcap, out_scale};
+  const MaskKind kind = mask_kind(mask);
   int rc = TL_ERR_ARG;
 #define TL_FLASH_CASE(HDT)                                                                                       \
   case HDT:                                                                                                      \
-    rc = (softcap > 0.f ? launch_flash<HDT, true> : launch_flash<HDT, false>)((const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,           \
+    rc = (kind == kMaskCapped  ? launch_flash<HDT, kMaskCapped>                                                   \
+          : kind == kMaskKeeps ? launch_flash<HDT, kMaskKeeps>                                                   \
+                               : launch_flash<HDT, kMaskPlain>)((const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,           \
                            block_tables, max_blocks, tile_req, tile_tok0, tile_ntok, positions, (bf16_t*)out,    \
                            out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, block_size, scale, mask, sink,   \
                            n_splits, fused, stream);                                                             \
