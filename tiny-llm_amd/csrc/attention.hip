@@ -41,8 +41,9 @@ struct KeyMask {
   float out_scale;
 };
 // The bfloat16 kernels are compiled for the plain mask, for one with kept tokens, and for capped scores (with or without
-// kept tokens): the plain one would pay a tenth of its time for what it does not use.
-enum MaskKind { kMaskPlain = 0, kMaskKeeps = 1, kMaskCapped = 2 };
+// kept tokens): the plain one would pay a tenth of its time for what it does not use.  kMaskFinished is the plain mask with
+// a result that is more than divided by its denominator (`Finish`); the kinds other than kMaskPlain all allow for that.
+enum MaskKind { kMaskPlain = 0, kMaskKeeps = 1, kMaskCapped = 2, kMaskFinished = 3 };
 __device__ __forceinline__ bool key_visible(int j, int pos, int row_lo, int keep) {
   return j <= pos && (j >= row_lo || j < keep);
 }
@@ -57,11 +58,28 @@ __device__ __forceinline__ float capped_score(float s, float c_in, float c_out) 
   return c_out * __builtin_fmaf(-2.f, __builtin_amdgcn_rcpf(1.f + e), 1.f);
 }
 
-// The `sink` argument of every entry point and kernel here is a set of flags: bit 0, the softmax's denominator has
+// The `sink` argument of every entry point here is a set of flags: bit 0, the softmax's denominator has
 // one more term (the sink); bit 1 (the general kernel and the bfloat16 kernels), the result leaves as float32
 // whatever the type of queries and cache (`out` then points to floats, out_stride counts floats): for a caller
 // that goes on in float32 with it (a difference of two maps, a norm per head).
 constexpr int kFlagSink = 1, kFlagOutF32 = 2;
+
+// How a row's weighted sum leaves a kernel.  The sink's term is exp(sinks[head]) (no `sinks`: exp(0)), whatever the scale
+// and the cap of the scores; the result is multiplied by sigmoid(gate[token, head]) (float32, rows gate_stride apart; null:
+// no gate); of a head's columns the first `vdim` are kept, and the heads lie side by side in rows of vdim.
+struct Finish {
+  int flags;
+  const float* sinks;
+  const float* gate;
+  int64_t gate_stride;
+  int vdim;
+};
+constexpr float kLog2e = 1.44269504088896341f;
+// the sink's score of a head, and the factor on a head's result
+__device__ __forceinline__ float sink_score(const Finish& fin, int h) { return fin.sinks ? fin.sinks[h] : 0.f; }
+__device__ __forceinline__ float gate_factor(const Finish& fin, int64_t t, int h) {
+  return fin.gate ? 1.f / (1.f + expf(-fin.gate[t * fin.gate_stride + h])) : 1.f;
+}
 template <typename T>
 __device__ __forceinline__ void store_result(T* out, int64_t at, float v, int flags) {
   if (flags & kFlagOutF32) reinterpret_cast<float*>(out)[at] = v;
@@ -77,7 +95,7 @@ __global__ __launch_bounds__(TL_WAVE) void paged_attention_kernel(
     const T* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ req_of_token, const int32_t* __restrict__ positions,
     T* __restrict__ out, int64_t out_stride, int nq, int nkv, int hd, int block_size, float scale,
-    KeyMask mask, int sink) {
+    KeyMask mask, const Finish fin) {
   __shared__ float qs[kMaxHd];
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int r = req_of_token[t];
@@ -135,13 +153,14 @@ __global__ __launch_bounds__(TL_WAVE) void paged_attention_kernel(
     base += TL_WAVE;
     if (end == kept_end && base >= kept_end) base = kv_begin;
   }
-  // a sink: one more term in the denominator, exp(0 - m) in the scores' own scale, that carries no value
-  if (sink & kFlagSink) l += expf(-m);
-  const int64_t orow = (int64_t)t * out_stride + (int64_t)h * hd;
+  // a sink: one more term in the denominator, exp(its score - m), that carries no value
+  if (fin.flags & kFlagSink) l += expf(sink_score(fin, h) - m);
+  const float f = mask.out_scale * gate_factor(fin, t, h);
+  const int64_t orow = (int64_t)t * out_stride + (int64_t)h * fin.vdim;
 #pragma unroll
   for (int i = 0; i < kDPL; ++i) {
     const int d = lane + i * TL_WAVE;
-    if (d < hd) store_result(out, orow + d, o[i] * mask.out_scale / l, sink);
+    if (d < fin.vdim) store_result(out, orow + d, o[i] * f / l, fin.flags);
   }
 }
 
@@ -171,11 +190,11 @@ constexpr int FA_KT = 64;
 constexpr int FA_VPAD = 8;      // padding of a row of the row-major V tile in LDS (elements)
 constexpr float kNegBig = -1.0e30f;   // "no key yet": finite, so exp2(m - m') never sees inf - inf
 
-// A sink: one more term in the softmax's denominator, with score 0 and no value.  l is the sum of
-// exp2(s - m) over the keys, m in units of log2 e; the term is exp2(0 - m) (infinite for a very negative m,
+// A sink: one more term in the softmax's denominator, with a score of its own and no value.  l is the sum of
+// exp2(s - m) over the keys, m in units of log2 e; the term is exp2(score * log2 e - m) (infinite for an m far below,
 // which makes the result the zero it then is).
-__device__ __forceinline__ float with_sink(float l, float m, int sink) {
-  return (sink & kFlagSink) ? l + __builtin_amdgcn_exp2f(-m) : l;
+__device__ __forceinline__ float with_sink(float l, float m, int flags, float score) {
+  return (flags & kFlagSink) ? l + __builtin_amdgcn_exp2f(score * kLog2e - m) : l;
 }
 
 // Two probabilities as two bfloat16 terms each, p = hi + lo, packed pairwise.  hi is p with the low
@@ -239,9 +258,9 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
     const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
     const int32_t* __restrict__ tile_ntok, const int32_t* __restrict__ positions, bf16_t* __restrict__ out,
     int64_t out_stride, float* __restrict__ part_o, float* __restrict__ part_ml, int nq, int nkv,
-    int block_size, float scale, KeyMask mask, int sink, int n_splits, int n_tokens, const FusedRope fused) {
+    int block_size, float scale, KeyMask mask, const Finish fin, int n_splits, int n_tokens, const FusedRope fused) {
   constexpr int HD = HDT * 16;
-  constexpr bool CAP = KIND == kMaskCapped, KEEPS = KIND != kMaskPlain;
+  constexpr bool CAP = KIND == kMaskCapped, KEEPS = KIND == kMaskKeeps || CAP, FIN = KIND != kMaskPlain;
   const int keep = KEEPS ? mask.keep : 0;
   constexpr int KS = (HD + 31) / 32;       // k-steps of the score product
   constexpr int VS = HD + FA_VPAD;         // row stride of a wave's V tile in LDS
@@ -295,6 +314,12 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
     }
   }
   const int row_lo = first_visible_key(pos, mask.window);
+  // what the end of the kernel needs of this lane's row is requested here, too
+  float row_sink = 0.f, row_gate = 0.f;
+  if constexpr (FIN) {
+    if (fin.sinks) row_sink = fin.sinks[min(head, nq - 1)];
+    if (fin.gate) row_gate = fin.gate[(int64_t)tok * fin.gate_stride + min(head, nq - 1)];
+  }
 
   // key range of the tile: union over its rows
   const int hi = row_max_i32(pos), lo = row_min_i32(row_valid ? row_lo : 0x7fffffff);
@@ -562,7 +587,7 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   __syncthreads();      // the merge below writes over the staging areas
 
   // merge the waves: each leaves (m, l, O[16][HD]) as floats in its own LDS area
-  constexpr int MROW = HD + 2;
+  constexpr int MROW = HD + (FIN ? 4 : 2);
   float* Mw = (float*)(smem + wave * WAVE_ELEMS);
 #pragma unroll
   for (int dt = 0; dt < HDT; ++dt)
@@ -571,6 +596,10 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
   if (g == 0) {
     Mw[r16 * MROW + HD] = m_run;
     Mw[r16 * MROW + HD + 1] = l_run;
+    if constexpr (FIN) {
+      Mw[r16 * MROW + HD + 2] = row_sink;
+      Mw[r16 * MROW + HD + 3] = fin.gate ? mask.out_scale / (1.f + expf(-row_gate)) : mask.out_scale;
+    }
   }
   __syncthreads();
   for (int e = tid; e < 16 * HD; e += WAVES * TL_WAVE) {      // one output element a thread
@@ -593,8 +622,16 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_attn_bf16_kernel(
       acc += wgt * area[d];
     }
     if (n_splits == 1) {
-      const float Ls = with_sink(L, M, sink);
-      store_result(out, (int64_t)t * out_stride + (int64_t)h * HD + d, Ls > 0.f ? acc * (KEEPS ? mask.out_scale : 1.f) / Ls : 0.f, sink);
+      float score = 0.f, f = 1.f;
+      if constexpr (FIN) {
+        const float* first = (const float*)smem + row * MROW;
+        score = first[HD + 2];
+        f = first[HD + 3];
+      }
+      const float Ls = with_sink(L, M, fin.flags, score);
+      const int width = FIN ? fin.vdim : HD;
+      if (!FIN || d < width)
+        store_result(out, (int64_t)t * out_stride + (int64_t)h * width + d, Ls > 0.f ? acc * f / Ls : 0.f, fin.flags);
     } else {
       part_o[(((int64_t)split * n_tokens + t) * nq + h) * HD + d] = acc;
       if (d == 0) {
@@ -781,8 +818,8 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_kernel(
     const float* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
     const int32_t* __restrict__ tile_ntok, const int32_t* __restrict__ positions, float* __restrict__ out,
-    int64_t out_stride, float* __restrict__ part, int nq, int nkv, int block_size, float scale, KeyMask mask, int sink,
-    int n_tokens) {
+    int64_t out_stride, float* __restrict__ part, int nq, int nkv, int block_size, float scale, KeyMask mask,
+    const Finish fin, int n_tokens) {
   constexpr int HD = HDT * 16;
   constexpr int PS = HD + 4;                       // row stride of a tile's O in LDS
   constexpr int EPT = 16 * HD / A32_THREADS;       // output elements a thread merges (= HDT)
@@ -876,8 +913,8 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_kernel(
     if (t_local >= TW || t_local >= ntok) continue;
     const int t = tok0 + t_local, h = kvh * G + h_local;
     if (gridDim.z == 1) {
-      const float Ls = with_sink(Lrun[u], Mrun[u], sink);
-      out[(int64_t)t * out_stride + (int64_t)h * HD + d] = Ls > 0.f ? Orun[u] * mask.out_scale / Ls : 0.f;
+      const float Ls = with_sink(Lrun[u], Mrun[u], fin.flags, sink_score(fin, h)), f = mask.out_scale * gate_factor(fin, t, h);
+      if (d < fin.vdim) out[(int64_t)t * out_stride + (int64_t)h * fin.vdim + d] = Ls > 0.f ? Orun[u] * f / Ls : 0.f;
     } else {
       float* pr = part + (((int64_t)blockIdx.z * n_tokens + t) * nq + h) * (HD + 2);
       pr[d] = Orun[u];
@@ -902,7 +939,7 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
     const float* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
     const int32_t* __restrict__ tile_ntok, const int32_t* __restrict__ positions, float* __restrict__ out,
-    int64_t out_stride, int nq, int nkv, int block_size, float scale, KeyMask mask, int sink, int n_tiles) {
+    int64_t out_stride, int nq, int nkv, int block_size, float scale, KeyMask mask, const Finish fin, int n_tiles) {
   constexpr int HD = HDT * 16;
   extern __shared__ __attribute__((aligned(16))) float smem32[];
   const int tid = threadIdx.x, lane = tid % TL_WAVE, wave = tid / TL_WAVE;
@@ -967,12 +1004,16 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
       for (int r = 0; r < 4; ++r) Orun[dt][r] = merge_f32_value(Orun[dt][r], Oc[dt][r], wa, wb);
   }
   if (!row_valid) return;
-  float* orow = out + (int64_t)tok * out_stride + (int64_t)(kvh * G + hh) * HD;
-  const float Ls = with_sink(Lrun, Mrun, sink);
+  const int h = kvh * G + hh;
+  float* orow = out + (int64_t)tok * out_stride + (int64_t)h * fin.vdim;
+  const float Ls = with_sink(Lrun, Mrun, fin.flags, sink_score(fin, h)), f = mask.out_scale * gate_factor(fin, tok, h);
 #pragma unroll
   for (int dt = 0; dt < HDT; ++dt)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) orow[dt * 16 + kk * 4 + r] = Ls > 0.f ? Orun[dt][r] * mask.out_scale / Ls : 0.f;
+    for (int r = 0; r < 4; ++r) {
+      const int d = dt * 16 + kk * 4 + r;
+      if (d < fin.vdim) orow[d] = Ls > 0.f ? Orun[dt][r] * f / Ls : 0.f;
+    }
 }
 
 // Merges the chunks that attention_f32_kernel left in `part` [chunks][tokens][heads][hd + 2], in
@@ -981,17 +1022,18 @@ __global__ __launch_bounds__(A32_THREADS) void attention_f32_rows_kernel(
 __global__ __launch_bounds__(TL_WAVE) void attention_f32_combine_kernel(const float* __restrict__ part,
                                                                        float* __restrict__ out, int64_t out_stride,
                                                                        int n_tokens, int nq, int hd, int n_chunks,
-                                                                       int sink, float out_scale) {
+                                                                       const Finish fin, float out_scale) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
-  for (int d = lane; d < hd; d += TL_WAVE) {
+  const float score = sink_score(fin, h), f = out_scale * gate_factor(fin, t, h);
+  for (int d = lane; d < fin.vdim; d += TL_WAVE) {
     float M = kNegBig, L = 0.f, O = 0.f, wa, wb;
     for (int c = 0; c < n_chunks; ++c) {
       const float* pr = part + (((int64_t)c * n_tokens + t) * nq + h) * (hd + 2);
       merge_f32(M, L, pr[hd], pr[hd + 1], wa, wb);
       O = merge_f32_value(O, pr[d], wa, wb);
     }
-    const float Ls = with_sink(L, M, sink);
-    out[(int64_t)t * out_stride + (int64_t)h * hd + d] = Ls > 0.f ? O * out_scale / Ls : 0.f;
+    const float Ls = with_sink(L, M, fin.flags, score);
+    out[(int64_t)t * out_stride + (int64_t)h * fin.vdim + d] = Ls > 0.f ? O * f / Ls : 0.f;
   }
 }
 
@@ -1012,9 +1054,9 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
     const int32_t* __restrict__ tile_req, const int32_t* __restrict__ tile_tok0,
     const int32_t* __restrict__ tile_ntok, const int32_t* __restrict__ positions, bf16_t* __restrict__ out,
     int64_t out_stride, float* __restrict__ part_o, float* __restrict__ part_ml, int n_tiles, int n_tokens,
-    int n_splits, int nq, int nkv, int block_size, int bs_shift, float scale, KeyMask mask, int sink) {
+    int n_splits, int nq, int nkv, int block_size, int bs_shift, float scale, KeyMask mask, const Finish fin) {
   constexpr int HD = HDT * 16;
-  constexpr bool CAP = KIND == kMaskCapped, KEEPS = KIND != kMaskPlain;
+  constexpr bool CAP = KIND == kMaskCapped, KEEPS = KIND == kMaskKeeps || CAP, FIN = KIND != kMaskPlain;
   const int keep = KEEPS ? mask.keep : 0;
   constexpr int KS = (HD + 31) / 32;
   constexpr int KP = KS * 32 + 8;
@@ -1355,10 +1397,36 @@ __global__ __launch_bounds__(WAVES * TL_WAVE) void flash_prefill_bf16_kernel(
       }
       continue;
     }
-    const float ls = with_sink(l, m_run[rt], sink);
-    const float inv = ls > 0.f ? (KEEPS ? mask.out_scale : 1.f) / ls : 0.f;
+    float f = 1.f, score = 0.f;
+    if constexpr (FIN) {
+      score = sink_score(fin, head);
+      f = mask.out_scale * gate_factor(fin, tok[rt], head);
+    }
+    const float ls = with_sink(l, m_run[rt], fin.flags, score);
+    const float inv = ls > 0.f ? f / ls : 0.f;
+    if constexpr (FIN) {
+      if (fin.vdim < HD) {            // the head's first columns only
+        const int64_t at = (int64_t)tok[rt] * out_stride + (int64_t)head * fin.vdim;
+        const bool rows4 = fin.vdim % 4 == 0 && !(fin.flags & kFlagOutF32);
+#pragma unroll
+        for (int dt = 0; dt < HDT; ++dt) {
+          const int d0 = dt * 16 + g * 4;
+          if (rows4) {
+            bf16x4 v4;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v4[r] = (bf16_t)(o[rt][dt][r] * inv);
+            if (d0 < fin.vdim) *(bf16x4*)(out + at + d0) = v4;
+          } else {
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+              if (d0 + r < fin.vdim) store_result(out, at + d0 + r, o[rt][dt][r] * inv, fin.flags);
+          }
+        }
+        continue;
+      }
+    }
     const int64_t oat = (int64_t)tok[rt] * out_stride + (int64_t)head * HD + g * 4;
-    if (sink & kFlagOutF32) {
+    if (fin.flags & kFlagOutF32) {
       float* orow = reinterpret_cast<float*>(out) + oat;
 #pragma unroll
       for (int dt = 0; dt < HDT; ++dt) {
@@ -1388,9 +1456,10 @@ template <int FC_BATCH>
 __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __restrict__ part_o,
                                                                 const float* __restrict__ part_ml,
                                                                 bf16_t* __restrict__ out, int64_t out_stride,
-                                                                int n_tokens, int nq, int hd, int n_splits, int sink,
-                                                                float out_scale) {
+                                                                int n_tokens, int nq, int hd, int n_splits,
+                                                                const Finish fin, float out_scale) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+  const float score = sink_score(fin, h), f = out_scale * gate_factor(fin, t, h);
   const int64_t row = (int64_t)t * nq + h, step = (int64_t)n_tokens * nq;      // split s: row + s * step
   // maxima are in units of log2 e; a split without keys has l = 0 and O = 0
   if (n_splits <= FC_BATCH) {      // the usual case: ONE round trip, the maximum comes from the same loads
@@ -1401,7 +1470,7 @@ __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __r
       m[u] = part_ml[base * 2];
       l[u] = part_ml[base * 2 + 1];
     }
-    for (int d = lane; d < hd; d += TL_WAVE) {
+    for (int d = lane; d < fin.vdim; d += TL_WAVE) {
       float o[FC_BATCH];
 #pragma unroll
       for (int u = 0; u < FC_BATCH; ++u) o[u] = part_o[(row + (int64_t)min(u, n_splits - 1) * step) * hd + d];
@@ -1417,8 +1486,8 @@ __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __r
           acc += wgt * o[u];
         }
       }
-      const float Ls = with_sink(L, M, sink);
-      store_result(out, (int64_t)t * out_stride + (int64_t)h * hd + d, Ls > 0.f ? acc * out_scale / Ls : 0.f, sink);
+      const float Ls = with_sink(L, M, fin.flags, score);
+      store_result(out, (int64_t)t * out_stride + (int64_t)h * fin.vdim + d, Ls > 0.f ? acc * f / Ls : 0.f, fin.flags);
     }
     return;
   }
@@ -1429,7 +1498,7 @@ __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __r
     M = fmaxf(M, s < n_splits ? part_ml[(row + s * step) * 2] : kNegBig);
   }
   M = wave_max(M);
-  for (int d = lane; d < hd; d += TL_WAVE) {
+  for (int d = lane; d < fin.vdim; d += TL_WAVE) {
     float acc = 0.f, L = 0.f;
     for (int s0 = 0; s0 < n_splits; s0 += FC_BATCH) {
       float m[FC_BATCH], l[FC_BATCH], o[FC_BATCH];
@@ -1449,8 +1518,8 @@ __global__ __launch_bounds__(TL_WAVE) void flash_combine_kernel(const float* __r
         }
       }
     }
-    const float Ls = with_sink(L, M, sink);
-    store_result(out, (int64_t)t * out_stride + (int64_t)h * hd + d, Ls > 0.f ? acc * out_scale / Ls : 0.f, sink);
+    const float Ls = with_sink(L, M, fin.flags, score);
+    store_result(out, (int64_t)t * out_stride + (int64_t)h * fin.vdim + d, Ls > 0.f ? acc * f / Ls : 0.f, fin.flags);
   }
 }
 
@@ -1459,7 +1528,7 @@ static int launch_flash_w(const bf16_t* q, int64_t q_stride, const bf16_t* k_cac
                           const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                           const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, bf16_t* out,
                           int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq,
-                          int nkv, int block_size, float scale, KeyMask mask, int sink, int n_splits, const FusedRope& fused,
+                          int nkv, int block_size, float scale, KeyMask mask, const Finish& fin, int n_splits, const FusedRope& fused,
                           hipStream_t stream) {
   constexpr int HD = HDT * 16;
   constexpr size_t stage = (size_t)WAVES * FA_KT * (HD + FA_VPAD) * sizeof(bf16_t);
@@ -1474,7 +1543,7 @@ static int launch_flash_w(const bf16_t* q, int64_t q_stride, const bf16_t* k_cac
   }
   hipLaunchKernelGGL((flash_attn_bf16_kernel<HDT, WAVES, KIND>), dim3(n_tiles, nkv, n_splits), dim3(WAVES * TL_WAVE), stage,
                      stream, q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
-                     positions, out, out_stride, part_o, part_ml, nq, nkv, block_size, scale, mask, sink, n_splits,
+                     positions, out, out_stride, part_o, part_ml, nq, nkv, block_size, scale, mask, fin, n_splits,
                      n_tokens, fused);
   return TL_OK;
 }
@@ -1492,22 +1561,27 @@ static int launch_flash(const bf16_t* q, int64_t q_stride, const bf16_t* k_cache
                         const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                         const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, bf16_t* out,
                         int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq, int nkv,
-                        int block_size, float scale, KeyMask mask, int sink, int n_splits, const FusedRope& fused,
+                        int block_size, float scale, KeyMask mask, const Finish& fin, int n_splits, const FusedRope& fused,
                         hipStream_t stream) {
   if constexpr (HDT <= 4) {
     if (flash_waves(HDT * 16, n_tiles * nkv) == 8)
       return launch_flash_w<HDT, 8, KIND>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0,
                                     tile_ntok, positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv,
-                                    block_size, scale, mask, sink, n_splits, fused, stream);
+                                    block_size, scale, mask, fin, n_splits, fused, stream);
   }
   return launch_flash_w<HDT, 4, KIND>(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                                 positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, block_size,
-                                scale, mask, sink, n_splits, fused, stream);
+                                scale, mask, fin, n_splits, fused, stream);
 }
 
 static bool mask_ok(int keep, float softcap) { return keep >= 0 && softcap >= 0.f; }
-static MaskKind mask_kind(const KeyMask& m) {
-  return m.cap > 0.f ? kMaskCapped : m.keep > 0 || m.out_scale != 1.f ? kMaskKeeps : kMaskPlain;
+static bool finish_ok(const Finish& f, int nq, int hd) {
+  return f.vdim > 0 && f.vdim <= hd && (!f.sinks || (f.flags & kFlagSink)) && (!f.gate || f.gate_stride >= nq);
+}
+static MaskKind mask_kind(const KeyMask& m, const Finish& f, int hd) {
+  if (m.cap > 0.f) return kMaskCapped;
+  if (m.keep > 0) return kMaskKeeps;
+  return f.sinks || f.gate || f.vdim != hd || m.out_scale != 1.f ? kMaskFinished : kMaskPlain;
 }
 
 }  // namespace
@@ -1519,7 +1593,8 @@ extern "C" {
 int tl_paged_attention(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                        const int32_t* block_tables, int max_blocks, const int32_t* req_of_token,
                        const int32_t* positions, void* out, int64_t out_stride, int n_tokens, int nq,
-                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int dtype,
+                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink,
+                       const float* sinks, const float* gate, int64_t gate_stride, int vdim, int dtype,
                        hipStream_t stream) {
   if (n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || hd <= 0 || hd > kMaxHd || block_size <= 0 || max_blocks <= 0 ||
@@ -1527,15 +1602,17 @@ int tl_paged_attention(const void* q, int64_t q_stride, const void* k_cache, con
     return TL_ERR_ARG;
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
   const KeyMask mask{window, keep, softcap, out_scale};
+  const Finish fin{sink, sinks, gate, gate_stride, vdim > 0 ? vdim : hd};
+  if (!finish_ok(fin, nq, hd)) return TL_ERR_ARG;
   dim3 g(n_tokens, nq), b(TL_WAVE);
   if (dtype == 0)
     hipLaunchKernelGGL(paged_attention_kernel<float>, g, b, 0, stream, (const float*)q, q_stride,
                        (const float*)k_cache, (const float*)v_cache, block_tables, max_blocks, req_of_token,
-                       positions, (float*)out, out_stride, nq, nkv, hd, block_size, scale, mask, sink);
+                       positions, (float*)out, out_stride, nq, nkv, hd, block_size, scale, mask, fin);
   else if (dtype == 1)
     hipLaunchKernelGGL(paged_attention_kernel<bf16_t>, g, b, 0, stream, (const bf16_t*)q, q_stride,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_blocks, req_of_token,
-                       positions, (bf16_t*)out, out_stride, nq, nkv, hd, block_size, scale, mask, sink);
+                       positions, (bf16_t*)out, out_stride, nq, nkv, hd, block_size, scale, mask, fin);
   else
     return TL_ERR_ARG;
   return tl_launch_status();
@@ -1549,7 +1626,8 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
                      const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                      const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, float* out,
                      int64_t out_stride, float* part, int n_tiles, int n_tokens, int nq, int nkv, int hd,
-                     int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int n_chunks, hipStream_t stream) {
+                     int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink,
+                       const float* sinks, const float* gate, int64_t gate_stride, int vdim, int n_chunks, hipStream_t stream) {
   if (n_tiles <= 0 || n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || nq / nkv > 16 || hd <= 0 || hd % 16 || hd > 128 || block_size <= 0 ||
       max_blocks <= 0 || n_chunks < 1 || nkv > 65535 || n_chunks > 65535 || q_stride % 4 ||
@@ -1560,6 +1638,8 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
   if (tile_req && (!tile_tok0 || !tile_ntok)) return TL_ERR_ARG;
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
   const KeyMask mask{window, keep, softcap, out_scale};
+  const Finish fin{sink, sinks, gate, gate_stride, vdim > 0 ? vdim : hd};
+  if (!finish_ok(fin, nq, hd)) return TL_ERR_ARG;
   const size_t smem = (size_t)(A32_WAVES * FA_KT * A32_VS + A32_CHUNK * 16 * (hd + 4) + A32_CHUNK * 16 * 2) * sizeof(float);
   // Many query tiles (prompts): a wave a tile, four neighbouring tiles a workgroup; few (decode steps, small
   // steps): a workgroup a tile, its waves sharing the key tiles out.  The same bits either way.
@@ -1577,7 +1657,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
     hipLaunchKernelGGL(attention_f32_rows_kernel<HDT>, dim3((n_tiles + A32_WAVES - 1) / A32_WAVES, nkv),           \
                        dim3(A32_THREADS), smem_rows, stream, q, q_stride, k_cache, v_cache, block_tables,          \
                        max_blocks, tile_req, tile_tok0, tile_ntok, positions, out, out_stride, nq, nkv,            \
-                       block_size, scale, mask, sink, n_tiles);                                                        \
+                       block_size, scale, mask, fin, n_tiles);                                                        \
   } break;
     switch (hd / 16) {
       TL_A32_ROWS(1) TL_A32_ROWS(2) TL_A32_ROWS(3) TL_A32_ROWS(4)
@@ -1597,7 +1677,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
     }                                                                                                             \
     hipLaunchKernelGGL(attention_f32_kernel<HDT>, dim3(n_tiles, nkv, n_chunks), dim3(A32_THREADS), smem, stream,  \
                        q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,   \
-                       positions, out, out_stride, part, nq, nkv, block_size, scale, mask, sink, n_tokens);           \
+                       positions, out, out_stride, part, nq, nkv, block_size, scale, mask, fin, n_tokens);           \
   } break;
   switch (hd / 16) {
     TL_A32_CASE(1) TL_A32_CASE(2) TL_A32_CASE(3) TL_A32_CASE(4)
@@ -1606,7 +1686,7 @@ int tl_attention_f32(const float* q, int64_t q_stride, const float* k_cache, con
 #undef TL_A32_CASE
   if (n_chunks > 1)
     hipLaunchKernelGGL(attention_f32_combine_kernel, dim3(n_tokens, nq), dim3(TL_WAVE), 0, stream, part, out,
-                       out_stride, n_tokens, nq, hd, n_chunks, sink, out_scale);
+                       out_stride, n_tokens, nq, hd, n_chunks, fin, out_scale);
   return tl_launch_status();
 }
 
@@ -1617,7 +1697,8 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
                      const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                      const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
                      int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq, int nkv,
-                     int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int tile_waves, int n_splits,
+                     int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink,
+                       const float* sinks, const float* gate, int64_t gate_stride, int vdim, int tile_waves, int n_splits,
                      hipStream_t stream) {
   if (n_tiles <= 0) return TL_OK;
   if (tile_waves != 8 && tile_waves != 4) return TL_ERR_ARG;
@@ -1632,7 +1713,9 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
     return TL_ERR_ARG;
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
   const KeyMask mask{window, keep, softcap, out_scale};
-  const MaskKind kind = mask_kind(mask);
+  const Finish fin{sink, sinks, gate, gate_stride, vdim > 0 ? vdim : hd};
+  if (!finish_ok(fin, nq, hd)) return TL_ERR_ARG;
+  const MaskKind kind = mask_kind(mask, fin, hd);
   int bs_shift = -1;      // log2 of the page size where it is a power of two
   for (int sh = 0; sh < 31; ++sh)
     if ((1 << sh) == block_size) bs_shift = sh;
@@ -1641,13 +1724,15 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
                      stream, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,          \
                      block_tables, max_blocks, tile_req, tile_tok0, tile_ntok, positions, (bf16_t*)out,           \
                      out_stride, part_o, part_ml, n_tiles, n_tokens, n_splits, nq, nkv, block_size, bs_shift,     \
-                     scale, mask, sink)
+                     scale, mask, fin)
 #define TL_PREFILL_CASE(HDT)                        \
   case HDT:                                         \
     if (kind == kMaskCapped && tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, kMaskCapped);     \
     else if (kind == kMaskCapped) TL_PREFILL_LAUNCH(HDT, 4, kMaskCapped);                   \
     else if (kind == kMaskKeeps && tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, kMaskKeeps);  \
     else if (kind == kMaskKeeps) TL_PREFILL_LAUNCH(HDT, 4, kMaskKeeps);                     \
+    else if (kind == kMaskFinished && tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, kMaskFinished); \
+    else if (kind == kMaskFinished) TL_PREFILL_LAUNCH(HDT, 4, kMaskFinished);               \
     else if (tile_waves == 8) TL_PREFILL_LAUNCH(HDT, 8, kMaskPlain);                        \
     else TL_PREFILL_LAUNCH(HDT, 4, kMaskPlain);                                             \
     break;
@@ -1659,7 +1744,7 @@ int tl_flash_prefill(const void* q, int64_t q_stride, const void* k_cache, const
 #undef TL_PREFILL_LAUNCH
 #define TL_COMBINE(B)                                                                                          \
   hipLaunchKernelGGL(flash_combine_kernel<B>, dim3(n_tokens, nq), dim3(TL_WAVE), 0, stream, part_o, part_ml, \
-                     (bf16_t*)out, out_stride, n_tokens, nq, hd, n_splits, sink, out_scale)
+                     (bf16_t*)out, out_stride, n_tokens, nq, hd, n_splits, fin, out_scale)
   if (n_splits > 8) TL_COMBINE(16);
   else if (n_splits > 4) TL_COMBINE(8);
   else if (n_splits > 2) TL_COMBINE(4);
@@ -1679,7 +1764,8 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
                                const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                                const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
                                int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq,
-                               int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int n_splits,
+                               int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink,
+                       const float* sinks, const float* gate, int64_t gate_stride, int vdim, int n_splits,
                                const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
   if (n_tiles <= 0 || n_tokens <= 0) return TL_OK;
   if (nq <= 0 || nkv <= 0 || nq % nkv || nq / nkv > 16 || hd <= 0 || hd % 16 || hd > 128 || block_size <= 0 ||
@@ -1695,15 +1781,18 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
                   nq * hd, (nq + nkv) * hd};
   if (!mask_ok(keep, softcap)) return TL_ERR_ARG;
   const KeyMask mask{window, keep, softcap, out_scale};
-  const MaskKind kind = mask_kind(mask);
+  const Finish fin{sink, sinks, gate, gate_stride, vdim > 0 ? vdim : hd};
+  if (!finish_ok(fin, nq, hd)) return TL_ERR_ARG;
+  const MaskKind kind = mask_kind(mask, fin, hd);
   int rc = TL_ERR_ARG;
 #define TL_FLASH_CASE(HDT)                                                                                       \
   case HDT:                                                                                                      \
     rc = (kind == kMaskCapped  ? launch_flash<HDT, kMaskCapped>                                                   \
           : kind == kMaskKeeps ? launch_flash<HDT, kMaskKeeps>                                                   \
+          : kind == kMaskFinished ? launch_flash<HDT, kMaskFinished>                                             \
                                : launch_flash<HDT, kMaskPlain>)((const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,           \
                            block_tables, max_blocks, tile_req, tile_tok0, tile_ntok, positions, (bf16_t*)out,    \
-                           out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, block_size, scale, mask, sink,   \
+                           out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, block_size, scale, mask, fin,   \
                            n_splits, fused, stream);                                                             \
     break;
   switch (hd / 16) {
@@ -1714,7 +1803,7 @@ static int flash_attention_any(const void* q, int64_t q_stride, const void* k_ca
   if (rc != TL_OK) return rc;
 #define TL_COMBINE(B)                                                                                          \
   hipLaunchKernelGGL(flash_combine_kernel<B>, dim3(n_tokens, nq), dim3(TL_WAVE), 0, stream, part_o, part_ml, \
-                     (bf16_t*)out, out_stride, n_tokens, nq, hd, n_splits, sink, out_scale)
+                     (bf16_t*)out, out_stride, n_tokens, nq, hd, n_splits, fin, out_scale)
   if (n_splits > 8) TL_COMBINE(16);
   else if (n_splits > 4) TL_COMBINE(8);
   else if (n_splits > 2) TL_COMBINE(4);
@@ -1731,20 +1820,21 @@ int tl_flash_attention(const void* q, int64_t q_stride, const void* k_cache, con
                        const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
   return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                              positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
-                             scale, window, 0, 0.f, 1.f, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+                             scale, window, 0, 0.f, 1.f, sink, nullptr, nullptr, 0, 0, n_splits, rope_cos, rope_sin, fuse_store, stream);
 }
 
 // The same with the rest of the mask: the request's first `keep` tokens stay visible behind a window, and softcap > 0
-// caps the scores, cap * tanh(score / cap); the result is multiplied by out_scale.
+// caps the scores, cap * tanh(score / cap); the result is multiplied by out_scale and leaves as `Finish` says.
 int tl_flash_attention_masked(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                        const int32_t* block_tables, int max_blocks, const int32_t* tile_req,
                        const int32_t* tile_tok0, const int32_t* tile_ntok, const int32_t* positions, void* out,
                        int64_t out_stride, float* part_o, float* part_ml, int n_tiles, int n_tokens, int nq,
-                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink, int n_splits,
+                       int nkv, int hd, int block_size, float scale, int window, int keep, float softcap, float out_scale, int sink,
+                       const float* sinks, const float* gate, int64_t gate_stride, int vdim, int n_splits,
                        const float* rope_cos, const float* rope_sin, int fuse_store, hipStream_t stream) {
   return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                              positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
-                             scale, window, keep, softcap, out_scale, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+                             scale, window, keep, softcap, out_scale, sink, sinks, gate, gate_stride, vdim, n_splits, rope_cos, rope_sin, fuse_store, stream);
 }
 
 // ------------------------------------------------ the entry point that allocates nothing
@@ -1797,7 +1887,7 @@ int tl_flash_attention_static(const void* q, int64_t q_stride, const void* k_cac
   }
   return flash_attention_any(q, q_stride, k_cache, v_cache, block_tables, max_blocks, tile_req, tile_tok0, tile_ntok,
                              positions, out, out_stride, part_o, part_ml, n_tiles, n_tokens, nq, nkv, hd, block_size,
-                             scale, window, 0, 0.f, 1.f, sink, n_splits, rope_cos, rope_sin, fuse_store, stream);
+                             scale, window, 0, 0.f, 1.f, sink, nullptr, nullptr, 0, 0, n_splits, rope_cos, rope_sin, fuse_store, stream);
 }
 
 }  // extern "C"

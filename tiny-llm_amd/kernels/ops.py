@@ -609,6 +609,24 @@ def _attn_flags(sink: bool, q: torch.Tensor, out: torch.Tensor) -> int:
     return (1 if sink else 0) | (2 if (out.dtype == torch.float32 and q.dtype != torch.float32) else 0)
 
 
+def _attn_finish_args(sink: bool, sinks: Optional[torch.Tensor], gate: Optional[torch.Tensor], value_dim: int,
+                      q: torch.Tensor, out: torch.Tensor, num_heads: int, head_dim: int):
+    """How an attention kernel's result leaves it, checked: (flags, sinks, gate, its row stride, columns kept a head)."""
+    vdim = value_dim or head_dim
+    T = q.shape[0]
+    if not (0 < vdim <= head_dim and q.shape[1] == num_heads * head_dim and tuple(out.shape) == (T, num_heads * vdim)):
+        _fail("q must be [T, heads * head_dim] and the attention output [T, heads * value_dim], value_dim within head_dim")
+    if sinks is not None:
+        _dev(sinks)
+        _f32_vec(sinks, num_heads, "the sinks' scores")
+    if gate is not None:
+        _dev(gate)
+        _rows_2d(gate, "attention gate")
+        _need(gate.dtype == torch.float32 and tuple(gate.shape) == (T, num_heads), "the gate is float32 [T, heads]")
+    return (c_int(_attn_flags(sink or sinks is not None, q, out)), _ptr(sinks), _ptr(gate),
+            c_int64(gate.stride(0) if gate is not None else 0), c_int(vdim))
+
+
 def _attn_types_ok(q, k_cache, v_cache, out) -> bool:
     return q.dtype == k_cache.dtype == v_cache.dtype and out.dtype in (q.dtype, torch.float32)
 
@@ -617,18 +635,21 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     block_tables: torch.Tensor, req_of_token: torch.Tensor, positions: torch.Tensor,
                     out: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, scale: float,
                     window: int = 0, sink: bool = False, keep: int = 0, softcap: float = 0.0,
-                    out_scale: float = 1.0) -> torch.Tensor:
+                    out_scale: float = 1.0, sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+                    value_dim: int = 0) -> torch.Tensor:
     """Causal attention of every row of q (at its absolute position) over its
     request's cached keys 0..position (the last `window` of them if window > 0; the request's first `keep`
     stay visible behind the window).  softcap > 0: every score s becomes softcap * tanh(s / softcap).
     out_scale: a constant on the result.
-    sink: the softmax's denominator has one more term, exp(0), that carries no value."""
+    sink: the softmax's denominator has one more term, exp(0), that carries no value; `sinks` (float32 [heads]): the
+    term is exp(sinks[head]), whatever the scale and the cap of the scores.  gate (float32 [T, heads], rows may be wider
+    apart): the result times sigmoid(gate), one number per row and head.  value_dim: of every head's numbers the first
+    so many are values; the output is [T, heads * value_dim], the heads side by side (0: head_dim)."""
     _dev(q, k_cache, v_cache, block_tables, req_of_token, positions, out)
     _rows_2d(q, "q")
     _rows_2d(out, "attention output")
     T = q.shape[0]
-    if not (q.shape[1] == num_heads * head_dim and tuple(out.shape) == (T, num_heads * head_dim)):
-        _fail("q and the attention output must be [T, heads * head_dim]")
+    finish = _attn_finish_args(sink, sinks, gate, value_dim, q, out, num_heads, head_dim)
     if not _attn_types_ok(q, k_cache, v_cache, out):
         _fail("q and caches must share an element type; the output has it too or is float32")
     if not (k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dim() == 4
@@ -648,7 +669,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         _ptr(q), c_int64(q.stride(0)), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
         c_int(block_tables.shape[1]), _ptr(req_of_token), _ptr(positions), _ptr(out), c_int64(out.stride(0)),
         c_int(T), c_int(num_heads), c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]),
-        c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), c_int(_attn_flags(sink, q, out)), c_int(_dt(q)),
+        c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), *finish, c_int(_dt(q)),
         _stream()), "paged_attention")
     return out
 
@@ -666,7 +687,8 @@ def attention_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                   tiles, positions: torch.Tensor, out: torch.Tensor, num_heads: int, num_kv_heads: int,
                   head_dim: int, scale: float, window: int = 0, n_chunks: int = 1,
                   scratch: Optional[torch.Tensor] = None, sink: bool = False, keep: int = 0,
-                  softcap: float = 0.0, out_scale: float = 1.0) -> torch.Tensor:
+                  softcap: float = 0.0, out_scale: float = 1.0, sinks: Optional[torch.Tensor] = None,
+                  gate: Optional[torch.Tensor] = None, value_dim: int = 0) -> torch.Tensor:
     """The same function as `paged_attention` in true float32 on the matrix cores.  `tiles` as for
     `flash_attention` (None: row i is the one new token of request i).  n_chunks == 1: one
     workgroup per tile and kv head walks all keys; n_chunks > 1 (at least ceil(longest context /
@@ -681,8 +703,7 @@ def attention_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
     if not attention_f32_supported(q.dtype, num_heads, num_kv_heads, head_dim):
         _fail("the float32 matrix-core attention kernel takes float32, head sizes in steps of 16 up to 128, up "
               "to 16 heads per kv head")
-    if not (q.shape[1] == num_heads * head_dim and tuple(out.shape) == (T, num_heads * head_dim)):
-        _fail("q and the attention output must be [T, heads * head_dim]")
+    finish = _attn_finish_args(sink, sinks, gate, value_dim, q, out, num_heads, head_dim)
     if not (k_cache.dtype == v_cache.dtype == out.dtype == torch.float32):
         _fail("q, caches and output must be float32")
     if not (k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dim() == 4
@@ -713,7 +734,7 @@ def attention_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         _ptr(q, 16), c_int64(q.stride(0)), _ptr(k_cache, 16), _ptr(v_cache, 16), _ptr(block_tables),
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out), c_int64(out.stride(0)), _ptr(scratch), c_int(n_tiles), c_int(T), c_int(num_heads),
-        c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), c_int(1 if sink else 0),
+        c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), *finish,
         c_int(n_chunks), _stream()), "attention_f32")
     return out
 
@@ -729,7 +750,8 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     head_dim: int, scale: float, window: int = 0, n_splits: int = 1,
                     scratch: Optional[torch.Tensor] = None, fused_rope=None, static_scratch: bool = False,
                     sink: bool = False, keep: int = 0, softcap: float = 0.0,
-                    out_scale: float = 1.0) -> torch.Tensor:
+                    out_scale: float = 1.0, sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+                    value_dim: int = 0) -> torch.Tensor:
     """The same function as `paged_attention` on the matrix cores (bfloat16).  `tiles` =
     (tile_req, tile_tok0, tile_ntok): groups of at most 16 // (heads / kv_heads) consecutive
     tokens of one request; None for a decode step, where row i is the one new token of request i
@@ -750,8 +772,7 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     if not (flash_attention_supported(q.dtype, num_heads, num_kv_heads, head_dim)):
         _fail("the MFMA attention kernel takes bfloat16, head sizes in steps of 16 up to 128, up to 16 "
               "heads per kv head")
-    if not (q.shape[1] == num_heads * head_dim and tuple(out.shape) == (T, num_heads * head_dim)):
-        _fail("q and the attention output must be [T, heads * head_dim]")
+    finish = _attn_finish_args(sink, sinks, gate, value_dim, q, out, num_heads, head_dim)
     if not _attn_types_ok(q, k_cache, v_cache, out):
         _fail("q and caches must share an element type; the output has it too or is float32")
     if not (k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dim() == 4
@@ -796,8 +817,9 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         if not (q.stride(0) >= (num_heads + 2 * num_kv_heads) * head_dim):
             _fail("fused mode needs q inside its qkv rows")
     if static_scratch:
-        _need(keep == 0 and softcap == 0.0 and out_scale == 1.0, "flash_attention: the static entry point takes no kept tokens, "
-              "no soft cap and no constant on the result")
+        _need(keep == 0 and softcap == 0.0 and out_scale == 1.0 and sinks is None and gate is None and out.shape == q.shape,
+              "flash_attention: the static entry point takes no kept tokens, no soft cap, and a result that is only divided "
+              "by its denominator")
         code = _lib().tl_flash_attention_static(
             _ptr(q, 16), c_int64(q.stride(0)), _ptr(k_cache, 16), _ptr(v_cache, 16), _ptr(block_tables),
             c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
@@ -814,7 +836,7 @@ def flash_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out, 8), c_int64(out.stride(0)), _ptr(part_o), _ptr(part_ml), c_int(n_tiles), c_int(T),
         c_int(num_heads), c_int(num_kv_heads), c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale),
-        c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), c_int(_attn_flags(sink, q, out)), c_int(n_splits), _ptr(cos), _ptr(sin),
+        c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), *finish, c_int(n_splits), _ptr(cos), _ptr(sin),
         c_int(1 if fused_rope is not None else 0), _stream()), "flash_attention")
     return out
 
@@ -905,7 +927,8 @@ def flash_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                   tiles, positions: torch.Tensor, out: torch.Tensor, num_heads: int, num_kv_heads: int,
                   head_dim: int, scale: float, window: int = 0, tile_waves: int = 8, n_splits: int = 1,
                   scratch: Optional[torch.Tensor] = None, sink: bool = False, keep: int = 0,
-                  softcap: float = 0.0, out_scale: float = 1.0) -> torch.Tensor:
+                  softcap: float = 0.0, out_scale: float = 1.0, sinks: Optional[torch.Tensor] = None,
+                  gate: Optional[torch.Tensor] = None, value_dim: int = 0) -> torch.Tensor:
     """`flash_attention` arranged for prompt portions: `tiles` are groups of at most
     tile_waves * (16 // (heads / kv_heads)) consecutive tokens of one request, and a key or value
     row is staged once per such group.  tile_waves is PREFILL_TILES (8), or 4 for steps with few
@@ -921,8 +944,7 @@ def flash_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
     if not (flash_attention_supported(q.dtype, num_heads, num_kv_heads, head_dim)):
         _fail("the MFMA attention kernel takes bfloat16, head sizes in steps of 16 up to 128, up to 16 "
               "heads per kv head")
-    if not (q.shape[1] == num_heads * head_dim and tuple(out.shape) == (T, num_heads * head_dim)):
-        _fail("q and the attention output must be [T, heads * head_dim]")
+    finish = _attn_finish_args(sink, sinks, gate, value_dim, q, out, num_heads, head_dim)
     if not _attn_types_ok(q, k_cache, v_cache, out):
         _fail("q and caches must share an element type; the output has it too or is float32")
     if not (k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dim() == 4
@@ -955,7 +977,7 @@ def flash_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         c_int(block_tables.shape[1]), _ptr(tile_req), _ptr(tile_tok0), _ptr(tile_ntok), _ptr(positions),
         _ptr(out, 16 if out.dtype == torch.float32 else 8), c_int64(out.stride(0)), _ptr(part_o, 16), _ptr(part_ml), c_int(n_tiles), c_int(T),
         c_int(num_heads), c_int(num_kv_heads),
-        c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), c_int(_attn_flags(sink, q, out)), c_int(tile_waves),
+        c_int(head_dim), c_int(k_cache.shape[2]), c_float(scale), c_int(window), c_int(keep), c_float(softcap), c_float(out_scale), *finish, c_int(tile_waves),
         c_int(n_splits),
         _stream()), "flash_prefill")
     return out
@@ -1661,21 +1683,30 @@ def layer_norm_sum(y: Optional[torch.Tensor], weight: torch.Tensor, bias: torch.
     return x
 
 
-LAYER_NORM_ADD_MAX = 8192       # widest row `layer_norm_add` keeps in registers (csrc/layer_norm.hip)
+LAYER_NORM_ADD_MAX = 8192       # widest row `layer_norm_add` and `rms_norm_add` keep in registers (csrc/layer_norm.hip)
+
+
+def _norm_add_rows(what: str, y, x, shift):
+    """(T, H) of a norm that is added to the stream, checked."""
+    _dev(y, x, shift)
+    if not (x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous()):
+        _fail(f"{what}: the stream is contiguous float32 [T, H]")
+    T, H = x.shape
+    _need(H <= LAYER_NORM_ADD_MAX, f"{what}: rows of at most {LAYER_NORM_ADD_MAX} elements")
+    if not (y.dtype == torch.float32 and y.is_contiguous() and tuple(y.shape) == (T, H)):
+        _fail(f"{what}: the sublayer's result is contiguous float32 [T, H]")
+    if shift is not None:
+        _f32_vec(shift, H, f"{what}: the vector added to every row")
+    return T, H
 
 
 def layer_norm_add(y: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, x: torch.Tensor, mult: float, eps: float,
-                   then=None) -> torch.Tensor:
-    """x[t] <- x[t] + mult * (LN(y[t]) * weight + bias), in place, float32 (y the sublayer's result, float32 [T, H]).
-    then = (weight2, bias2, eps2, out): out[t] ([T, H] of either element type) also receives LN(x[t]) * weight2 +
-    bias2 of the new rows, in the same kernel."""
-    _dev(y, weight, bias, x)
-    if not (x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous()):
-        _fail("layer_norm_add: the stream is contiguous float32 [T, H]")
-    T, H = x.shape
-    _need(H <= LAYER_NORM_ADD_MAX, f"layer_norm_add: rows of at most {LAYER_NORM_ADD_MAX} elements")
-    if not (y.dtype == torch.float32 and y.is_contiguous() and tuple(y.shape) == (T, H)):
-        _fail("layer_norm_add: the sublayer's result is contiguous float32 [T, H]")
+                   then=None, shift: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x[t] <- x[t] + mult * (LN(y[t]) * weight + bias) + shift, in place, float32 (y the sublayer's result, float32
+    [T, H]; shift a vector, or None).  then = (weight2, bias2, eps2, out): out[t] ([T, H] of either element type) also
+    receives LN(x[t]) * weight2 + bias2 of the new rows, in the same kernel."""
+    T, H = _norm_add_rows("layer_norm_add", y, x, shift)
+    _dev(weight, bias)
     _f32_vec(weight, H, "the layer norm's weight")
     _f32_vec(bias, H, "the layer norm's bias")
     w2 = b2 = out = None
@@ -1687,9 +1718,40 @@ def layer_norm_add(y: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, x:
         _f32_vec(b2, H, "the next norm's bias")
         if not (out.is_contiguous() and tuple(out.shape) == (T, H)):
             _fail("layer_norm_add: the next norm's output is contiguous [T, H]")
-    _check(_lib().tl_layer_norm_add(_ptr(y), _ptr(weight), _ptr(bias), _ptr(x), _ptr(w2), _ptr(b2), _ptr(out), c_int(T),
-                                    c_int(H), c_float(mult), c_float(eps), c_float(eps2),
+    _check(_lib().tl_layer_norm_add(_ptr(y), _ptr(weight), _ptr(bias), _ptr(x), _ptr(w2), _ptr(b2), _ptr(shift), _ptr(out),
+                                    c_int(T), c_int(H), c_float(mult), c_float(eps), c_float(eps2),
                                     c_int(_dt(out) if out is not None else 0), _stream()), "layer_norm_add")
+    return x
+
+
+def rms_norm_add(y: torch.Tensor, weight: torch.Tensor, x: torch.Tensor, mult: float, eps: float, then=None,
+                 shift: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """`layer_norm_add` with RMS norms: x[t] <- x[t] + mult * y[t] / sqrt(mean(y[t]^2) + eps) * weight + shift;
+    then = (weight2, eps2, out): out[t] also receives the RMS norm of the new rows."""
+    T, H = _norm_add_rows("rms_norm_add", y, x, shift)
+    _dev(weight)
+    _f32_vec(weight, H, "the RMS norm's weight")
+    w2 = out = None
+    eps2 = 0.0
+    if then is not None:
+        w2, eps2, out = then
+        _dev(w2, out)
+        _f32_vec(w2, H, "the next norm's weight")
+        if not (out.is_contiguous() and tuple(out.shape) == (T, H)):
+            _fail("rms_norm_add: the next norm's output is contiguous [T, H]")
+    _check(_lib().tl_rms_norm_add(_ptr(y), _ptr(weight), _ptr(x), _ptr(w2), _ptr(shift), _ptr(out), c_int(T), c_int(H),
+                                  c_float(mult), c_float(eps), c_float(eps2), c_int(_dt(out) if out is not None else 0),
+                                  _stream()), "rms_norm_add")
+    return x
+
+
+def add_row_vector(x: torch.Tensor, vec: torch.Tensor) -> torch.Tensor:
+    """x[t] += vec for every row of the stream (float32 [T, H], in place)."""
+    _dev(x, vec)
+    if not (x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous()):
+        _fail("add_row_vector: the stream is contiguous float32 [T, H]")
+    _f32_vec(vec, x.shape[1], "add_row_vector: the vector")
+    _check(_lib().tl_add_row_vector(_ptr(x), _ptr(vec), c_int(x.shape[0]), c_int(x.shape[1]), _stream()), "add_row_vector")
     return x
 
 

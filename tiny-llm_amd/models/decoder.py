@@ -15,6 +15,7 @@ import torch
 from ..config.spec import LayerSpec, ModelSpec, PartSpec
 from ..kernels import ops
 from ..parts import BLOCKS, REGISTRIES, CacheSpec, LayerCache, Part, StateSpec, WeightSpec
+from ..parts.block import NormedRows, NormedRowsWanted
 
 TORCH_DTYPES = {"float32": torch.float32, "bfloat16": torch.bfloat16}
 
@@ -194,7 +195,7 @@ class Decoder:
         # them: in a buffer by name, so that a later call for the same step finds it.  The stream then goes on in a
         # buffer of its own (by a copy here if layers run ahead of the first such part, else that part moves it).
         origin = None
-        if self.stream_parts:
+        if any(p.reads_origin for p in self.stream_parts):
             if first == 0:
                 origin = x
                 if plan[0].before is None:
@@ -204,32 +205,45 @@ class Decoder:
         # A block may prepare the norm that reads its result (the next block's first norm, or the
         # final norm) in its last product; `prepared` carries that from one block to the next.
         prepared = None
+        all_rows = getattr(ctx, "logits_all_rows", False)
+        shifted = False             # the block in front has done what the stream part ahead of this one does
         for st in range(max(first, 1), min(last, n - 1)):
             i = st - 1
             block = self.layers[plan[i].layer].block
-            if plan[i].before is not None:
+            if plan[i].before is not None and not shifted:
                 part, turn = plan[i].before
                 x, prepared = self.stream_parts[part].forward(x, origin, ctx, turn), None
+            shifted = False
             if not hasattr(block, "forward_chained"):
                 x, prepared = block.forward(x, ctx, self.caches[i], self.states[i]), None
                 continue
-            next_norm = None
+            next_norm, extra = None, {}
             if st + 1 < last:                    # what reads this block's result runs in this call
-                if i + 1 < len(plan) and plan[i + 1].before is not None:
-                    next_norm = None             # a stream part stands between: it reads the stream itself
-                elif i + 1 < len(plan):
+                before = plan[i + 1].before if i + 1 < len(plan) else None
+                if before is not None:
+                    # a stream part stands between: it reads the stream itself, unless it only adds a vector to it and
+                    # this block's last kernel can do that
+                    vector = getattr(self.stream_parts[before[0]], "row_vector", None)
+                    if vector is not None and getattr(block, "takes_shift", False):
+                        extra, shifted = {"shift": vector(before[1])}, True
+                if i + 1 < len(plan):
                     nxt = self.layers[plan[i + 1].layer].block
-                    next_norm = getattr(nxt, "first_norm", None) if hasattr(nxt, "forward_chained") else None
+                    if before is None or shifted:
+                        next_norm = getattr(nxt, "first_norm", None) if hasattr(nxt, "forward_chained") else None
+                elif getattr(block, "hands_normed_rows", False):
+                    next_norm = NormedRowsWanted(self.final_norm) if wants_logits and all_rows else None
                 else:
                     next_norm = self.final_norm if wants_logits and lazy_head else None
-            x, prepared = block.forward_chained(x, ctx, self.caches[i], self.states[i], prepared, next_norm)
+            x, prepared = block.forward_chained(x, ctx, self.caches[i], self.states[i], prepared, next_norm, **extra)
         if last < n:
             return x
         if not wants_logits:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=x.device)
         norm = self.final_norm
-        rows = None if getattr(ctx, "logits_all_rows", False) else ctx.logit_rows
-        if lazy_head:
+        rows = None if all_rows else ctx.logit_rows
+        if isinstance(prepared, NormedRows):      # of every row, and every row is wanted
+            h = prepared.rows
+        elif lazy_head:
             h = norm.lazy(x, rows, prepared=prepared) if prepared is not None else norm.lazy(x, rows)
         else:
             h = norm.forward(x, rows)

@@ -96,13 +96,18 @@ class Attention(Mixer):
         out, prepared = project_into_residual(attn, self.w_o, residual, next_norm)
         return out if next_norm is None else (out, prepared)
 
-    def _attend(self, q, ctx, cache: LayerCache, attn, fused_rope=None, sink: bool = False, out_scale: float = 1.0):
+    def _attend(self, q, ctx, cache: LayerCache, attn, fused_rope=None, sink: bool = False, out_scale: float = 1.0,
+                sinks=None, gate=None, value_dim: int = 0):
         """attn <- attention of the step's query rows q [T, heads * head_dim] over the cache, by the kernel that
-        takes this step's shape.  sink: one more term exp(0) in every softmax's denominator.  `self.window`: 0
+        takes this step's shape.  sink: one more term exp(0) in every softmax's denominator (`sinks`, float32 [heads]:
+        exp(sinks[head])).  `self.window`: 0
         (every earlier key), n > 0 (the last n positions) or -n (the row's own run of n positions, runs counted
         from position 0: a chunked mask); the request's first `self.keep` positions are seen in any case.
-        `self.softcap` > 0: scores s become softcap * tanh(s / softcap).  out_scale: a constant on the result."""
-        mask = {"sink": sink, "keep": self.keep if self.window else 0, "softcap": self.softcap, "out_scale": out_scale}
+        `self.softcap` > 0: scores s become softcap * tanh(s / softcap).  out_scale: a constant on the result; gate: the
+        result times sigmoid(gate) (float32 [T, heads]); value_dim: attn is [T, heads * value_dim], the first so many
+        numbers of every head."""
+        mask = {"sink": sink, "keep": self.keep if self.window else 0, "softcap": self.softcap, "out_scale": out_scale,
+                "sinks": sinks, "gate": gate, "value_dim": value_dim}
         T, device = q.shape[0], q.device
         group = self.num_heads // self.num_kv_heads
         flash = ops.flash_attention_supported(self.dtype, self.num_heads, self.num_kv_heads, self.head_dim)
@@ -276,6 +281,8 @@ class GatedAttention(Attention):
         keys seen: all earlier ones, the last `window` (and the request's first `keep_first`), or those of the row's own
         run of `chunk` positions
         scores s become softcap * tanh(s / softcap)                                    `softcap`
+        the softmax's denominator has one more term, exp(sink_h) with a learned sink_h per head, neither scaled nor capped,
+        without a value                                                                `learned_sink`
         `maps=2`: two score maps per head (q and k hold [map 1 | map 2] head by head) over the same values,
                   o = a1 - lambda a2, lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff (a scalar of the layer)
         o divided by its root mean square over the head, no weight (`sub_norm`), times `out_scale`
@@ -286,7 +293,8 @@ class GatedAttention(Attention):
     own sizes (a zero adds nothing to a score, and the values' columns come first in the result), and the two maps
     are two passes of the kernel over caches of their own keys and the one cache of values.  One product reads h for
     [q | k | v | gates] and leaves float32; everything up to the rounded queries and cached keys is float32
-    arithmetic in one kernel, everything behind the attention kernel in another.  An output bias is a column of
+    arithmetic in one kernel, everything behind the attention kernel in another (one map without a norm behind it, with
+    or without a gate per head: the attention kernel leaves the output product's operand itself).  An output bias is a column of
     the output product's weight that meets a column of ones.  Returns the result by itself in float32 when
     `residual` is None."""
     graph_safe = True
@@ -297,7 +305,7 @@ class GatedAttention(Attention):
                  value_dim: int = None, position: dict = None, window: int = 0, chunk: int = 0, scale: float = None,
                  bias: bool = False, out_bias: bool = None, qk_norm: str = None, eps: float = 1e-6, q_temp=None,
                  maps: int = 1, diff: float = 0.0, sub_norm: bool = False, out_scale: float = 1.0, gate: str = None,
-                 conv_taps: int = 0, keep_first: int = 0, softcap: float = 0.0,
+                 conv_taps: int = 0, keep_first: int = 0, softcap: float = 0.0, learned_sink: bool = False,
                  names: Dict[str, str] = None, bias_suffix: str = ".b", norm_suffix: str = ".norm",
                  conv_suffix: str = ".conv", max_position: int = 0):
         dim, vdim = int(head_dim), int(value_dim if value_dim is not None else head_dim)
@@ -343,7 +351,8 @@ class GatedAttention(Attention):
         if self.q_temp and self.q_temp[1] <= 0:
             raise ValueError(f"{prefix}: the query temperature's step must be positive")
         self.sub_norm, self.out_scale, self.gate = bool(sub_norm), float(out_scale), gate
-        n = {k: k for k in ("q", "k", "v", "g", "o", "lq1", "lk1", "lq2", "lk2")}
+        self.learned_sink = bool(learned_sink)
+        n = {k: k for k in ("q", "k", "v", "g", "o", "lq1", "lk1", "lq2", "lk2", "sink")}
         n.update(names or {})
         self.names = {k: f"{prefix}.{v}" for k, v in n.items()}
         self.bias_suffix, self.norm_suffix, self.conv_suffix = bias_suffix, norm_suffix, conv_suffix
@@ -357,7 +366,7 @@ class GatedAttention(Attention):
         self.out_cols = H * vdim
         self.out_tail = 8 if self.out_bias else 0       # a column of ones for the bias, zeros up to a multiple of 8
         ops.check_linear_sizes(dtype, self.out_cols, f"{prefix}: num_heads * value_dim")
-        self.w_in = self.b_in = self.norm_w = self.head_w = self.conv_w = self.w_o = None
+        self.w_in = self.b_in = self.norm_w = self.head_w = self.conv_w = self.w_o = self.sink_w = None
         self.lam = 0.0
 
     def weights(self) -> List[WeightSpec]:
@@ -377,6 +386,8 @@ class GatedAttention(Attention):
                     for k, cols in (("q", self.q_cols), ("k", self.k_cols), ("v", self.v_cols))]
         if self.maps == 2:
             out += [WeightSpec(n[k], (self.qk_dim,), role="vector", init="normal") for k in ("lq1", "lk1", "lq2", "lk2")]
+        if self.learned_sink:
+            out.append(WeightSpec(n["sink"], (self.num_heads,), **vec))
         if self.gate:
             out.append(WeightSpec(n["g"], (self.g_cols, W)))
         out.append(WeightSpec(n["o"], (W, self.out_cols)))
@@ -405,6 +416,8 @@ class GatedAttention(Attention):
             self.conv_w = torch.cat([f32(tensors[n[k] + self.conv_suffix]) for k in ("q", "k", "v")]).contiguous()
         elif self.convolved:        # one tap of one: the value itself
             self.conv_w = torch.ones((self.v_off + self.v_cols, 1), dtype=torch.float32, device=dev)
+        if self.learned_sink:
+            self.sink_w = f32(tensors[n["sink"]]).contiguous()
         w_o = tensors[n["o"]]
         if self.out_bias:
             wide = torch.zeros((self.hidden_size, self.out_cols + self.out_tail), dtype=self.dtype, device=dev)
@@ -474,16 +487,17 @@ class GatedAttention(Attention):
                              cache.tensors["v"] if write else None, H, self.num_kv_heads, self.maps, self.qk_dim,
                              self.value_dim, self.v_off, rot, pairing, self.qk_norm == "whole", self.qk_norm == "unit",
                              self.eps, self.q_temp)
-        if self.maps == 1 and self.value_dim == self.head_dim and not (self.sub_norm or self.gate or self.out_tail):
-            # nothing lies behind the weighted sum but a constant: the attention kernel leaves the operand itself
-            return self._attend(q[0], ctx, cache, z, out_scale=self.out_scale)
+        gate = p[:, self.g_off:self.g_off + self.g_cols] if self.gate else None
+        if self.maps == 1 and self.gate in (None, "head") and not (self.sub_norm or self.out_tail):
+            # nothing lies behind the weighted sum but a factor per row and head: the attention kernel leaves the operand
+            return self._attend(q[0], ctx, cache, z, out_scale=self.out_scale, sinks=self.sink_w, gate=gate,
+                                value_dim=self.value_dim)
         outs = []
         for m in range(self.maps):
             # float32 whatever the engine's type: the maps' difference, the head's norm and the gates follow in float32
             attn = ops.scratch("attention_out" if m == 0 else "attention_out2", (T, self.q_size), torch.float32, dev)
             view = LayerCache({"k": k_caches[m], "v": cache.tensors["v"]}, cache.group, cache.write)
-            outs.append(self._attend(q[m], ctx, view, attn))
-        gate = p[:, self.g_off:self.g_off + self.g_cols] if self.gate else None
+            outs.append(self._attend(q[m], ctx, view, attn, sinks=self.sink_w))
         return ops.attn_finish(outs[0], outs[1] if self.maps == 2 else None, gate, z, H, self.value_dim, self.lam, self.sub_norm,
                                self.eps, self.out_scale, self.gate, self.out_tail)
 

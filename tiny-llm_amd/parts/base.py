@@ -177,7 +177,10 @@ class FeedForward(Part):
 class StreamPart(Part):
     """A part that acts on the residual stream between two layer runs: `forward(x, origin, ctx, turn)` returns the
     new stream (float32 [T, hidden]; it may write into x but not into origin).  `origin` is the embedding's output
-    of this step, `turn` the number the plan gives (which pass through a repeated run of layers begins)."""
+    of this step, `turn` the number the plan gives (which pass through a repeated run of layers begins).  A part that does
+    nothing but add one vector to every row may say which (`row_vector(turn)`): the block in front may then add it in its
+    last kernel, and `forward` is not called."""
+    reads_origin = True         # False: `origin` may be None, and x may be the embedding's output itself
 
     def forward(self, x: torch.Tensor, origin: torch.Tensor, ctx, turn: int) -> torch.Tensor:
         raise NotImplementedError

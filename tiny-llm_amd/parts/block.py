@@ -175,20 +175,31 @@ class SumNormBlock(Block):
         return x, copy
 
 
+class NormedRowsWanted:
+    """What a reader of the stream that takes its norm's rows ready-made shows to the block in front of it: the norm
+    it begins with.  (Another kind of block in front takes no notice of it.)"""
+
+    def __init__(self, norm):
+        self.norm = norm
+
+
 class NormedRows:
-    """What a sandwich block hands to the block behind it: the stream as that block's first norm sees it,
-    formed by the kernel that wrote the stream."""
+    """What a sandwich block hands to such a reader: the stream as that reader's norm sees it, formed by the kernel that
+    wrote the stream."""
 
     def __init__(self, norm, rows: torch.Tensor):
         self.norm, self.rows = norm, rows
 
 
 class SandwichBlock(Block):
-    """x <- x + mult * LNb(mixer(LNa(x))); x <- x + mult * LNd(ffn(LNc(x))): a norm in front of and behind every
-    sublayer.  The sublayers are called with `residual=None` and return their result by itself in float32; the norm
-    behind a sublayer, the scaled sum and the norm in front of whatever reads the stream next (this block's
-    feed-forward, or the next block's mixer if that block says which norm it begins with) are ONE kernel.  A layer
+    """x <- x + mult * Nb(mixer(Na(x))); x <- x + mult * Nd(ffn(Nc(x))): a norm in front of and behind every
+    sublayer (layer norms or RMS norms).  The sublayers are called with `residual=None` and return their result by itself
+    in float32; the norm behind a sublayer, the scaled sum and the norm in front of whatever reads the stream next (this
+    block's feed-forward, the next block's mixer or the output head, if the reader says which norm it begins with) are ONE
+    kernel, which also adds a vector to every row of the stream where the model wants one there (`takes_shift`).  A layer
     may have no feed-forward (and then neither of its norms)."""
+    takes_shift = True          # `forward_chained` takes `shift=`: a vector that every row of the result gains
+    hands_normed_rows = True    # and may hand NormedRows to whoever asks with NormedRowsWanted
     roles = {"mixer_norm": "norm", "mixer": "mixer", "mixer_out_norm": "norm",
              "ffn_norm": "norm", "ffn": "feed_forward", "ffn_out_norm": "norm"}
     optional = ("ffn_norm", "ffn", "ffn_out_norm")
@@ -204,10 +215,7 @@ class SandwichBlock(Block):
             if n is not None and not hasattr(n, "add_scaled_norm"):
                 raise ValueError(f"sandwich: the norm {type(n).__name__} cannot sit on a sublayer's result (no add_scaled_norm)")
 
-    @property
-    def first_norm(self):
-        """The norm that reads this block's input, for whoever writes that input."""
-        return self.mixer_norm
+        self.first_norm = NormedRowsWanted(self.mixer_norm)
 
     def forward(self, x, ctx, caches, states):
         return self.forward_chained(x, ctx, caches, states)[0]
@@ -217,26 +225,28 @@ class SandwichBlock(Block):
         """Whether `out_norm.add_scaled_norm` can also produce `next_norm` of the new stream."""
         return type(next_norm) is type(out_norm) and getattr(next_norm, "hidden_size", None) == out_norm.hidden_size
 
-    def forward_chained(self, x, ctx, caches, states, prepared=None, next_norm=None):
+    def forward_chained(self, x, ctx, caches, states, prepared=None, next_norm=None, shift=None):
         """`prepared`: NormedRows of this block's first norm if the block in front formed them; returned likewise
-        for the block behind when `next_norm` is a norm this block's last kernel can form."""
+        for the reader behind when `next_norm` is its NormedRowsWanted and this block's last kernel can form that norm.
+        `shift`: a vector that every row of the result gains (ahead of that norm)."""
+        next_norm = next_norm.norm if isinstance(next_norm, NormedRowsWanted) else None
         if isinstance(prepared, NormedRows) and prepared.norm is self.mixer_norm:
             h = prepared.rows
         else:
             h = self.mixer_norm.forward(x)
         y = self.mixer.forward(h, ctx, caches.get("mixer"), states.get("mixer"), None)
         if self.ffn is None:
-            return x, self._add(self.mixer_out_norm, y, x, next_norm)
+            return x, self._add(self.mixer_out_norm, y, x, next_norm, shift)
         handed = self._add(self.mixer_out_norm, y, x, self.ffn_norm)
         h = handed.rows if handed is not None else self.ffn_norm.forward(x)
         y = self.ffn.forward(h, ctx, None)
-        return x, self._add(self.ffn_out_norm, y, x, next_norm)
+        return x, self._add(self.ffn_out_norm, y, x, next_norm, shift)
 
-    def _add(self, out_norm, y, x, next_norm):
+    def _add(self, out_norm, y, x, next_norm, shift=None):
         if next_norm is not None and self._fusable(out_norm, next_norm):
-            rows = out_norm.add_scaled_norm(y, x, self.mult, then=next_norm)
+            rows = out_norm.add_scaled_norm(y, x, self.mult, then=next_norm, shift=shift)
             return NormedRows(next_norm, rows) if rows is not None else None
-        out_norm.add_scaled_norm(y, x, self.mult)
+        out_norm.add_scaled_norm(y, x, self.mult, shift=shift)
         return None
 
 

@@ -85,12 +85,29 @@ class RMSNorm(Norm):
                    copy: Optional[torch.Tensor] = None) -> torch.Tensor:
         """x += scale * norm(y) for a norm that sits on a sublayer's output (y float32, one kernel);
         `copy` receives the new x in its own element type."""
+        return ops.norm_scale_add(y, self.weight_f32, self.eps, x, scale, copy)
+
+    @property
+    def weight_f32(self) -> torch.Tensor:
+        """The weight in float32 (converted once, not at every step)."""
         w = self.weight
-        if w.dtype != torch.float32:        # converted once, not at every step
-            if self._weight_f32 is None or self._weight_f32.device != w.device:
-                self._weight_f32 = w.to(torch.float32)
-            w = self._weight_f32
-        return ops.norm_scale_add(y, w, self.eps, x, scale, copy)
+        if w.dtype == torch.float32:
+            return w
+        if self._weight_f32 is None or self._weight_f32.device != w.device:
+            self._weight_f32 = w.to(torch.float32)
+        return self._weight_f32
+
+    def add_scaled_norm(self, y: torch.Tensor, x: torch.Tensor, mult: float = 1.0, then: "RMSNorm" = None,
+                        shift: Optional[torch.Tensor] = None):
+        """As `LayerNorm.add_scaled_norm`: x <- x + mult * norm(y) (+ shift) in place, and `then` of the new x."""
+        if self.hidden_size > ops.LAYER_NORM_ADD_MAX:
+            raise ValueError(f"{self.tensor_name}: a norm behind a sublayer takes rows of at most {ops.LAYER_NORM_ADD_MAX}")
+        if then is None:
+            ops.rms_norm_add(y, self.weight_f32, x, mult, self.eps, shift=shift)
+            return None
+        out = ops.scratch("normed", x.shape, then.dtype, x.device, rotate=2)
+        ops.rms_norm_add(y, self.weight_f32, x, mult, self.eps, then=(then.weight_f32, then.eps, out), shift=shift)
+        return out
 
     def lazy(self, x: torch.Tensor, rows: Optional[torch.Tensor] = None, prepared=None):
         """The norm rides in the consumer's first product: in bfloat16 always (`ops.linear_norm`), in
@@ -156,17 +173,19 @@ class LayerNorm(Norm):
         its own element type."""
         return ops.layer_norm_sum(y, self.weight, self.bias, x, alpha, self.eps, copy)
 
-    def add_scaled_norm(self, y: torch.Tensor, x: torch.Tensor, mult: float = 1.0, then: "LayerNorm" = None):
+    def add_scaled_norm(self, y: torch.Tensor, x: torch.Tensor, mult: float = 1.0, then: "LayerNorm" = None,
+                        shift: Optional[torch.Tensor] = None):
         """x <- x + mult * LN(y) in place, for a norm that sits on a sublayer's result (y float32, one kernel).
-        `then`: the layer norm that reads the new x next; its result comes out of the same kernel and is returned
-        (None without one, or where the kernel does not take the width)."""
+        `shift`: a vector every row of the new x gains.  `then`: the layer norm that reads the new x next; its result
+        comes out of the same kernel and is returned (None without one)."""
         if self.hidden_size > ops.LAYER_NORM_ADD_MAX:
             raise ValueError(f"{self.prefix}: a layer norm behind a sublayer takes rows of at most {ops.LAYER_NORM_ADD_MAX}")
         if then is None:
-            ops.layer_norm_add(y, self.weight, self.bias, x, mult, self.eps)
+            ops.layer_norm_add(y, self.weight, self.bias, x, mult, self.eps, shift=shift)
             return None
         out = ops.scratch("normed", x.shape, then.dtype, x.device, rotate=2)
-        ops.layer_norm_add(y, self.weight, self.bias, x, mult, self.eps, then=(then.weight, then.bias, then.eps, out))
+        ops.layer_norm_add(y, self.weight, self.bias, x, mult, self.eps, then=(then.weight, then.bias, then.eps, out),
+                           shift=shift)
         return out
 
     def forward(self, x: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
