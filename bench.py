@@ -13,7 +13,8 @@ Llama-3-8B shape; 64 requests of 1,024 tokens that nearly fill the cache at the 
 `--only` picks a part (for profiling), or one of the measurements that are not part of the line:
 `attention` (the attention kernels alone at contexts up to 131,072 tokens), `long_context` (the Llama-3-8B
 shape with 8 requests of 32,000 tokens and one of 131,000), `decode_shapes` (decode steps at the two larger
-shapes by batch), `host` (a step's wall time against its time on the GPU), `mogutar`, `vevapel`, `gesutar` and `fofapel` (those designs, as `lufazen`), `lufazen` (the Lufazen design,
+shapes by batch), `host` (a step's wall time against its time on the GPU), `nililix`, `mogutar`, `vevapel`, `gesutar`
+and `fofapel` (those designs, as `lufazen`), `lufazen` (the Lufazen design,
 recurrent and latent-attention layers, at two sizes beside a Llama of equal size: prefill, decode, time by kernel).
 """
 import argparse
@@ -956,6 +957,51 @@ def mogutar_figures(args):
     return design_beside_llama(args, "mogutar", mogutar_config, bounds, beside=(("fofapel", fofapel_config),))
 
 
+def nililix_config(layers, width, ff, heads, vocab=32000, window=512):
+    """`layers` layer RUNS: layers - 2 layers, of which the second and third run twice (a loop over two layers).  Attention
+    in a window of 512 tokens (heads of 128, four query heads a kv head, 4 taps on q, k and v, a sink and a gate per head,
+    half of a head rotated with Llama 3.1's frequency scaling); feed-forwards in the order dense (ff), experts (16 of ff / 8
+    in four groups of which two are kept, four a token: half of a dense layer's hidden units a token)."""
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "router": {"experts": 16, "top": 4, "groups": {"count": 4, "keep": 2}}, "expert": {"ff": ff // 8}}
+    mixer = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "conv": 4, "mask": {"size": window},
+             "scale": 128 ** -0.5,
+             "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 2048}}}
+    out = [{"type": "attention", "mixer": mixer, "mlp": moe if i % 2 else dense} for i in range(max(3, layers - 2))]
+    return {"architecture": "Nililix", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "residual_mult": 0.5,
+            "logit_softcap": 30.0, "layers": out, "loop": {"start": 1, "stop": 3, "times": 2}, "max_position": 8192}
+
+
+def nililix_figures(args):
+    """The Nililix design at two sizes beside the closest designs of the tree, Mogutar (attention with short convolutions in
+    a window, the same experts) and Vevapel (norms around every sublayer, a repeated run of layers), and a Llama, each of
+    equal layer runs, width, feed-forward size, heads of 128 and vocabulary, as `lufazen_figures`; bounds for the kernels
+    that this design runs."""
+    def bounds(dtype, heads, width, ff):
+        e = ELT[dtype]
+        T, ctx, B, win = PREFILL_TOKENS, PROMPT_LEN, 8, 512
+        kv = max(1, heads // 4)
+        cols = (heads + 2 * kv) * 128
+        return {
+            "window attention prefill (flops of scores and values inside the window)":
+                round(2.0 * heads * T * min(win, T / 2) * 2 * 128 / (PEAK_TFLOPS[dtype] * 1e12) * 1e6, 1),
+            "window attention decode b8 (the cached keys and values of the window once)":
+                round(B * min(ctx, win) * 2 * kv * 128 * e / (HBM_GBS * 1e9) * 1e6, 2),
+            "convolution, rotation and cache write prefill (the float32 product read, queries, keys and values written)":
+                round(T * cols * (4 + e) / (HBM_GBS * 1e9) * 1e6, 1),
+            "the norm behind a sublayer, sum and next norm prefill (two float32 rows read, one and its norm written)":
+                round(T * width * (12 + e) / (HBM_GBS * 1e9) * 1e6, 1),
+            "dense feed-forward decode b8 (its weights once)": round(2 * width * ff * e / (HBM_GBS * 1e9) * 1e6, 2),
+            "dense feed-forward prefill (flops)": round(2.0 * T * 2 * width * ff / (PEAK_TFLOPS[dtype] * 1e12) * 1e6, 1),
+            "experts decode b8 (the weights of all 16 experts once)":
+                round(16 * 3 * width * (ff // 8) * e / (HBM_GBS * 1e9) * 1e6, 2),
+            "experts prefill (flops of four experts a token)":
+                round(2.0 * T * 4 * 3 * width * (ff // 8) / (PEAK_TFLOPS[dtype] * 1e12) * 1e6, 1),
+        }
+    return design_beside_llama(args, "nililix", nililix_config, bounds,
+                               beside=(("mogutar", mogutar_config), ("vevapel", vevapel_config)))
+
+
 def design_beside_llama(args, design, config_of, bounds_of, beside=()):
     """`beside`: (name, config function) of further designs of the tree to measure at the same sizes."""
     import torch
@@ -1020,6 +1066,9 @@ def run(args):
         return
     if args.only == "mogutar":
         print(json.dumps({"mogutar_beside_fofapel_and_llama": mogutar_figures(args)}), flush=True)
+        return
+    if args.only == "nililix":
+        print(json.dumps({"nililix_beside_mogutar_vevapel_and_llama": nililix_figures(args)}), flush=True)
         return
     if args.only == "attention":
         print(json.dumps({"decode_attention": attention_sweep()}), flush=True)
@@ -1097,7 +1146,7 @@ def main():
     ap.add_argument("--only", default="all",
                     choices=["all", "headline", "decode", "prefill", "fp32", "kernels", "peaks", "llama3_8b", "llama3_8b_prefill", "llama2_13b", "host",
                              "attention", "long_context", "decode_shapes", "lufazen", "fofapel", "gesutar", "vevapel",
-                             "mogutar"],
+                             "mogutar", "nililix"],
                     help="all: everything in one line; headline: the bfloat16 TinyLlama figures only; decode / prefill: "
                          "one of them (profiling); fp32: the float32 figures as the headline; kernels: decode with the time of "
                          "a step by kernel (torch's profiler); peaks / llama3_8b / "
@@ -1107,7 +1156,8 @@ def main():
                          "lufazen: prefill and decode of the Lufazen design at two sizes beside a Llama of equal size, by kernel; "
                          "fofapel, gesutar: the same for the Fofapel and the Gesutar design; "
                          "vevapel: the Vevapel design beside Lufazen and a Llama of equal size; "
-                         "mogutar: the Mogutar design beside Fofapel and a Llama of equal size")
+                         "mogutar: the Mogutar design beside Fofapel and a Llama of equal size; "
+                         "nililix: the Nililix design beside Mogutar, Vevapel and a Llama of equal size")
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         if int(os.environ.get("RANK", "0")) == 0:
