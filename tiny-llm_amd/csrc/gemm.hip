@@ -33,6 +33,17 @@ constexpr int F_KBLOCK = 256;     // the k block of the order of addition
 constexpr int F_BK = 16, F_THREADS = 256;
 constexpr int F_LD = F_BK + 4;    // LDS row stride in floats (80 bytes: 16-byte aligned rows)
 
+// What a bfloat16 product may apply to its float32 sums before they are rounded (a run-time choice, the same for the whole
+// launch; epilogue 2 of the entry points): the square of max(v, 0).
+constexpr int kActNone = 0, kActRelu2 = 2;
+__device__ __forceinline__ float act_value(float v, int act) {
+  if (act == kActRelu2) {
+    v = fmaxf(v, 0.f);
+    v *= v;
+  }
+  return v;
+}
+
 // silu(g) * u of an interleaved gate|up pair of output columns, as the reference computes it
 // (tiny_llm/ops/cuda/silu.cu:10, arithmetic.cu:13), from the float32 accumulators.
 __device__ __forceinline__ float swiglu_pair(float g, float u) { return g / (1.f + expf(-g)) * u; }
@@ -462,6 +473,7 @@ struct TileNorm {
   const float* row_scale = nullptr;
   const void* emit_w = nullptr;
   int emit_w_is_f32 = 0;
+  int act = kActNone;                 // bfloat16 output: applied before rounding
   bf16_t* emit_operand = nullptr;
   int64_t emit_ld = 0;                // row stride of the operand
   float* emit_sumsq = nullptr;
@@ -476,7 +488,7 @@ struct TileNorm {
   const int32_t* tile_group = nullptr;
   int64_t group_stride = 0;
   TileNorm() = default;
-  TileNorm(const float* rs) : row_scale(rs) {}
+  TileNorm(const float* rs, int act_ = kActNone) : row_scale(rs), act(act_) {}
 };
 
 template <int BM, int BN, int WM, int WN>
@@ -745,6 +757,10 @@ __global__ __launch_bounds__(WM * WN * TL_WAVE) void gemm_bf16_kernel(const bf16
             }
           }
         } else {
+          if (nm.act != kActNone) {     // uniform
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = act_value(v[e], nm.act);
+          }
           bf16x4 sv = {(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
           *(bf16x4*)((bf16_t*)out + o) = sv;
         }
@@ -752,6 +768,7 @@ __global__ __launch_bounds__(WM * WN * TL_WAVE) void gemm_bf16_kernel(const bf16
         for (int e = 0; e < 4 && n + e < N; ++e) {
           float x = v[e];
           if (residual) x += residual[o + e];
+          if constexpr (sizeof(TO) == 2) x = act_value(x, nm.act);
           out[o + e] = from_f32<TO>(x);
         }
       }
@@ -1047,6 +1064,7 @@ struct ReduceArgs {
   int emit_w_is_f32;
   bf16_t* emit_operand;
   float* emit_sumsq;
+  int act = kActNone;       // bfloat16 output: applied before rounding
 };
 
 template <typename TO, bool SWIGLU>
@@ -1106,7 +1124,8 @@ __global__ __launch_bounds__(R_THREADS) void splitk_reduce_kernel(const ReduceAr
         out[(int64_t)m * p.ldo + n / 2 + 1] = from_f32<TO>(swiglu_pair_fast(v[2] * scale, v[3] * scale));
     } else {
       for (int e = 0; e < 4 && n + e < N; ++e) {
-        const float x = v[e] * scale + res[e];
+        float x = v[e] * scale + res[e];
+        if constexpr (sizeof(TO) == 2) x = act_value(x, p.act);
         out[(int64_t)m * p.ldo + n + e] = from_f32<TO>(x);
         if (p.emit_operand) {
           p.emit_operand[(int64_t)m * N + n + e] = (bf16_t)(wn[e] * x);
@@ -1204,6 +1223,7 @@ struct SkinnyArgs {
   // The columns a workgroup owns, even, at most 16 a column tile (0: all of them).  Fewer make one
   // balanced round of workgroups out of a product whose column tiles do not divide by 256.
   int cols_wg = 0;
+  int act = kActNone;       // bfloat16 output: applied before rounding
 };
 
 // One 8-wide k chunk of an activation row, as loaded (Raw) and as an MFMA operand.  With the norm
@@ -1508,6 +1528,7 @@ __global__ __launch_bounds__(S_THREADS) void gemm_skinny_bf16_kernel(const Skinn
         if constexpr (HALF) v += part[wv * TILES + tile][nn + 8][m_local + 8];
       }
       v = v * scale + res_v[j];
+      if constexpr (sizeof(TO) == 2) v = act_value(v, p.act);
       if (valid) out[(int64_t)m * p.ldo + n] = from_f32<TO>(v);
       if constexpr (sizeof(TO) == 4) {
         if (p.emit_operand) {             // uniform: the lanes of a row group stay together
@@ -1764,16 +1785,19 @@ int tl_norm_prescale_f32(const float* x, const float* norm_w, const int32_t* row
 // epilogue 0: (+ residual[m, n]), out is [M, N].
 // epilogue 1: SiLU-gate of interleaved columns, out[m, j] = silu(c[m, 2j]) * c[m, 2j+1], out is
 //             [M, N/2] of the input's type; N must be even; no residual.
+// epilogue 2 (bfloat16 in and out): out[m, n] = max(c[m, n], 0)^2; no residual.
 // tile (bfloat16, M > 64): 0 lets the size decide; 1..4 force 256x256, 256x128, 128x128, 64x128.
 int tl_linear_tile(const void* a, const void* w, void* out, const float* residual, const float* row_scale, int M,
                    int N, int K, int64_t lda, int64_t ldo, int dtype, int out_dtype, int epilogue, int tile,
                    hipStream_t stream) {
   if (M <= 0) return TL_OK;
   const bool swiglu = epilogue == 1;
-  if (N <= 0 || K <= 0 || lda < K || ldo < (swiglu ? N / 2 : N) || epilogue < 0 || epilogue > 1 || tile < 0 ||
+  if (N <= 0 || K <= 0 || lda < K || ldo < (swiglu ? N / 2 : N) || epilogue < 0 || epilogue > 2 || tile < 0 ||
       tile > 4)
     return TL_ERR_ARG;
   if (swiglu && ((N & 1) || residual || out_dtype != dtype)) return TL_ERR_ARG;
+  const int act = epilogue == 2 ? kActRelu2 : kActNone;
+  if (act != kActNone && (dtype != 1 || out_dtype != 1 || residual)) return TL_ERR_ARG;
   if (dtype == 0) {
     if (out_dtype != 0) return TL_ERR_ARG;
     const bool vec = K % 4 == 0 && lda % 4 == 0 && ((uintptr_t)a | (uintptr_t)w) % 16 == 0;
@@ -1881,6 +1905,7 @@ int tl_linear_tile(const void* a, const void* w, void* out, const float* residua
     if (out_dtype != 0 && out_dtype != 1) return TL_ERR_ARG;
     if (M <= 64) {
       SkinnyArgs p{a, (const bf16_t*)w, out, residual, nullptr, nullptr, row_scale, 0.f, 0, M, N, K, lda, ldo};
+      p.act = act;
       const int rc = launch_skinny_out<PRO_NONE>(p, out_dtype, swiglu, stream);
       if (rc != TL_OK) return rc;
     } else {
@@ -1893,7 +1918,7 @@ int tl_linear_tile(const void* a, const void* w, void* out, const float* residua
                                                 M, N, K, lda, ldo, tile, 0, stream);
       else
         rc = launch_gemm_bf16_any<bf16_t, false>((const bf16_t*)a, (const bf16_t*)w, (bf16_t*)out, residual,
-                                                 row_scale, M, N, K, lda, ldo, tile, 0, stream);
+                                                 TileNorm(row_scale, act), M, N, K, lda, ldo, tile, 0, stream);
       if (rc != TL_OK) return rc;
     }
   } else {
@@ -2037,9 +2062,11 @@ int tl_linear_splitk(const void* a, const void* w, void* out, const float* resid
                      int64_t ldo, int out_dtype, int epilogue, float* workspace, hipStream_t stream) {
   const bool swiglu = epilogue == 1;
   if (M <= 0 || N <= 0 || K <= 0 || K % 8 || lda % 8 || lda < K || ldo < (swiglu ? N / 2 : N) || epilogue < 0 ||
-      epilogue > 1 || (out_dtype != 0 && out_dtype != 1) || !workspace)
+      epilogue > 2 || (out_dtype != 0 && out_dtype != 1) || !workspace)
     return TL_ERR_ARG;
   if (swiglu && ((N & 1) || residual || out_dtype != 1)) return TL_ERR_ARG;
+  const int act = epilogue == 2 ? kActRelu2 : kActNone;
+  if (act != kActNone && (out_dtype != 1 || residual)) return TL_ERR_ARG;
   if (in_sumsq && (in_parts <= 0 || in_width <= 0)) return TL_ERR_ARG;
   const bool emit = emit_operand != nullptr;
   if (emit && (!emit_w || !emit_sumsq || swiglu || out_dtype != 0 || (emit_w_dtype != 0 && emit_w_dtype != 1)))
@@ -2066,7 +2093,7 @@ int tl_linear_splitk(const void* a, const void* w, void* out, const float* resid
   }
   if (rc != TL_OK) return rc;
   ReduceArgs p{workspace, splits, M, N, out, ldo, residual, row_scale, in_sumsq, in_parts, in_width, in_eps, emit_w,
-               emit_w_dtype == 0 ? 1 : 0, (bf16_t*)emit_operand, emit_sumsq};
+               emit_w_dtype == 0 ? 1 : 0, (bf16_t*)emit_operand, emit_sumsq, act};
   if (M > 65535) return TL_ERR_ARG;
   dim3 g(M, (N + R_CHUNK - 1) / R_CHUNK), b(R_THREADS);
   if (swiglu)

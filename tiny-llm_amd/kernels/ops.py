@@ -227,7 +227,7 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, residual: Option
     """out = a @ w.T (+ residual).  a [M, K], w [N, K] share an element type; out [M, N] is that
     type or float32; residual float32 with out's strides.  epilogue="swiglu": the N columns are
     interleaved (gate_j, up_j) pairs and out [M, N/2] = silu(gate) * up, computed from the float32
-    accumulators.  row_scale [M] (float32) multiplies the rows of the product first.
+    accumulators; epilogue="relu2" (bfloat16 in and out, no residual): out = max(., 0)^2 likewise.  row_scale [M] (float32) multiplies the rows of the product first.
     tile: 0 lets the sizes choose the tile of the bfloat16 product for more than 64 rows; 1 to 4
     force 256x256, 256x128, 128x128, 64x128 (tests and tuning)."""
     _dev(a, w, out, residual, row_scale)
@@ -235,12 +235,15 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, residual: Option
     _rows_2d(out, "linear output")
     M, K = a.shape
     N = w.shape[0]
-    swiglu = _epilogue(epilogue)
+    code = EPILOGUES["relu2"] if epilogue == "relu2" else _epilogue(epilogue)
+    swiglu = code == EPILOGUES["swiglu"]
     if not (w.dim() == 2 and w.is_contiguous() and w.shape[1] == K):
         _fail(f"weight must be contiguous [N, {K}]")
     if not (a.dtype == w.dtype):
         _fail("input and weight must share an element type")
     dt, odt = _dt(a), _dt(out)
+    if epilogue == "relu2" and not (dt == odt == 1 and residual is None):
+        _fail("the squared-relu epilogue takes and leaves bfloat16, without a residual")
     if swiglu:
         if not (N % 2 == 0 and tuple(out.shape) == (M, N // 2) and odt == dt and residual is None):
             _fail(f"the SiLU-gate epilogue writes [{M}, {N // 2}] of the input's type and takes no residual")
@@ -266,11 +269,14 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, residual: Option
     if dt == 1 and tile == 0 and M > 16:
         splits = split_k(M, N, K)
         if splits > 1:
-            return _linear_split(a, w, out, residual, swiglu, row_scale, None, 0, 0.0, 0, None, splits)
+            return _linear_split(a, w, out, residual, code, row_scale, None, 0, 0.0, 0, None, splits)
     _check(_lib().tl_linear_tile(_ptr(a, al), _ptr(w, al), _ptr(out, ao), _ptr(residual, ao), _ptr(row_scale),
                                  c_int(M), c_int(N), c_int(K), c_int64(a.stride(0)), c_int64(out.stride(0)), c_int(dt),
-                                 c_int(odt), c_int(swiglu), c_int(tile), _stream()), "linear")
+                                 c_int(odt), c_int(code), c_int(tile), _stream()), "linear")
     return out
+
+
+EPILOGUES = {None: 0, "swiglu": 1, "relu2": 2}      # what `linear` does to its sums, by the number the kernels take
 
 
 def _epilogue(name: Optional[str]) -> int:

@@ -140,9 +140,9 @@ class GeluGLU(FeedForward):
 
 
 class ActMLP(FeedForward):
-    """down(act(up(h))): a feed-forward without a gate.  act "relu2" is the square of max(., 0).  The up
-    product leaves float32 and the activation rounds once to the engine's element type for the down
-    product.  `names`: the tensors' names below the prefix, (up, down).  With `residual=None` the result
+    """down(act(up(h))): a feed-forward without a gate.  act "relu2" is the square of max(., 0).  The activation is
+    applied to the up product's float32 sums, in that product's epilogue (bfloat16) or by a kernel of its own, and the
+    result is rounded once to the engine's element type for the down product.  `names`: the tensors' names below the prefix, (up, down).  With `residual=None` the result
     is returned by itself in float32."""
     graph_safe = True
 
@@ -172,10 +172,13 @@ class ActMLP(FeedForward):
 
     def forward(self, h, ctx, residual):
         T, dev = h.shape[0], h.device
-        u = ops.scratch("ffn_up", (T, self.intermediate_size), torch.float32, dev)
-        ops.linear(h, self.w_up, u)
         z = ops.scratch("ffn_gated", (T, self.intermediate_size), self.dtype, dev)
-        ops.activate_rows(u, z, self.activation)
+        if self.dtype == torch.bfloat16 and self.activation in ops.EPILOGUES:
+            ops.linear(h, self.w_up, z, epilogue=self.activation)
+        else:
+            u = ops.scratch("ffn_up", (T, self.intermediate_size), torch.float32, dev)
+            ops.linear(h, self.w_up, u)
+            ops.activate_rows(u, z, self.activation)
         if residual is None:
             return ops.linear(z, self.w_down, ops.scratch("sublayer_out", (T, self.hidden_size), torch.float32, dev))
         return ops.linear(z, self.w_down, residual, residual)
