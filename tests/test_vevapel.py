@@ -39,7 +39,7 @@ def test_reader_takes_every_size_from_the_configuration():
 
 
 def test_plan_of_a_repeated_run():
-    """Layers start .. stop - 1 run `times` times in a row; every run is a plan entry of its own (caches and
+    """The repeated layers come `times` times over; every run is a plan entry of its own (caches and
     states of its own), and the first run of every pass is entered through the stream part."""
     _, spec, dec = _decoder(MIX_A)
     assert [e.layer for e in spec.plan] == [0, 1, 2, 3, 1, 2, 3, 1, 2, 3, 4, 5]

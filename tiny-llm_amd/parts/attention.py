@@ -273,7 +273,7 @@ class GatedAttention(Attention):
                                                                                         `qk_norm="whole"`
         q, k rotated on the first rotary_dim dims (`position`, either pairing); `qk_norm="unit"`: each head by itself
         q, k and v, each channel by itself, through a causal convolution of `conv_taps` taps behind the biases, ahead of
-        everything else (y_t = sum_j w_j u_(t - taps + 1 + j), zeros ahead of the request's first token; its last taps - 1
+        everything else (y[t] = sum over i < taps of w[taps - 1 - i] u[t - i], zeros ahead of the request's first token; its last taps - 1
         inputs are per-request state)
         q (and k) divided by the root mean square over each head, times a weight per dim that the heads share, ahead of
         the rotation                                                                    `qk_norm="head"`
